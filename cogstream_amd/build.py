@@ -18,7 +18,10 @@ OBJ = HERE / "csrc" / "build"
 LIB = HERE / "libcogs_hip.so"
 HIPCC = os.environ.get("HIPCC", "/opt/rocm/bin/hipcc")
 ARCH = "gfx950"
-FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Wall", "-Wno-unused-function"]
+# no packed fp32 arithmetic (v_pk_add / mul / fma_f32): some of its forms have given wrong results on these boards, and -O3
+# forms them from ordinary float code. (hipcc's host pass warns that it does not know the target feature; that is harmless.)
+NO_PACKED_FP32 = ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+FLAGS = ["-O3", "-std=c++17", "-fPIC", f"--offload-arch={ARCH}", "-Wall", "-Wno-unused-function"] + NO_PACKED_FP32
 # per-source additions. attn_vit.hip: its row maxima run on MFMA results, which hipcc otherwise canonicalises (v_max x, x)
 # in front of every v_max3 chain -- four extra vector instructions per 32-key block on the port that bounds the kernel;
 # scores are finite or -inf (masked), never NaN, and the kernel's own NaN-sensitive test (`!(d > -inf)`) keeps its
@@ -42,7 +45,7 @@ _VMEM = re.compile(r"^\s*(global_load|global_store|buffer_load|buffer_store|flat
 def epi_pair_vmem_ops(epi: int) -> int:
     """csrc/gemm_epilogue.h::epi_pair_vmem_ops<EPI>()"""
     if epi & EPI_SWIGLU:
-        return 8
+        return 8 + (4 if epi & EPI_BIAS else 0)
     return 16 + (4 if epi & EPI_BIAS else 0) + (16 if epi & EPI_RES else 0) + \
         ((8 if epi & EPI_ROPE_LUT else 32) if epi & EPI_ROPE else 0) + (8 if epi & EPI_LNFOLD else 0) + \
         (8 if epi & EPI_ROWSTAT else 0)
@@ -147,7 +150,7 @@ def build(force: bool = False, verbose: bool = False) -> Path:
         return r.stderr
 
     if jobs:
-        with ThreadPoolExecutor(max_workers=min(4, len(jobs))) as ex:
+        with ThreadPoolExecutor(max_workers=min(8, len(jobs))) as ex:
             for warn in ex.map(cc, jobs):
                 if warn and verbose:
                     print(warn)
