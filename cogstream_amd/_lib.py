@@ -116,6 +116,27 @@ class KV(C.Structure):
     _fields_ = [("k", c_void_p), ("v", c_void_p), ("max_len", c_int), ("len", c_int)]
 
 
+class LatentMixer(C.Structure):
+    _fields_ = [("heads", c_int), ("dim", c_int), ("rot_dim", c_int), ("vdim", c_int), ("q_rank", c_int), ("kv_rank", c_int),
+                ("kv_from", c_int), ("gated", c_int), ("scale", c_float), ("rot_mag", c_float), ("rot_freq", C.POINTER(C.c_double)),
+                ("in_w", c_void_p), ("q_norm", c_void_p), ("kv_norm", c_void_p), ("q_w", c_void_p), ("kv_w", c_void_p),
+                ("k_abs", c_void_p), ("sink", c_void_p), ("o_w", c_void_p)]
+
+
+class GatedMlp(C.Structure):
+    _fields_ = [("ff", c_int), ("gu_w", c_void_p), ("gu_b", c_void_p), ("down_w", c_void_p), ("down_b", c_void_p)]
+
+
+class DecoderLayer(C.Structure):
+    _fields_ = [("norm1", c_void_p), ("norm1b", c_void_p), ("norm2", c_void_p), ("norm2b", c_void_p),
+                ("mixer", LatentMixer), ("mlp", GatedMlp)]
+
+
+class DecoderWeights(C.Structure):
+    _fields_ = [("dtype", c_int), ("width", c_int), ("vocab", c_int), ("layers", c_int), ("eps", c_float),
+                ("final_norm", c_void_p), ("head", c_void_p), ("layer", C.POINTER(DecoderLayer))]
+
+
 # every symbol include/cogs.h declares: name -> (restype, argtypes)
 SIGNATURES = {
     "cogs_status_string": (C.c_char_p, [c_int]),
@@ -179,6 +200,11 @@ SIGNATURES = {
     "cogs_llm_forward_segments": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int, c_void_p, c_void_p, c_size_t]),
     "cogs_llm_forward": (c_int, [c_void_p, c_void_p, c_void_p, c_int, C.POINTER(KV), c_void_p, c_void_p, c_void_p,
                                  c_void_p, c_size_t]),
+    "cogs_decoder_load": (c_int, [c_void_p, C.POINTER(DecoderWeights)]),
+    "cogs_decoder_cache_width": (c_int, [c_void_p, C.POINTER(c_int64)]),
+    "cogs_decoder_workspace_bytes": (c_int, [c_void_p, c_int, c_int, c_int64, c_int, C.POINTER(c_size_t)]),
+    "cogs_decoder_forward": (c_int, [c_void_p, c_void_p, c_void_p, C.POINTER(C.POINTER(KV)), C.POINTER(C.c_int32), c_int,
+                                     C.POINTER(C.c_int32), c_int, c_void_p, c_void_p, c_void_p, c_size_t]),
 }
 
 for _name, (_res, _args) in SIGNATURES.items():

@@ -9,7 +9,9 @@ the way `trust_remote_code` does it: the checkpoint directory's own `auto_map` n
     model.load_adapter(adapter_2, adapter_name="language_module")
     model.to(local_rank)
 
-runs unchanged after `from cogstream_amd.auto import AutoModelForCausalLM, AutoProcessor, PeftModel`."""
+runs unchanged after `from cogstream_amd.auto import AutoModelForCausalLM, AutoProcessor, PeftModel`.
+A config.json without an auto_map but with an "architecture" (or HF's "architectures") this package knows resolves through
+ARCHITECTURES."""
 from __future__ import annotations
 
 import importlib
@@ -17,6 +19,11 @@ import json
 import os
 
 _DEFAULT_MODEL = "cogreasoner_chat.Videollama3Qwen2ForCausalLM"
+# architecture name -> module.class
+ARCHITECTURES = {
+    "Videollama3Qwen2ForCausalLM": _DEFAULT_MODEL,
+    "Pabalix": "pabalix.PabalixForCausalLM",
+}
 _DEFAULT_PROCESSOR = "processing_cogreasoner.Videollama3Qwen2Processor"
 
 
@@ -25,7 +32,13 @@ def _resolve(path: str, json_name: str, key: str, default: str):
     p = os.path.join(path, json_name)
     if os.path.exists(p):
         with open(p, encoding="utf-8") as f:
-            target = (json.load(f).get("auto_map") or {}).get(key, default)
+            c = json.load(f)
+        if key == "AutoModelForCausalLM":
+            names = [c["architecture"]] if "architecture" in c else list(c.get("architectures") or [])
+            if "architecture" in c and c["architecture"] not in ARCHITECTURES:
+                raise ValueError(f"{p}: architecture {c['architecture']!r} (known: {', '.join(ARCHITECTURES)})")
+            default = next((ARCHITECTURES[n] for n in names if n in ARCHITECTURES), default)
+        target = (c.get("auto_map") or {}).get(key, default)
     module, _, cls = target.rpartition(".")
     try:
         mod = importlib.import_module(f"{__package__}.{module}")

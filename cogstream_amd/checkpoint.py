@@ -22,7 +22,7 @@ from typing import Dict, Iterable, List, Optional, Tuple
 
 import torch
 
-from .weights import LlmConfig, VisionConfig
+from .weights import DecoderConfig, LlmConfig, VisionConfig, decoder_tensors
 
 INDEX = "model.safetensors.index.json"
 SINGLE = "model.safetensors"
@@ -35,10 +35,21 @@ def _read_json(path: str, name: str, required: bool = True) -> dict:
     p = os.path.join(path, name)
     if not os.path.exists(p):
         if required:
-            raise FileNotFoundError(f"{p}: not a CogReasoner checkpoint directory (no {name})")
+            raise FileNotFoundError(f"{p}: not a checkpoint directory (no {name})")
         return {}
     with open(p, encoding="utf-8") as f:
         return json.load(f)
+
+
+def read_config(path: str) -> dict:
+    return _read_json(path, "config.json")
+
+
+def load_generation(path: str) -> dict:
+    """the sampling defaults of generation_config.json ({} without the file)"""
+    gen = _read_json(path, "generation_config.json", required=False)
+    return {k: v for k, v in gen.items() if k in ("do_sample", "temperature", "top_k", "top_p", "repetition_penalty",
+                                                  "eos_token_id", "pad_token_id", "bos_token_id")}
 
 
 def load_configs(path: str) -> Dict[str, object]:
@@ -62,9 +73,7 @@ def load_configs(path: str) -> Dict[str, object]:
                     rms_norm_eps=c.get("rms_norm_eps", 1e-6), rope_theta=c.get("rope_theta", 1e6),
                     image_token_index=c.get("image_token_index", 151665),
                     eos_token_id=eos[0] if isinstance(eos, (list, tuple)) else eos)
-    gen = _read_json(path, "generation_config.json", required=False)
-    gen = {k: v for k, v in gen.items() if k in ("do_sample", "temperature", "top_k", "top_p", "repetition_penalty",
-                                                 "eos_token_id", "pad_token_id", "bos_token_id")}
+    gen = load_generation(path)
     pre = _read_json(path, "preprocessor_config.json", required=False)
     prc = _read_json(path, "processor_config.json", required=False)
     processor = {"max_tokens": pre.get("max_tokens", 16384), "min_tokens": pre.get("min_tokens", 16),
@@ -217,6 +226,27 @@ def state_views(ckpt: Checkpoint, tie_word_embeddings: bool = False):
     alias = {"lm_head.weight": LLM_PREFIX + "embed_tokens.weight"} if tie_word_embeddings and "lm_head.weight" not in ckpt.weight_map else None
     return (StateView(ckpt, VIT_PREFIX), StateView(ckpt, PROJ_PREFIX),
             StateView(ckpt, LLM_PREFIX, top_level=("lm_head.weight",), alias=alias, exclude=(VIT_PREFIX, PROJ_PREFIX)))
+
+
+def open_decoder(path: str, cfg: DecoderConfig, device):
+    """-> (state mapping for weights.PackedDecoder, the reader behind it): the tensors of a decoder described layer by layer,
+    by the names and shapes its configuration implies"""
+    reader = Checkpoint(path, device=device)
+    want = decoder_tensors(cfg)
+    lacking = sorted(set(want) - set(reader.weight_map))
+    if lacking:
+        raise RuntimeError(f"{path}: checkpoint lacks {len(lacking)} tensors its config.json implies, e.g. {lacking[:4]}")
+    reader.check_shapes(want)
+    return StateView(reader, ""), reader
+
+
+def save_decoder(path: str, config: dict, state: Dict[str, torch.Tensor], dtype=torch.bfloat16) -> None:
+    """config.json + model.safetensors of a decoder described layer by layer"""
+    from safetensors.torch import save_file
+    os.makedirs(path, exist_ok=True)
+    save_file({k: v.detach().to("cpu", dtype).contiguous() for k, v in state.items()}, os.path.join(path, SINGLE))
+    with open(os.path.join(path, "config.json"), "w") as f:
+        json.dump(config, f, indent=1)
 
 
 def load_tokenizer(path: str):

@@ -48,6 +48,10 @@
     /* ---- encoder / LLM drivers (csrc/capi.hip), k-means ---- */                                                          \
     X(vit_split_max, 1099511627776LL, "clips above this many patches are encoded on one stream")                           \
     X(llm_split_keys, 0, "> 0: keys per split of the decode attention (0: chosen from the context)")                        \
+    X(mla_rowwise, 0, "1: latent attention always through the row-wise kernel")                                            \
+    X(mla_absorb, 1, "0: steps of one token per sequence also expand keys and values instead of absorbing W_uk / W_uv")     \
+    X(mla_split_keys, 0, "> 0: keys per split of the latent decode attention (0: chosen from the batch and the context)")   \
+    X(gemm_skinny, 1, "0: the decoder's few-row products through the general GEMM")                                         \
     X(km_row_groups, 0, "> 0: row groups of the k-means distance pass (0: sized to fill the chip)")
 
 struct CogsDebug {
@@ -55,7 +59,7 @@ struct CogsDebug {
     COGS_DEBUG_SWITCHES(COGS_DBG_FIELD)
 #undef COGS_DBG_FIELD
     // read-only reports (cogs_debug_get): what the last cogs_gemm of this process dispatched to
-    // 0 none yet, 1 128x128, 2 256x128 ring, 3 K-tile ping-pong, 4 whole-line ping-pong, 5 ping-pong + ring (split), 6 GEMV
+    // 0 none yet, 1 128x128, 2 256x128 ring, 3 K-tile ping-pong, 4 whole-line ping-pong, 5 ping-pong + ring (split), 6 GEMV, 7 few-row GEMM
     std::atomic<long long> gemm_last_body{0};
     // ... and the last cogs_attention: 1 general MFMA kernel, 2 ViT unpipelined, 3 ViT pipelined (row-major K/V), 4 single-token
     // decode (+ combine), 5 prompt LDS-DMA kernel, 7 row-wise fp32 kernel, 8 ViT pipelined, head-major K/V (6 and 9 were the archived

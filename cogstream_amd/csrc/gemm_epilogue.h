@@ -766,10 +766,18 @@ __device__ __forceinline__ void epilogue_pair_fast(const EpiArgs& p, int mb, int
 // v_permlane32_swap), and lane group t ends up with the 8 consecutive output columns of n-tile t: ONE 16-byte store per lane and
 // 16-row block, 64 contiguous bytes per row, 8 store instructions per wave and tile -- and an exact count for the relaxed vmcnt
 // of the next tile's first slab. Same arithmetic per element (silu_f(gate) * up, one rounding), so the bits do not change.
+// EPI_BIAS: b[n] (interleaved like the rows) joins the accumulators first; four 8-byte loads per lane for the whole region.
+template <int EPI>
 __device__ __forceinline__ void epilogue_pair_swiglu(const EpiArgs& p, int mb, int nb, int lane, f32x4 (&acc0)[4][4],
                                                      f32x4 (&acc1)[4][4]) {
     asm volatile("s_nop 8" ::: "memory");      // region markers of the build-time vmem-count check (see epilogue_pair_fast)
     const int r = lane & 15, g4 = lane >> 4;
+    f32x4 bias_v[4];
+    if constexpr ((EPI & EPI_BIAS) != 0) {
+        const char* bbase = reinterpret_cast<const char*>(p.bias) + (long)nb * 2;
+#pragma unroll
+        for (int ni = 0; ni < 4; ++ni) bias_v[ni] = ld4_f<bf16_t>(reinterpret_cast<const bf16_t*>(bbase + (unsigned)(g4 * 8 + ni * 32)));
+    }
     char* cbase = p.C + ((long)mb * p.ldc + (nb >> 1)) * 2;
     const unsigned c_lane = ((unsigned)r * (unsigned)p.ldc + (unsigned)(8 * g4)) * 2u;
     const long c_row16 = p.ldc * 32;
@@ -778,7 +786,8 @@ __device__ __forceinline__ void epilogue_pair_swiglu(const EpiArgs& p, int mb, i
         unsigned d[4];
 #pragma unroll
         for (int ni = 0; ni < 4; ++ni) {
-            const f32x4 v = blk < 4 ? acc0[blk][ni] : acc1[blk - 4][ni];
+            f32x4 v = blk < 4 ? acc0[blk][ni] : acc1[blk - 4][ni];
+            if constexpr ((EPI & EPI_BIAS) != 0) v += bias_v[ni];
             d[ni] = pack_bf2(silu_f(v[0]) * v[1], silu_f(v[2]) * v[3]);
         }
         // 4 x 4 transpose over the lane rows {r, r+16, r+32, r+48}: row t collects n-tile t's dwords of rows 0..3 in order
@@ -794,7 +803,7 @@ __device__ __forceinline__ void epilogue_pair_swiglu(const EpiArgs& p, int mb, i
 // vector-memory instructions (loads + stores; they share the in-order vmcnt queue) one epilogue_pair_fast<EPI> issues
 template <int EPI>
 constexpr int epi_pair_vmem_ops() {
-    if ((EPI & EPI_SWIGLU) != 0) return 8;      // epilogue_pair_swiglu: one 16-byte store per 16-row block, no loads
+    if ((EPI & EPI_SWIGLU) != 0) return 8 + ((EPI & EPI_BIAS) ? 4 : 0);      // epilogue_pair_swiglu: one 16-byte store per 16-row block (+ the bias)
     return 16 + ((EPI & EPI_BIAS) ? 4 : 0) + ((EPI & EPI_RES) ? 16 : 0) +
            ((EPI & EPI_ROPE) ? ((EPI & EPI_ROPE_LUT) ? 8 : 32) : 0) + ((EPI & EPI_LNFOLD) ? 8 : 0) +
            ((EPI & EPI_ROWSTAT) ? 8 : 0);
@@ -805,10 +814,10 @@ template <typename T, int EPI>
 __device__ __forceinline__ int epilogue_wave_pair(const EpiArgs& p, int mb, int nb, int M, int N, int lane,
                                                   f32x4 (&acc0)[4][4], f32x4 (&acc1)[4][4]) {
 #ifndef COGS_EPI_NOPAIR   // (A/B builds; also the build's fallback when the vmem-count check fails)
-    if constexpr (sizeof(T) == 2 && EPI == EPI_SWIGLU) {
+    if constexpr (sizeof(T) == 2 && (EPI & ~EPI_BIAS) == EPI_SWIGLU) {
         // N / 2 output columns: the wave's 64 input columns are 32 outputs = 64 bytes per row
         if (mb + 128 <= M && nb + 64 <= N && (p.ldc & 7) == 0 && (reinterpret_cast<unsigned long>(p.C) & 15) == 0) {
-            epilogue_pair_swiglu(p, mb, nb, lane, acc0, acc1);
+            epilogue_pair_swiglu<EPI>(p, mb, nb, lane, acc0, acc1);
             return epi_pair_vmem_ops<EPI>();
         }
     }
@@ -836,7 +845,7 @@ __device__ __forceinline__ int epilogue_wave_pair(const EpiArgs& p, int mb, int 
 }
 
 inline int cogs_fill_epi(const CogsGemm& g, EpiArgs* e) {
-    if (g.act == COGS_ACT_SWIGLU && (g.bias || g.residual || g.out_f32)) return COGS_E_INVALID;
+    if (g.act == COGS_ACT_SWIGLU && (g.residual || g.out_f32)) return COGS_E_INVALID;
     if (g.rope_cos && (g.head_dim <= 0 || g.head_dim % 4 != 0 || g.rope_cols % g.head_dim != 0)) return COGS_E_INVALID;
     if (g.q_scale != 1.f && (!g.rope_cos || g.q_cols % 4 != 0 || g.q_cols > g.rope_cols)) return COGS_E_INVALID;   // rope epilogues only
     e->C = (char*)g.C; e->ldc = g.ldc;
@@ -880,6 +889,7 @@ inline int cogs_epi_mask(const CogsGemm& g) {
     switch (m) {
         case 0: case EPI_BIAS: case EPI_RES: case EPI_BIAS | EPI_RES: case EPI_BIAS | EPI_ROPE:
         case EPI_BIAS | EPI_GELU_TANH: case EPI_BIAS | EPI_GELU_ERF: case EPI_SWIGLU: case EPI_F32OUT:
+        case EPI_ROPE: case EPI_SWIGLU | EPI_BIAS:
         case EPI_BIAS | EPI_ROWSTAT: case EPI_BIAS | EPI_RES | EPI_ROWSTAT:
         case EPI_BIAS | EPI_ROPE | EPI_LNFOLD: case EPI_BIAS | EPI_GELU_TANH | EPI_LNFOLD: case EPI_BIAS | EPI_LNFOLD:
         case EPI_BIAS | EPI_ROPE | EPI_HM: case EPI_BIAS | EPI_ROPE | EPI_LNFOLD | EPI_HM:

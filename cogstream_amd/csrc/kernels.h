@@ -80,6 +80,9 @@ struct CogsAttn {
 int cogs_k_attention_vit(hipStream_t st, const struct CogsAttn& a);   // attn_vit.hip: block-diagonal, hd 72, pre-scaled Q
 int cogs_k_attention_decode(hipStream_t st, const struct CogsAttn& a, float* part_o, float* part_ml);   // attn_decode.hip: one query row, hd 128, key-split partials
 int cogs_k_attention(hipStream_t st, const CogsAttn& a);
+// few-row GEMM (gemm_skinny.hip): bf16, 2 <= M <= 64; opt-in per call site (its summation order differs from cogs_k_gemm's)
+bool cogs_k_gemm_skinny_fits(const CogsGemm& g);
+int cogs_k_gemm_skinny(hipStream_t st, const CogsGemm& g);
 long cogs_k_gemm_launch_count();   // kernels launched by cogs_k_gemm so far on this thread
 
 
@@ -158,3 +161,67 @@ size_t cogs_k_sample_ws();
 int cogs_k_sample(hipStream_t st, const float* logits, int n, float temperature, int top_k, double top_p, const float* draws, uint64_t seed,
                   uint64_t offset, int64_t* out_token, int32_t* kept_idx, float* kept_prob, int* n_kept, int kept_cap,
                   void* ws);
+
+// ---- decoder-only models described layer by layer (decoder.hip) ----
+
+// one sequence of a step; device table
+struct CogsSeq {
+    char* cache;         // its cache: cached layers back to back, layer at (offset of the layer's first column) * max_len elements
+    long max_len;        // rows per cached layer
+    int row0, len;       // its new rows are rows row0 .. row0 + len - 1 of the step
+    int pos0;            // rows already cached
+    int ctx0;            // first row of its context (pos0 + len rows) in buffers that hold every sequence's context back to back
+};
+int cogs_k_seq_rows(hipStream_t st, const CogsSeq* seqs, int nseq, int rows, int* rowseq, int* rowpos);
+
+// (cos, sin) * mag of the pairs of a head, [rows][pairs][2] at table + off * rows: pairs first .. first + n - 1 turn with freq[i]
+// radians per position, the others stand still (1, 0). Angles are reduced in fp64. One launch for `nsets` such tables.
+struct CogsRopeSet { long off; int pairs, first, n; float mag; const double* freq; };
+int cogs_k_rope_sets(hipStream_t st, float* table, const CogsRopeSet* sets_dev, int nsets, int max_pairs, const int* rowpos, int rows);
+
+// fp32 residual stream x [rows][Hp] (H of the Hp columns are real, the rest zero):
+//   init: x = embeds, else x += y (y_gamma != null: x += RMSnorm(y) * y_gamma); then, out != null, out = RMSnorm(x) * out_gamma
+// y in `dtype`, gammas fp32 [Hp] (zero padded). pick (nullable, with out): only rows pick[i] are normed, into out row i, x untouched
+struct CogsStreamNorm {
+    float* x = nullptr; const void* embeds = nullptr; const void* y = nullptr; const float* y_gamma = nullptr;
+    void* out = nullptr; const float* out_gamma = nullptr; const int* pick = nullptr;
+    int rows = 0, H = 0, Hp = 0; float eps = 0.f;
+};
+int cogs_k_stream_norm(hipStream_t st, int dtype, const CogsStreamNorm& a);
+int cogs_k_zero(hipStream_t st, void* p, size_t bytes);      // 16-byte multiples
+
+// multi-head latent attention (mla.hip)
+struct CogsMlaLatent {
+    const float* t; long ldt; int qr, qrp, kvr, kvp, dr, krc, own_kv, gate_col, heads;
+    const float* q_norm; const float* kv_norm; float eps;
+    const float* rope; int rope_pairs, rope_first;
+    void* cq; float* gate;
+    const CogsSeq* seqs; const int* rowseq; const int* rowpos; long layer_off;
+};
+int cogs_k_mla_latent(hipStream_t st, int dtype, const CogsMlaLatent& a, int rows);
+int cogs_k_mla_gather(hipStream_t st, int dtype, const CogsSeq* seqs, int nseq, int max_ctx, long layer_off, int kvw, void* out);
+struct CogsHeadGemm {      // y[b][h][n] = gate[b][h] * sum_k x[b][h][k] W[h][n][k], then `tail` columns copied from x (zero past tail_n)
+    const void* X; long ldxb; int ldxh; const void* W; void* Y; long ldyb; int ldyh; int B, heads, N, K;
+    const float* gate; int tail, tail_src, tail_n;
+};
+int cogs_k_head_gemm(hipStream_t st, int dtype, const CogsHeadGemm& a);
+struct CogsMla {
+    const void* Q; long ldq; int q_head;         // per head [dn | dr | zeros], scores in log2 units
+    const void* K; long ldk; int k_head;         // expanded keys; absorbed: ldk = ldkr = ldv = cache row, pointers from the sequence
+    const void* KR; long ldkr;
+    const void* V; long ldv; int v_head;
+    void* O; long ldo; int o_head;
+    int dn, dr, dv, heads;
+    const float* sink;                           // [heads] in log2 units, or null
+    const float* gate;                           // [rows][heads], or null
+    const CogsSeq* seqs; int nseq; const int* rowseq; int rows, max_new;
+    int absorbed; long layer_off; int kr_col;
+};
+int cogs_k_mla_attention(hipStream_t st, int dtype, const CogsMla& a);
+struct CogsMlaDecode {
+    const void* Q; long ldq; int q_head; const CogsSeq* seqs; int nseq; long layer_off; int kvw, kvp, heads, nsplit;
+    const float* sink; float* part; void* out;   // part: nseq * nsplit * heads * (kvp + 2) floats; out [nseq][heads][kvp]
+};
+bool cogs_k_mla_decode_fits(int kvw, int kvp);
+int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx);
+int cogs_k_mla_decode(hipStream_t st, const CogsMlaDecode& a);

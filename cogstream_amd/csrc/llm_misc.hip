@@ -137,7 +137,63 @@ __global__ __launch_bounds__(1024) void topk_kernel(const float* __restrict__ lo
     }
 }
 
+// sequence and position of every new row of a step
+__global__ __launch_bounds__(256) void seq_rows_kernel(const CogsSeq* __restrict__ seqs, int nseq, int rows, int* __restrict__ rowseq,
+                                                       int* __restrict__ rowpos) {
+    const int r = blockIdx.x * 256 + threadIdx.x;
+    if (r >= rows) return;
+    int lo = 0, hi = nseq;
+    while (hi - lo > 1) { const int mid = (lo + hi) >> 1; if (seqs[mid].row0 <= r) lo = mid; else hi = mid; }
+    rowseq[r] = lo;
+    rowpos[r] = seqs[lo].pos0 + r - seqs[lo].row0;
+}
+
+__global__ __launch_bounds__(256) void rope_sets_kernel(float* __restrict__ table, const CogsRopeSet* __restrict__ sets,
+                                                        const int* __restrict__ rowpos, int rows) {
+    const CogsRopeSet s = sets[blockIdx.y];
+    const long total = (long)rows * s.pairs;
+    f32x2* out = reinterpret_cast<f32x2*>(table + s.off * rows);
+    for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < total; i += (long)gridDim.x * 256) {
+        const int r = (int)(i / s.pairs), p = (int)(i % s.pairs) - s.first;
+        f32x2 cs = {1.f, 0.f};
+        if (p >= 0 && p < s.n) {
+            // the angle reaches thousands of radians: whole turns are removed in fp64, the fp32 functions see |a| <= pi
+            const double turns = (double)rowpos[r] * s.freq[p] * 0.15915494309189535;
+            const float a = (float)((turns - rint(turns)) * 6.283185307179586);
+            cs = f32x2{cosf(a) * s.mag, sinf(a) * s.mag};
+        }
+        out[i] = cs;
+    }
+}
+
+__global__ __launch_bounds__(256) void zero_kernel(u32x4* __restrict__ p, long n) {
+    for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) p[i] = u32x4{0, 0, 0, 0};
+}
+
 }  // namespace
+
+int cogs_k_seq_rows(hipStream_t st, const CogsSeq* seqs, int nseq, int rows, int* rowseq, int* rowpos) {
+    if (nseq <= 0 || rows <= 0) return COGS_E_INVALID;
+    hipLaunchKernelGGL(seq_rows_kernel, dim3((rows + 255) / 256), dim3(256), 0, st, seqs, nseq, rows, rowseq, rowpos);
+    return COGS_LAUNCH_CHECK();
+}
+
+int cogs_k_rope_sets(hipStream_t st, float* table, const CogsRopeSet* sets_dev, int nsets, int max_pairs, const int* rowpos, int rows) {
+    if (nsets <= 0 || rows <= 0 || max_pairs <= 0) return COGS_E_INVALID;
+    long g = ((long)rows * max_pairs + 255) / 256;
+    if (g > 2048) g = 2048;
+    hipLaunchKernelGGL(rope_sets_kernel, dim3((unsigned)g, nsets), dim3(256), 0, st, table, sets_dev, rowpos, rows);
+    return COGS_LAUNCH_CHECK();
+}
+
+int cogs_k_zero(hipStream_t st, void* p, size_t bytes) {
+    if (!p || bytes % 16) return COGS_E_INVALID;
+    if (!bytes) return COGS_OK;
+    long g = ((long)(bytes / 16) + 255) / 256;
+    if (g > 2048) g = 2048;
+    hipLaunchKernelGGL(zero_kernel, dim3((unsigned)g), dim3(256), 0, st, (u32x4*)p, (long)(bytes / 16));
+    return COGS_LAUNCH_CHECK();
+}
 
 int cogs_k_copy_cols(hipStream_t st, int dtype, const void* src, long ld_src, void* dst, long ld_dst, int rows, int cols) {
     if (rows <= 0 || cols <= 0) return COGS_OK;

@@ -203,7 +203,96 @@ __global__ __launch_bounds__(256) void ln_finalize_kernel(const float* __restric
     *reinterpret_cast<f32x2*>(ab + 2 * (long)r) = f32x2{rstd, (float)(-(double)rstd * mean)};
 }
 
+// fp32 residual stream around a sublayer (kernels.h, CogsStreamNorm): one 256-thread workgroup per row, the row in registers
+// (C chunks of four columns per thread). Norms entirely in fp32, one rounding of the normed row.
+template <typename T, int C>
+__global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
+    __shared__ float red[2][4];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const long row = p.pick ? p.pick[blockIdx.x] : blockIdx.x;
+    float* x = p.x + row * p.Hp;
+    auto row_rstd = [&](float ss, int which) {
+        ss = wave_sum(ss);
+        if (lane == 0) red[which][wid] = ss;
+        __syncthreads();
+        ss = (red[which][0] + red[which][1]) + (red[which][2] + red[which][3]);
+        return 1.f / sqrtf(ss / (float)p.H + p.eps);
+    };
+    f32x4 v[C];
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+        const int i = tid * 4 + 1024 * c;
+        v[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (i < p.Hp) v[c] = p.embeds ? ld4_f<T>(reinterpret_cast<const T*>(p.embeds) + row * p.Hp + i) : *reinterpret_cast<const f32x4*>(x + i);
+    }
+    if (p.y) {
+        f32x4 y[C];
+        float ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < C; ++c) {
+            const int i = tid * 4 + 1024 * c;
+            y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (i < p.Hp) y[c] = ld4_f<T>(reinterpret_cast<const T*>(p.y) + row * p.Hp + i);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ss += y[c][e] * y[c][e];
+        }
+        if (p.y_gamma) {
+            const float rs = row_rstd(ss, 0);
+#pragma unroll
+            for (int c = 0; c < C; ++c) {
+                const int i = tid * 4 + 1024 * c;
+                if (i >= p.Hp) continue;
+                const f32x4 g = *reinterpret_cast<const f32x4*>(p.y_gamma + i);
+#pragma unroll
+                for (int e = 0; e < 4; ++e) y[c][e] = y[c][e] * rs * g[e];
+            }
+        }
+#pragma unroll
+        for (int c = 0; c < C; ++c) v[c] += y[c];
+    }
+    if (p.y || p.embeds) {
+#pragma unroll
+        for (int c = 0; c < C; ++c) {
+            const int i = tid * 4 + 1024 * c;
+            if (i < p.Hp) *reinterpret_cast<f32x4*>(x + i) = v[c];
+        }
+    }
+    if (!p.out) return;
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < C; ++c)
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += v[c][e] * v[c][e];
+    const float rs = row_rstd(ss, 1);
+    T* o = reinterpret_cast<T*>(p.out) + (long)blockIdx.x * p.Hp;
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+        const int i = tid * 4 + 1024 * c;
+        if (i >= p.Hp) continue;
+        const f32x4 g = *reinterpret_cast<const f32x4*>(p.out_gamma + i);
+        st4_f<T>(o + i, f32x4{v[c][0] * rs * g[0], v[c][1] * rs * g[1], v[c][2] * rs * g[2], v[c][3] * rs * g[3]});
+    }
+}
+
+template <typename T>
+int launch_stream_norm(hipStream_t st, const CogsStreamNorm& a) {
+    const dim3 grid(a.rows), blk(256);
+    if (a.Hp <= 1024) hipLaunchKernelGGL((stream_norm_kernel<T, 1>), grid, blk, 0, st, a);
+    else if (a.Hp <= 2048) hipLaunchKernelGGL((stream_norm_kernel<T, 2>), grid, blk, 0, st, a);
+    else if (a.Hp <= 4096) hipLaunchKernelGGL((stream_norm_kernel<T, 4>), grid, blk, 0, st, a);
+    else if (a.Hp <= 8192) hipLaunchKernelGGL((stream_norm_kernel<T, 8>), grid, blk, 0, st, a);
+    else if (a.Hp <= 16384) hipLaunchKernelGGL((stream_norm_kernel<T, 16>), grid, blk, 0, st, a);
+    else return COGS_E_UNSUPPORTED;
+    return COGS_LAUNCH_CHECK();
+}
+
 }  // namespace
+
+int cogs_k_stream_norm(hipStream_t st, int dtype, const CogsStreamNorm& a) {
+    if (a.rows <= 0) return COGS_OK;
+    if (!a.x || a.Hp % 4 || a.H <= 0 || a.H > a.Hp || (a.out && !a.out_gamma) || (a.pick && (!a.out || a.y || a.embeds))) return COGS_E_INVALID;
+    return dtype == COGS_DT_BF16 ? launch_stream_norm<bf16_t>(st, a) : launch_stream_norm<float>(st, a);
+}
 
 int cogs_k_layernorm(hipStream_t st, int dtype, const void* x, void* y, const void* gamma, const void* beta,
                      int rows, int H, float eps) {

@@ -1,17 +1,21 @@
-"""Host mirror of the Qwen2 seams the reference calls (transformers, pinned 4.46.3):
+"""Language-model engines: prefill / decode steps over caller-owned caches, generation, and batches of live requests.
+
+Qwen2Engine is the host mirror of the Qwen2 seams the reference calls (transformers, pinned 4.46.3):
 self.get_model()(inputs_embeds=..., attention_mask=...) (model/cogreasoner_chat.py:312-316,322) and
-super().generate(inputs_embeds=...) (:802-807), computing through cogs_llm_forward."""
+super().generate(inputs_embeds=...) (:802-807), computing through cogs_llm_forward. DecoderEngine runs decoder-only models
+described layer by layer (weights.DecoderConfig) through cogs_decoder_forward. Both share CausalEngine's generation loop,
+PrefixKV, and the batch steps of Sequences."""
 from __future__ import annotations
 
 import ctypes as C
-from typing import Dict, List, Optional, Sequence
+from typing import Dict, Hashable, List, Optional, Sequence, Tuple
 
 import torch
 
 from . import _lib as L
 from . import ops
 from .runtime import get_handle
-from .weights import LlmConfig, PackedLlm
+from .weights import DecoderConfig, LlmConfig, PackedDecoder, PackedLlm
 
 
 class KVCache:
@@ -25,8 +29,36 @@ class KVCache:
     def len(self) -> int:
         return self.struct.len
 
+    @property
+    def max_len(self) -> int:
+        return self.struct.max_len
+
     def reset(self, length: int = 0):
         self.struct.len = length
+
+    def _blocks(self) -> List[torch.Tensor]:
+        """views [..., max_len, columns] that hold the cached rows"""
+        return [self.k, self.v]
+
+    def copy_rows_from(self, old: "KVCache", n: int):
+        for dst, src in zip(self._blocks(), old._blocks()):
+            dst[..., :n, :].copy_(src[..., :n, :])
+
+
+class LatentCache(KVCache):
+    """one sequence's rows [latent | rotated key part] of every layer that has its own (weights.PackedDecoder.cache_widths)"""
+
+    def __init__(self, widths: Sequence[int], max_len: int, dtype, device):
+        self.widths = list(widths)
+        self.k = torch.empty(sum(self.widths) * max_len, device=device, dtype=dtype)
+        self.struct = L.KV(self.k.data_ptr(), None, max_len, 0)
+
+    def _blocks(self) -> List[torch.Tensor]:
+        out, at = [], 0
+        for w in self.widths:
+            out.append(self.k[at:at + w * self.max_len].view(self.max_len, w))
+            at += w * self.max_len
+        return out
 
 
 class PrefixKV:
@@ -37,7 +69,7 @@ class PrefixKV:
     history turn dropped by the selection stage, another question) is covered by that comparison. Only rows that
     were PREFILLED are reused -- rows written by decode steps went through the GEMV kernels."""
 
-    def __init__(self, engine: "Qwen2Engine"):
+    def __init__(self, engine: "CausalEngine"):
         self.engine = engine
         self.cache: Optional[KVCache] = None
         self.rows: Optional[torch.Tensor] = None   # [n, H] embeddings whose KV rows 0..n-1 are in `cache`
@@ -46,13 +78,11 @@ class PrefixKV:
 
     def plan(self, embeds: torch.Tensor, need: int) -> int:
         """-> number of leading rows of `embeds` whose KV is already in self.cache (at most len(embeds) - 2)"""
-        if self.cache is None or self.cache.k.shape[1] < need:
+        if self.cache is None or self.cache.max_len < need:
             old = self.cache
             self.cache = self.engine.new_cache(need + need // 2)   # sessions grow: leave room for the next turns
             if old is not None and self.rows is not None:
-                n = self.rows.shape[0]
-                self.cache.k[:, :n].copy_(old.k[:, :n])
-                self.cache.v[:, :n].copy_(old.v[:, :n])
+                self.cache.copy_rows_from(old, self.rows.shape[0])
             else:
                 self.rows = None
         p = 0
@@ -72,66 +102,42 @@ class PrefixKV:
         self.rows = None
 
 
-class Qwen2Engine:
-    def __init__(self, state: Dict[str, torch.Tensor], cfg: LlmConfig, dtype=torch.bfloat16, device="cuda"):
-        self.cfg, self.dtype, self.device = cfg, dtype, torch.device(device)
-        self.handle = get_handle(self.device)
-        self.packed = PackedLlm(state, cfg, dtype, self.device)
-        self._activate()
-
-    def _activate(self):
-        self.handle.activate("llm", self, lambda: L.check(
-            L.lib.cogs_llm_load(self.handle.h, C.byref(self.packed.struct)), "cogs_llm_load"))
+class CausalEngine:
+    """what generation needs of a model: cfg.vocab_size, new_cache, embed_tokens, forward (one sequence) and forward_batch"""
+    cfg = None
+    dtype = None
+    device = None
 
     def new_cache(self, max_len: int) -> KVCache:
-        return KVCache(self.cfg, max_len, self.dtype, self.device)
+        raise NotImplementedError
 
     def embed_tokens(self, ids: torch.Tensor) -> torch.Tensor:
-        return ops.gather_rows(self.packed.embed, None, ids.reshape(-1).to(self.device, torch.int64))
+        raise NotImplementedError
 
-    def forward(self, embeds: torch.Tensor, cache: Optional[KVCache] = None, *, want_logits: bool = True,
-                want_pooled: bool = False, want_hidden: bool = False):
-        """returns dict(logits fp32 [vocab] | pooled fp32 [H] | hidden [S,H])"""
-        self._activate()
-        embeds = embeds.contiguous()
-        S = embeds.shape[0]
-        ctx = S + (cache.len if cache is not None else 0)
-        nbytes = C.c_size_t()
-        L.check(L.lib.cogs_llm_workspace_bytes(self.handle.h, S, ctx, C.byref(nbytes)), "cogs_llm_workspace_bytes")
-        ws = self.handle.workspace("llm", nbytes.value)
-        out = {}
-        logits = torch.empty(self.cfg.vocab_size, device=self.device, dtype=torch.float32) if want_logits else None
-        pooled = torch.empty(self.cfg.hidden_size, device=self.device, dtype=torch.float32) if want_pooled else None
-        hidden = torch.empty(S, self.cfg.hidden_size, device=self.device, dtype=self.dtype) if want_hidden else None
-        L.check(L.lib.cogs_llm_forward(self.handle.h, L.current_stream(), embeds.data_ptr(), S,
-                                       C.byref(cache.struct) if cache is not None else None, L.ptr(logits),
-                                       L.ptr(pooled), L.ptr(hidden), ws.data_ptr(), ws.numel()), "cogs_llm_forward")
-        if want_logits:
-            out["logits"] = logits
-        if want_pooled:
-            out["pooled"] = pooled
-        if want_hidden:
-            out["hidden"] = hidden
-        return out
+    def forward(self, embeds: torch.Tensor, cache: Optional[KVCache] = None, **want) -> Dict[str, torch.Tensor]:
+        raise NotImplementedError
 
-    def forward_segments(self, embeds: torch.Tensor, seg_lens: Sequence[int]) -> torch.Tensor:
-        """several independent sequences stored back to back -> mean of the final hidden states of each, fp32
-        [nseg, H] (cogs_llm_forward_segments): one var-len prefill instead of one forward per sequence"""
-        self._activate()
-        embeds = embeds.contiguous()
-        S = embeds.shape[0]
-        cu = [0]
-        for n in seg_lens:
-            cu.append(cu[-1] + int(n))
-        assert cu[-1] == S and all(int(n) > 0 for n in seg_lens)
-        nbytes = C.c_size_t()
-        L.check(L.lib.cogs_llm_workspace_bytes(self.handle.h, S, S, C.byref(nbytes)), "cogs_llm_workspace_bytes")
-        ws = self.handle.workspace("llm", nbytes.value)
-        out = torch.empty(len(seg_lens), self.cfg.hidden_size, device=self.device, dtype=torch.float32)
-        cua = (C.c_int32 * len(cu))(*cu)
-        L.check(L.lib.cogs_llm_forward_segments(self.handle.h, L.current_stream(), embeds.data_ptr(), S, cua, len(seg_lens),
-                                                out.data_ptr(), ws.data_ptr(), ws.numel()), "cogs_llm_forward_segments")
-        return out
+    def logits_of(self, hidden: torch.Tensor) -> torch.Tensor:
+        """final hidden states [n, hidden] -> fp32 logits [n, vocab]"""
+        raise NotImplementedError
+
+    def forward_batch(self, embeds: torch.Tensor, lens: Sequence[int], caches: Sequence[KVCache],
+                      want: Sequence[int]) -> Optional[torch.Tensor]:
+        """one step of several sequences: sequence i brings lens[i] rows of `embeds` (back to back) behind caches[i].
+        -> fp32 logits [len(want), vocab] of the rows `want` (None if empty). Here one sequence at a time; engines with a
+        batched step override it."""
+        rows: Dict[int, torch.Tensor] = {}
+        r0 = 0
+        for n, cache in zip(lens, caches):
+            mine = [w for w in want if r0 <= w < r0 + n]
+            if mine == [r0 + n - 1]:
+                rows[mine[0]] = self.forward(embeds[r0:r0 + n], cache)["logits"]
+            else:
+                hidden = self.forward(embeds[r0:r0 + n], cache, want_logits=False, want_hidden=bool(mine)).get("hidden")
+                for w in mine:
+                    rows[w] = self.logits_of(hidden[w - r0:w - r0 + 1])[0]
+            r0 += n
+        return torch.stack([rows[w] for w in want]) if len(want) else None
 
     def generate(self, embeds: torch.Tensor, *, max_new_tokens: int, eos_token_id: Sequence[int] = (),
                  do_sample: bool = False, temperature: float = 1.0, top_k: int = 0, top_p: float = 1.0,
@@ -227,8 +233,197 @@ class Qwen2Engine:
             cache.reset(min(cache.len, pos_start + stop_at - 1))
         return out
 
+    def generate_batch(self, prompts: Sequence[Sequence[int]], *, max_new_tokens: int, eos_token_id: Sequence[int] = (),
+                       do_sample: bool = False, temperature: float = 1.0, top_k: int = 0, top_p: float = 1.0,
+                       repetition_penalty: float = 1.0, seed: int = 0, max_batch: int = 64) -> List[List[int]]:
+        """new token ids of every prompt. Up to `max_batch` requests run at once: a group's prompts are one step, then every
+        step carries one token of each request that has not finished; a finished request leaves the batch and its cache with
+        it. Logits processors and samplers are generate()'s, per request (Philox offset = step, seed + request index)."""
+        out: List[List[int]] = [[] for _ in prompts]
+        eos = set(int(e) for e in eos_token_id)
+        for g0 in range(0, len(prompts), max_batch):
+            live = [i for i in range(g0, min(g0 + max_batch, len(prompts)))]
+            seqs = Sequences(self)
+            feed = {i: [int(t) for t in prompts[i]] for i in live}
+            if any(not f for f in feed.values()):
+                raise ValueError("empty prompt")
+            for step in range(max_new_tokens):
+                logits = seqs.step([(i, feed[i], [len(feed[i]) - 1]) for i in live])
+                picked = torch.empty(len(live), dtype=torch.int64, device=self.device)
+                for r, i in enumerate(live):
+                    if repetition_penalty != 1.0:
+                        prev = torch.tensor(list(prompts[i]) + out[i], dtype=torch.int64, device=self.device)
+                        ops.logits_process(logits[r], prev, repetition_penalty, None, 1.0)
+                    if do_sample:
+                        ops.sample(logits[r], top_k or 0, top_p, seed=seed + i, offset=step, temperature=temperature, out=picked[r:r + 1])
+                    else:
+                        ops.argmax(logits[r], out=picked[r:r + 1])
+                toks = picked.tolist()
+                for i, t in zip(live, toks):
+                    out[i].append(t)
+                    feed[i] = [t]
+                for i in [i for i in live if out[i][-1] in eos]:
+                    seqs.release(i)
+                live = [i for i in live if out[i][-1] not in eos]
+                if not live:
+                    break
+        return out
+
     def _draws(self, generator) -> torch.Tensor:
         """parity mode: the [vocab] Exponential(1) draws torch.multinomial(probs, 1) makes on the CPU generator
         (GenerationMixin._sample, transformers 4.46.3; the reference's CPU path draws from the global generator)"""
         q = torch.empty(self.cfg.vocab_size, dtype=torch.float32).exponential_(1, generator=generator)
         return q.to(self.device, non_blocking=True)
+
+
+class Qwen2Engine(CausalEngine):
+    def __init__(self, state: Dict[str, torch.Tensor], cfg: LlmConfig, dtype=torch.bfloat16, device="cuda"):
+        self.cfg, self.dtype, self.device = cfg, dtype, torch.device(device)
+        self.handle = get_handle(self.device)
+        self.packed = PackedLlm(state, cfg, dtype, self.device)
+        self._activate()
+
+    def _activate(self):
+        self.handle.activate("llm", self, lambda: L.check(
+            L.lib.cogs_llm_load(self.handle.h, C.byref(self.packed.struct)), "cogs_llm_load"))
+
+    def new_cache(self, max_len: int) -> KVCache:
+        return KVCache(self.cfg, max_len, self.dtype, self.device)
+
+    def embed_tokens(self, ids: torch.Tensor) -> torch.Tensor:
+        return ops.gather_rows(self.packed.embed, None, ids.reshape(-1).to(self.device, torch.int64))
+
+    def forward(self, embeds: torch.Tensor, cache: Optional[KVCache] = None, *, want_logits: bool = True,
+                want_pooled: bool = False, want_hidden: bool = False):
+        """returns dict(logits fp32 [vocab] | pooled fp32 [H] | hidden [S,H])"""
+        self._activate()
+        embeds = embeds.contiguous()
+        S = embeds.shape[0]
+        ctx = S + (cache.len if cache is not None else 0)
+        nbytes = C.c_size_t()
+        L.check(L.lib.cogs_llm_workspace_bytes(self.handle.h, S, ctx, C.byref(nbytes)), "cogs_llm_workspace_bytes")
+        ws = self.handle.workspace("llm", nbytes.value)
+        out = {}
+        logits = torch.empty(self.cfg.vocab_size, device=self.device, dtype=torch.float32) if want_logits else None
+        pooled = torch.empty(self.cfg.hidden_size, device=self.device, dtype=torch.float32) if want_pooled else None
+        hidden = torch.empty(S, self.cfg.hidden_size, device=self.device, dtype=self.dtype) if want_hidden else None
+        L.check(L.lib.cogs_llm_forward(self.handle.h, L.current_stream(), embeds.data_ptr(), S,
+                                       C.byref(cache.struct) if cache is not None else None, L.ptr(logits),
+                                       L.ptr(pooled), L.ptr(hidden), ws.data_ptr(), ws.numel()), "cogs_llm_forward")
+        if want_logits:
+            out["logits"] = logits
+        if want_pooled:
+            out["pooled"] = pooled
+        if want_hidden:
+            out["hidden"] = hidden
+        return out
+
+    def logits_of(self, hidden: torch.Tensor) -> torch.Tensor:
+        return ops.gemm(hidden.contiguous(), self.packed.lm_head, out_f32=True)
+
+    def forward_segments(self, embeds: torch.Tensor, seg_lens: Sequence[int]) -> torch.Tensor:
+        """several independent sequences stored back to back -> mean of the final hidden states of each, fp32
+        [nseg, H] (cogs_llm_forward_segments): one var-len prefill instead of one forward per sequence"""
+        self._activate()
+        embeds = embeds.contiguous()
+        S = embeds.shape[0]
+        cu = [0]
+        for n in seg_lens:
+            cu.append(cu[-1] + int(n))
+        assert cu[-1] == S and all(int(n) > 0 for n in seg_lens)
+        nbytes = C.c_size_t()
+        L.check(L.lib.cogs_llm_workspace_bytes(self.handle.h, S, S, C.byref(nbytes)), "cogs_llm_workspace_bytes")
+        ws = self.handle.workspace("llm", nbytes.value)
+        out = torch.empty(len(seg_lens), self.cfg.hidden_size, device=self.device, dtype=torch.float32)
+        cua = (C.c_int32 * len(cu))(*cu)
+        L.check(L.lib.cogs_llm_forward_segments(self.handle.h, L.current_stream(), embeds.data_ptr(), S, cua, len(seg_lens),
+                                                out.data_ptr(), ws.data_ptr(), ws.numel()), "cogs_llm_forward_segments")
+        return out
+
+
+class DecoderEngine(CausalEngine):
+    """a decoder-only model described layer by layer (weights.DecoderConfig), batched steps through cogs_decoder_forward"""
+
+    def __init__(self, state: Dict[str, torch.Tensor], cfg: DecoderConfig, dtype=torch.bfloat16, device="cuda"):
+        self.cfg, self.dtype, self.device = cfg, dtype, torch.device(device)
+        self.handle = get_handle(self.device)
+        self.packed = PackedDecoder(state, cfg, dtype, self.device)
+        self._activate()
+
+    def _activate(self):
+        self.handle.activate("decoder", self, lambda: L.check(
+            L.lib.cogs_decoder_load(self.handle.h, C.byref(self.packed.struct)), "cogs_decoder_load"))
+
+    def new_cache(self, max_len: int) -> LatentCache:
+        return LatentCache(self.packed.cache_widths, max_len, self.dtype, self.device)
+
+    def embed_tokens(self, ids: torch.Tensor) -> torch.Tensor:
+        return ops.gather_rows(self.packed.embed, None, ids.reshape(-1).to(self.device, torch.int64))
+
+    def forward_batch(self, embeds: torch.Tensor, lens: Sequence[int], caches: Sequence[KVCache], want: Sequence[int],
+                      streams: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+        """streams, when given: fp32 [layers, rows, padded width], receives the residual stream behind every layer"""
+        self._activate()
+        embeds = embeds.contiguous()
+        S, n, nw = embeds.shape[0], len(lens), len(want)
+        assert sum(lens) == S and len(caches) == n and embeds.shape[1] == self.packed.width_p and embeds.dtype == self.dtype
+        ctx = S + sum(c.len for c in caches)
+        nbytes = C.c_size_t()
+        L.check(L.lib.cogs_decoder_workspace_bytes(self.handle.h, S, n, ctx, nw, C.byref(nbytes)), "cogs_decoder_workspace_bytes")
+        ws = self.handle.workspace("decoder", nbytes.value)
+        logits = torch.empty(nw, self.packed.vocab_p, device=self.device, dtype=torch.float32) if nw else None
+        kv = (C.POINTER(L.KV) * n)(*[C.pointer(c.struct) for c in caches])
+        L.check(L.lib.cogs_decoder_forward(self.handle.h, L.current_stream(), embeds.data_ptr(), kv, (C.c_int32 * n)(*lens), n,
+                                           (C.c_int32 * max(nw, 1))(*want), nw, L.ptr(logits), L.ptr(streams), ws.data_ptr(),
+                                           ws.numel()), "cogs_decoder_forward")
+        return logits[:, :self.cfg.vocab_size] if nw else None
+
+    def forward(self, embeds: torch.Tensor, cache: Optional[KVCache] = None, *, want_logits: bool = True) -> Dict[str, torch.Tensor]:
+        """one sequence -> dict(logits fp32 [vocab]) of its last row"""
+        S = embeds.shape[0]
+        if cache is None:
+            cache = self.new_cache(S)
+        out = self.forward_batch(embeds, [S], [cache], [S - 1] if want_logits else [])
+        return {"logits": out[0]} if want_logits else {}
+
+
+class Sequences:
+    """the live requests of an engine: a cache per request id, steps that carry new tokens of any of them as one batch"""
+
+    def __init__(self, engine: CausalEngine, reserve: int = 64):
+        self.engine, self.reserve = engine, reserve
+        self.caches: Dict[Hashable, KVCache] = {}
+
+    def _cache(self, rid: Hashable, new: int) -> KVCache:
+        """the request's cache with room for `new` more rows; a full one moves to one of twice the size"""
+        old = self.caches.get(rid)
+        need = new + (old.len if old is not None else 0)
+        if old is None or old.max_len < need:
+            grown = self.engine.new_cache(max(-(-need // self.reserve) * self.reserve, 2 * old.max_len if old is not None else 0))
+            if old is not None:
+                grown.copy_rows_from(old, old.len)
+                grown.reset(old.len)
+            self.caches[rid] = grown
+        return self.caches[rid]
+
+    def step(self, entries: Sequence[Tuple[Hashable, Sequence[int], Sequence[int]]]) -> Optional[torch.Tensor]:
+        """entries (request id, its next token ids, places among them whose logits are wanted) -> fp32 logits, one row per
+        wanted place in order, or None"""
+        ids: List[int] = []
+        lens, caches, want = [], [], []
+        vocab = self.engine.cfg.vocab_size
+        if len({rid for rid, _, _ in entries}) != len(entries):
+            raise ValueError("a request appears twice in one step")
+        for rid, toks, places in entries:
+            if not toks or any(not 0 <= t < vocab for t in toks) or any(not 0 <= w < len(toks) for w in places):
+                raise ValueError(f"request {rid!r}: no tokens, a token outside the vocabulary, or a wanted place outside the step")
+            want += [len(ids) + w for w in places]
+            ids += toks
+            lens.append(len(toks))
+        for (rid, toks, _), n in zip(entries, lens):
+            caches.append(self._cache(rid, n))
+        embeds = self.engine.embed_tokens(torch.tensor(ids, dtype=torch.int64))
+        return self.engine.forward_batch(embeds, lens, caches, want)
+
+    def release(self, rid: Hashable) -> None:
+        del self.caches[rid]

@@ -10,8 +10,9 @@ torch is used here for tensor storage and the one-time reshuffles only."""
 from __future__ import annotations
 
 import ctypes as C
-from dataclasses import dataclass
-from typing import Dict, List, Optional
+import math
+from dataclasses import dataclass, field
+from typing import Dict, List, Optional, Tuple
 
 import torch
 
@@ -52,6 +53,86 @@ class LlmConfig:
     @property
     def head_dim(self) -> int:
         return self.hidden_size // self.num_attention_heads
+
+
+@dataclass
+class YarnScaling:
+    """context extension by slowing the pairs that turn rarely: pairs making more than `fast` turns over `original`
+    positions keep their frequency, pairs making fewer than `slow` are divided by `factor`, a ramp between"""
+    factor: float
+    original: float
+    fast: float
+    slow: float
+
+
+@dataclass
+class Rotation:
+    """rotary positions over `dims` dimensions: pair i is (2i, 2i+1) if interleaved, else (i, i + dims/2)"""
+    dims: int
+    base: float
+    interleaved: bool = False
+    scaling: Optional[YarnScaling] = None
+
+    def frequencies(self) -> List[float]:
+        """radians per position of every pair (float64)"""
+        n, s = self.dims, self.scaling
+        freq = [self.base ** (-2.0 * i / n) for i in range(n // 2)]
+        if s is None:
+            return freq
+        index = lambda turns: n * math.log(s.original / (2 * math.pi * turns)) / (2 * math.log(self.base))
+        lo, hi = max(math.floor(index(s.fast)), 0), min(math.ceil(index(s.slow)), n - 1)
+        ramp = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in range(n // 2)]
+        return [f / s.factor * r + f * (1.0 - r) for f, r in zip(freq, ramp)]
+
+    @property
+    def magnitude(self) -> float:
+        """factor on cos and sin"""
+        return 1.0 if self.scaling is None else 0.1 * math.log(self.scaling.factor) + 1.0
+
+    def pair_order(self) -> torch.Tensor:
+        """the packed order of the rotated rows: pairs adjacent"""
+        return torch.arange(self.dims) if self.interleaved else rope_perm(self.dims)
+
+
+@dataclass
+class LatentAttention:
+    """multi-head latent attention (include/cogs.h, cogs_latent_mixer)"""
+    heads: int
+    dim: int
+    rot_dim: int
+    vdim: int
+    q_rank: int
+    kv_rank: int
+    scale: float
+    rot: Rotation
+    kv_from: Optional[int] = None      # earlier layer whose cached latents this layer reads
+    sink: bool = False                 # a learned logit per head in the softmax sum
+    gate: bool = False                 # sigmoid gate per head on the output
+
+
+@dataclass
+class DecoderLayerConfig:
+    mixer: LatentAttention
+    ff: int = 0                        # gated-SiLU MLP width, 0 = no feed-forward sublayer
+    mlp_bias: bool = False
+    post_norm: bool = True             # norms on the sublayers' outputs
+
+
+@dataclass
+class DecoderConfig:
+    """a decoder-only model described layer by layer"""
+    width: int
+    vocab_size: int
+    eps: float
+    layers: List[DecoderLayerConfig] = field(default_factory=list)
+
+    @property
+    def hidden_size(self) -> int:
+        return self.width
+
+    @property
+    def num_hidden_layers(self) -> int:
+        return len(self.layers)
 
 
 def rope_perm(hd: int) -> torch.Tensor:
@@ -253,6 +334,131 @@ class PackedLlm:
         self.struct = w
 
 
+def _up(v: int, m: int) -> int:
+    return (v + m - 1) // m * m
+
+
+def _pad_to(x: torch.Tensor, *shape: int) -> torch.Tensor:
+    if tuple(x.shape) == shape:
+        return x.contiguous()
+    out = x.new_zeros(*shape)
+    out[tuple(slice(0, n) for n in x.shape)] = x
+    return out
+
+
+def decoder_tensors(cfg: DecoderConfig) -> Dict[str, Tuple[int, ...]]:
+    """name -> shape of every tensor of a decoder described layer by layer"""
+    W = cfg.width
+    out: Dict[str, Tuple[int, ...]] = {"embed": (cfg.vocab_size, W), "final.norm": (W,), "head": (cfg.vocab_size, W)}
+    for i, lay in enumerate(cfg.layers):
+        p, m = f"l{i}.", lay.mixer
+        out[p + "norm1"] = (W,)
+        if lay.post_norm:
+            out[p + "norm1b"] = (W,)
+        out[p + "mix.dq"], out[p + "mix.dq.norm"] = (m.q_rank, W), (m.q_rank,)
+        out[p + "mix.uq"] = (m.heads * (m.dim + m.rot_dim), m.q_rank)
+        if m.kv_from is None:
+            out[p + "mix.dkv"], out[p + "mix.dkv.norm"] = (m.kv_rank + m.rot_dim, W), (m.kv_rank,)
+        out[p + "mix.uk"], out[p + "mix.uv"] = (m.heads * m.dim, m.kv_rank), (m.heads * m.vdim, m.kv_rank)
+        if m.sink:
+            out[p + "mix.sink"] = (m.heads,)
+        if m.gate:
+            out[p + "mix.g"] = (m.heads, W)
+        out[p + "mix.o"] = (W, m.heads * m.vdim)
+        if lay.ff:
+            out[p + "norm2"] = (W,)
+            if lay.post_norm:
+                out[p + "norm2b"] = (W,)
+            for n, shape in (("gate", (lay.ff, W)), ("up", (lay.ff, W)), ("down", (W, lay.ff))):
+                out[p + "mlp." + n] = shape
+                if lay.mlp_bias:
+                    out[p + f"mlp.{n}.b"] = shape[:1]
+    return out
+
+
+class PackedDecoder:
+    """decoder_tensors -> the layouts of include/cogs.h (cogs_decoder_*): padded sizes, stacked down projections, rotary pairs
+    adjacent, gate / up rows interleaved, W_uk also transposed per head for the absorbed decode"""
+
+    def __init__(self, state: Dict[str, torch.Tensor], cfg: DecoderConfig, dtype=torch.bfloat16, device="cuda"):
+        self.cfg, self.dtype, self.device = cfg, dtype, torch.device(device)
+        self.keep: List[object] = []
+        self.width_p, self.vocab_p = _up(cfg.width, 64), _up(cfg.vocab_size, 4)
+        Wp = self.width_p
+
+        def hold(t):
+            t = t.contiguous()
+            self.keep.append(t)
+            return t
+
+        g = lambda k: state[k].to(device=self.device, dtype=dtype)
+        vec = lambda k, n: hold(_pad_to(state[k].to(device=self.device, dtype=torch.float32), n)).data_ptr()
+        self.embed = hold(_pad_to(g("embed"), cfg.vocab_size, Wp))
+        self.head = hold(_pad_to(g("head"), self.vocab_p, Wp))
+        self.layers = (L.DecoderLayer * len(cfg.layers))()
+        for i, lc in enumerate(cfg.layers):
+            p, lay, m = f"l{i}.", self.layers[i], lc.mixer
+            if m.rot.dims != m.rot_dim:
+                raise ValueError(f"layer {i}: rotation over {m.rot.dims} dimensions, rotated part of {m.rot_dim}")
+            a = p + "mix."
+            qrp, kvp, rotc, hp = _up(m.q_rank, 64), _up(m.kv_rank, 64), _up(m.rot_dim, 32), _up(m.heads, 4)
+            dn, dr, dk, dv = _up(m.dim, 8), _up(m.rot_dim, 8), _up(m.dim, 32), _up(m.vdim, 16)
+            dq = _up(dn + dr, 32)
+            order = m.rot.pair_order().to(self.device)
+            lay.norm1 = vec(p + "norm1", Wp)
+            if lc.post_norm:
+                lay.norm1b = vec(p + "norm1b", Wp)
+            x = lay.mixer
+            x.heads, x.dim, x.rot_dim, x.vdim, x.q_rank, x.kv_rank = m.heads, m.dim, m.rot_dim, m.vdim, m.q_rank, m.kv_rank
+            x.kv_from, x.gated = -1 if m.kv_from is None else m.kv_from, int(m.gate)
+            x.scale, x.rot_mag = m.scale, m.rot.magnitude
+            freq = (C.c_double * (m.rot_dim // 2))(*m.rot.frequencies())
+            self.keep.append(freq)
+            x.rot_freq = C.cast(freq, C.POINTER(C.c_double))
+            rows = [_pad_to(g(a + "dq"), qrp, Wp)]
+            x.q_norm = vec(a + "dq.norm", qrp)
+            if m.kv_from is None:
+                d = g(a + "dkv")
+                rows += [_pad_to(d[:m.kv_rank], kvp, Wp), _pad_to(d[m.kv_rank:][order], rotc, Wp)]
+                x.kv_norm = vec(a + "dkv.norm", kvp)
+            if m.gate:
+                rows.append(_pad_to(g(a + "g"), hp, Wp))
+            x.in_w = hold(torch.cat(rows, 0)).data_ptr()
+            uq = g(a + "uq").view(m.heads, m.dim + m.rot_dim, m.q_rank)
+            q = uq.new_zeros(m.heads, dq, qrp)
+            q[:, :m.dim, :m.q_rank] = uq[:, :m.dim]
+            q[:, dn:dn + m.rot_dim, :m.q_rank] = uq[:, m.dim:][:, order]
+            x.q_w = hold(q.view(m.heads * dq, qrp)).data_ptr()
+            uk = g(a + "uk").view(m.heads, m.dim, m.kv_rank)
+            uv = g(a + "uv").view(m.heads, m.vdim, m.kv_rank)
+            x.kv_w = hold(torch.cat([_pad_to(uk, m.heads, dn, kvp).view(-1, kvp), _pad_to(uv, m.heads, dv, kvp).view(-1, kvp)], 0)).data_ptr()
+            x.k_abs = hold(_pad_to(uk.transpose(1, 2), m.heads, kvp, dk)).data_ptr()
+            if m.sink:
+                x.sink = hold(state[a + "sink"].to(device=self.device, dtype=torch.float32) * math.log2(math.e)).data_ptr()
+            o = _pad_to(g(a + "o").view(cfg.width, m.heads, m.vdim), Wp, m.heads, dv).view(Wp, m.heads * dv)
+            x.o_w = hold(_pad_to(o, Wp, _up(m.heads * dv, 64))).data_ptr()
+            if lc.ff:
+                ffp = _up(lc.ff, 64)
+                lay.norm2 = vec(p + "norm2", Wp)
+                if lc.post_norm:
+                    lay.norm2b = vec(p + "norm2b", Wp)
+                f = p + "mlp."
+                gu = torch.stack([_pad_to(g(f + "gate"), ffp, Wp), _pad_to(g(f + "up"), ffp, Wp)], dim=1)
+                lay.mlp.ff, lay.mlp.gu_w = lc.ff, hold(gu.view(2 * ffp, Wp)).data_ptr()
+                lay.mlp.down_w = hold(_pad_to(g(f + "down"), Wp, ffp)).data_ptr()
+                if lc.mlp_bias:
+                    gb = torch.stack([_pad_to(g(f + "gate.b"), ffp), _pad_to(g(f + "up.b"), ffp)], dim=1)
+                    lay.mlp.gu_b = hold(gb.view(2 * ffp)).data_ptr()
+                    lay.mlp.down_b = hold(_pad_to(g(f + "down.b"), Wp)).data_ptr()
+        w = L.DecoderWeights()
+        w.dtype, w.width, w.vocab, w.layers, w.eps = L.dtype_code(dtype), cfg.width, cfg.vocab_size, len(cfg.layers), cfg.eps
+        w.final_norm, w.head = vec("final.norm", Wp), self.head.data_ptr()
+        w.layer = C.cast(self.layers, C.POINTER(L.DecoderLayer))
+        self.struct = w
+        # columns of every cached layer's block in a token's cache, in layer order
+        self.cache_widths = [_up(lc.mixer.kv_rank, 64) + _up(lc.mixer.rot_dim, 32) for lc in cfg.layers if lc.mixer.kv_from is None]
+
+
 # ---- random initialisation at arbitrary dimensions (no checkpoints are reachable: README.md:56-58) ----
 
 def random_vit_state(cfg: VisionConfig, seed: int = 0, device="cpu", dtype=torch.float32, std: float = 0.02):
@@ -300,6 +506,22 @@ def random_llm_state(cfg: LlmConfig, seed: int = 2, device="cpu", dtype=torch.fl
         st[p + "self_attn.o_proj.weight"] = r(H, H)
         st[p + "mlp.gate_proj.weight"], st[p + "mlp.up_proj.weight"] = r(I, H), r(I, H)
         st[p + "mlp.down_proj.weight"] = r(H, I)
+    return st
+
+
+def random_decoder_state(cfg: DecoderConfig, seed: int = 3, device="cpu", dtype=torch.float32, std: Optional[float] = None):
+    """decoder_tensors with norms near one and matrices of standard deviation `std` (default 1 / sqrt(inputs))"""
+    g = torch.Generator(device=device).manual_seed(seed)
+    st = {}
+    for name, shape in decoder_tensors(cfg).items():
+        t = torch.randn(*shape, generator=g, device=device, dtype=torch.float32)
+        if "norm" in name.rsplit(".", 1)[-1]:
+            t = 1 + 0.1 * t
+        elif len(shape) == 2 and name != "embed":
+            t = t * (shape[1] ** -0.5 if std is None else std)
+        elif name.endswith(".b"):
+            t = t * 0.1
+        st[name] = t.to(dtype)
     return st
 
 

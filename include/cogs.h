@@ -424,6 +424,67 @@ cogs_status cogs_llm_forward_segments(cogs_handle h, cogs_stream stream, const v
                                       const int32_t* cu_seqlens_host, int nseg, float* pooled_means, void* ws,
                                       size_t ws_bytes);
 
+/* ------------------------------------- decoder-only models described layer by layer ------ */
+
+/* A pre-normed decoder whose layers are listed one by one, each with a mixer and an optional gated MLP and optional norms on
+ * the sublayers' outputs:
+ *     x += norm1b(mixer(norm1(x)));   x += norm2b(mlp(norm2(x)));   logits = head . final_norm(x)
+ * The residual stream x, every norm, rotary angle, softmax and gate is fp32; matrix products take `dtype` operands.
+ *
+ * Padding (zeros, in weights, embeddings and norm vectors): width_p = width and ff_p = ff to a multiple of 64, vocab_p to 4;
+ * q_rank_p and kv_rank_p to 64; rot_c = rot_dim to 32 (its columns in the cache); dim_p = dim and rot_p = rot_dim to 8;
+ * dq = dim_p + rot_p to 32; vdim_p = vdim to 16; o_in = heads * vdim_p to 64; heads_p = heads to 4. dim_k = dim to 32.
+ * Norm vectors are fp32; everything else is in `dtype`.
+ *
+ * cogs_latent_mixer: multi-head latent attention. Per token a row [latent (kv_rank_p) | rotated key part (rot_c)] is cached;
+ * keys and values of all heads are linear images of the latent. Rotated dimensions are packed as adjacent pairs (2i, 2i+1),
+ * whatever pairs the model rotates (the packer permutes the rows of q_w and in_w alike).
+ *   in_w   [q_rank_p | kv_rank_p | rot_c | heads_p][width_p]: query latent, kv latent, rotated key part (the middle two absent
+ *          with kv_from >= 0), gate logits (absent unless gated), stacked in this order
+ *   q_w    [heads][dim_p | rot_p | 0 .. dq][q_rank_p]
+ *   kv_w   [heads * dim_p | heads * vdim_p][kv_rank_p]: keys, then values, head by head
+ *   k_abs  [heads][kv_rank_p][dim_k]: the key rows of kv_w transposed per head
+ *   o_w    [width_p][o_in]
+ *   sink   fp32 [heads] or NULL: a logit per head that joins the softmax sum and has no value, times log2(e)
+ *   gated  head h's output is multiplied by sigmoid(gate logit h)
+ *   kv_from >= 0: read the cached rows of that earlier layer (which has its own; equal kv_rank, rot_dim, rotation) */
+typedef struct {
+    int heads, dim, rot_dim, vdim, q_rank, kv_rank;
+    int kv_from;
+    int gated;
+    float scale;
+    float rot_mag;             /* factor on cos and sin */
+    const double* rot_freq;    /* host [rot_dim / 2]: radians per position of each pair */
+    const void* in_w; const float *q_norm, *kv_norm;
+    const void *q_w, *kv_w, *k_abs;
+    const float* sink;
+    const void* o_w;
+} cogs_latent_mixer;
+/* gu_w [2 * ff_p, width_p] rows interleaved (gate_i, up_i), gu_b likewise; down_w [width_p, ff_p]; biases nullable; ff = 0: none */
+typedef struct { int ff; const void *gu_w, *gu_b, *down_w, *down_b; } cogs_gated_mlp;
+typedef struct {
+    const float *norm1, *norm1b, *norm2, *norm2b;      /* norm1b, norm2b nullable: the sublayer's output is added as it is */
+    cogs_latent_mixer mixer;
+    cogs_gated_mlp mlp;
+} cogs_decoder_layer;
+typedef struct {
+    int dtype, width, vocab, layers;
+    float eps;
+    const float* final_norm;
+    const void* head;                                  /* [vocab_p][width_p] */
+    const cogs_decoder_layer* layer;                   /* host array [layers] */
+} cogs_decoder_weights;
+cogs_status cogs_decoder_load(cogs_handle h, const cogs_decoder_weights* w);
+/* elements per token of a sequence's cache (all cached layers). A cache is a cogs_kv with k = max_len * this many elements, v unused */
+cogs_status cogs_decoder_cache_width(cogs_handle h, int64_t* elements);
+cogs_status cogs_decoder_workspace_bytes(cogs_handle h, int rows, int nseq, int64_t total_context, int n_want, size_t* bytes);
+/* One step of `nseq` sequences: sequence i brings lens[i] >= 1 new tokens as rows of embeds [sum lens, width_p] (sequences back
+ * to back), at positions kv[i]->len ..; its cache rows are appended and kv[i]->len advances. No padding, any mix of lengths.
+ * want (host [n_want], row numbers) -> logits fp32 [n_want][vocab_p]. streams, nullable: fp32 [layers][rows][width_p], the
+ * residual stream behind every layer. Steps of one token per sequence take the absorbed form of latent attention. */
+cogs_status cogs_decoder_forward(cogs_handle h, cogs_stream stream, const void* embeds, cogs_kv* const* kv, const int32_t* lens, int nseq,
+                                 const int32_t* want, int n_want, float* logits, float* streams, void* ws, size_t ws_bytes);
+
 #ifdef __cplusplus
 }
 #endif
