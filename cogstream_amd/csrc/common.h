@@ -163,11 +163,8 @@ __device__ __forceinline__ float gelu_tanh_f(float x) {
     const float t = x * fmaf(b, x * x, a);
     return x * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(t));
 }
-// the same on four values in packed fp32 arithmetic: 2 x (v_pk_mul, v_pk_fma, v_pk_mul, v_pk_add, v_pk_mul) + 4 v_exp + 4 v_rcp
-// instead of 4 x 5 scalar VALU + the same transcendentals. Written on vectors because hipcc's SLP pass only packs about half of
-// the scalar form inside the GEMM epilogues, and every VALU instruction there is taken from the matrix pipe
-// (profiles/r5_prefill_attn_anatomy.txt section 4: ~2 cycles per instruction beside 16x16x32 MFMAs; v_exp / v_rcp run beside it).
-// Bit-identical to gelu_tanh_f per element (same operations in the same order).
+// the same on four values, bit-identical per element (same operations in the same order). Written on vectors so that the epilogues
+// keep the four values together; the build has packed fp32 instructions switched off, so each operation is four scalar ones.
 __device__ __forceinline__ f32x4 gelu_tanh_4(f32x4 x) {
     const float a = -2.3022082f, b = -0.10294324f;
     const f32x4 a4 = {a, a, a, a}, b4 = {b, b, b, b}, one = {1.f, 1.f, 1.f, 1.f};

@@ -141,8 +141,7 @@ __global__ __launch_bounds__(256, 4) void sqdist_kernel(const T* __restrict__ x,
             for (int q = 0; q < 4; ++q) {
                 const f32x4 c0 = *reinterpret_cast<const f32x4*>(cl + (m + q) * SL);
                 const f32x4 c1 = *reinterpret_cast<const f32x4*>(cl + (m + q) * SL + 256);
-                // the two rows ride in the two halves of a register pair: v_pk_add_f32 / v_pk_fma_f32 do both rows'
-                // subtraction and fma in one instruction each. Every accumulator still sees its own products in the same
+                // the two rows ride in the two halves of a register pair. Every accumulator still sees its own products in the same
                 // order (column e of the first half, then of the second), so the sums are bit-identical to the scalar form
                 f32x2 s = {0.f, 0.f};
 #pragma unroll

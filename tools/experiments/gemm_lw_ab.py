@@ -19,7 +19,7 @@ HERE = os.path.dirname(os.path.abspath(__file__))
 SO = os.path.join(HERE, "libgemm_lw.so")
 if not os.path.exists(SO) or os.path.getmtime(SO) < os.path.getmtime(os.path.join(HERE, "gemm_lw.hip")):
     import subprocess
-    subprocess.check_call(["/opt/rocm/bin/hipcc", "-O3", "-std=c++17", "-fPIC", "-shared", "--offload-arch=gfx950",
+    subprocess.check_call(["/opt/rocm/bin/hipcc", "-O3", "-std=c++17", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", "-fPIC", "-shared", "--offload-arch=gfx950",
                            "-I", os.path.join(ROOT, "cogstream_amd", "csrc"), os.path.join(HERE, "gemm_lw.hip"), "-o", SO])
 dev = torch.device("cuda:0")
 fn = C.CDLL(SO).cogs_x_gemm_lw

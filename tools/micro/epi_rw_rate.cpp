@@ -3,7 +3,7 @@
 // per row) move faster through the CU's vector-memory path? Each wave owns a 128-row x 128-byte region of a 256 x 256
 // bf16 tile (as in gemm_tn_pp64_kernel: 8 waves, region = rows 128 g.., columns 64 wc..), 16 instructions per region and
 // kind; 256 workgroups walk the tiles of an M x 1152 matrix (row stride 2 304 bytes) like the persistent GEMM does.
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 tools/micro/epi_rw_rate.cpp -o tools/micro/epi_rw_rate && tools/micro/epi_rw_rate
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/micro/epi_rw_rate.cpp -o tools/micro/epi_rw_rate && tools/micro/epi_rw_rate
 #include <hip/hip_runtime.h>
 #include <cstdio>
 #include <cstdint>

@@ -1,5 +1,5 @@
 // Cost of a grid-wide barrier inside one persistent kernel on MI355X (decode-path study):
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 tools/micro/grid_barrier.cpp -o tools/micro/grid_barrier
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/micro/grid_barrier.cpp -o tools/micro/grid_barrier
 // Every workgroup: (optional agent-scope release fence) -> atomic arrive -> spin on the generation word (bounded) ->
 // (optional acquire fence). Prints microseconds per barrier for 256 / 512 / 1024 workgroups of 256 threads.
 #include <hip/hip_runtime.h>

@@ -1,7 +1,7 @@
 // How fast does a CU take in LDS-DMA pieces (global_load_lds_dwordx4, 1 KiB per wave instruction) from L2-resident rows,
 // as a function of how a piece's 64 lanes are spread over rows? The GEMM K loop stages 16 rows x 64 B per piece (32-wide
 // bf16 K-tiles); the alternatives take whole 128-byte lines (8 rows x 128 B), 4 rows x 256 B, or 1 KiB of one row.
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 tools/micro/ldsdma_rate.cpp -o tools/micro/ldsdma_rate
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/micro/ldsdma_rate.cpp -o tools/micro/ldsdma_rate
 // 256 workgroups x 8 waves, every wave keeps 8 pieces in flight; all workgroups walk the same 512-row panel (L2 hits).
 #include <hip/hip_runtime.h>
 #include <cstdio>

@@ -1,6 +1,6 @@
 // Is a weight matrix that a previous kernel has touched cheaper to stream than one that comes from HBM? (decode: the next
 // GEMV's weights do not depend on the previous kernel's result, so a side stream could read them ahead into the Infinity Cache.)
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 tools/micro/mall_prefetch.cpp -o tools/micro/mall_prefetch
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/micro/mall_prefetch.cpp -o tools/micro/mall_prefetch
 // For sizes 26 / 33 / 136 / 272 MB: the streaming kernel (non-temporal 16-byte loads, 64 KiB per workgroup, like the GEMV) timed
 // cold (after 2 GB of other traffic) and after a prefetch pass of the same buffer with plain loads / with non-temporal loads.
 #include <hip/hip_runtime.h>

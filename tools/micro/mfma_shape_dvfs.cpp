@@ -4,7 +4,7 @@
 // holds (MI355X_MICROARCH.md, DVFS give-back item 7). Every CU runs 1 or 2 waves per SIMD, each wave a back-to-back stream of
 // MFMAs on four independent accumulator sets with operands in registers (random bf16 from a buffer; zeros as the control).
 // The in-kernel clock is measured the guide's way: d(s_memtime) / d(s_memrealtime) * 100 MHz over the loop of one workgroup.
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 tools/micro/mfma_shape_dvfs.cpp -o tools/micro/mfma_shape_dvfs && tools/micro/mfma_shape_dvfs
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/micro/mfma_shape_dvfs.cpp -o tools/micro/mfma_shape_dvfs && tools/micro/mfma_shape_dvfs
 #include <hip/hip_runtime.h>
 #include <algorithm>
 #include <cstdint>

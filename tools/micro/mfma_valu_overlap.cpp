@@ -1,7 +1,7 @@
 // Does the matrix pipe of a gfx950 SIMD run beside its VALU / transcendental pipe? One wave (or two) per SIMD issues, per
 // loop iteration (16 cycles of loop control included), M independent MFMAs and E independent v_exp_f32 / A independent v_add_f32, in a fixed interleaved order
 // (asm volatile keeps it); the shader-clock cycles per iteration say whether the times add or overlap.
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 tools/micro/mfma_valu_overlap.cpp -o tools/micro/mfma_valu_overlap
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/micro/mfma_valu_overlap.cpp -o tools/micro/mfma_valu_overlap
 #include <hip/hip_runtime.h>
 #include <cstdio>
 typedef __attribute__((__vector_size__(8 * sizeof(__bf16)))) __bf16 bf16x8;

@@ -1,7 +1,7 @@
 // Does a decode GEMV run faster when part of its weights is already in the 256 MiB Infinity Cache? One layer's gate/up
 // projection (N 37 888, K 3 584, 271.6 MB of bf16 weights, SwiGLU) behind a kernel that has just read the first P MB of
 // those weights with default-policy loads:
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -I cogstream_amd/csrc tools/micro/prefetch_micro.cpp -o tools/micro/prefetch_micro
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 -I cogstream_amd/csrc tools/micro/prefetch_micro.cpp -o tools/micro/prefetch_micro
 // Weights rotate through > 1 GiB, so whatever the GEMV finds on the die was put there by the prefetch of the same round.
 #include "../../cogstream_amd/csrc/gemv.hip"
 #include <cstdio>

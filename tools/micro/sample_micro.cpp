@@ -1,5 +1,5 @@
 // Phase stamps of the sampler's merge kernel (csrc/sample.hip):
-//   hipcc -O3 -std=c++17 --offload-arch=gfx950 -DCOGS_SAMPLE_STAMPS -I cogstream_amd/csrc tools/micro/sample_micro.cpp -o tools/micro/sample_micro
+//   hipcc -O3 -std=c++17 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 -DCOGS_SAMPLE_STAMPS -I cogstream_amd/csrc tools/micro/sample_micro.cpp -o tools/micro/sample_micro
 #include "../../cogstream_amd/csrc/sample.hip"
 #include <cstdio>
 #include <random>
