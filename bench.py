@@ -431,6 +431,123 @@ def launch_ranks(n: int) -> int:
     return proc.wait()
 
 
+# (name, width, heads, q_rank, kv_rank, ff, layers); unrotated / rotated / value head sizes 128 / 64 / 128. The Qwen2 model beside
+# each has the same width, heads (of 128), feed-forward, layers and vocabulary, and a quarter of the heads as key/value heads
+PABALIX_SIZES = [("w2048", 2048, 16, 768, 512, 5632, 9), ("w3584", 3584, 28, 1536, 512, 18944, 6), ("w4096", 4096, 32, 1536, 512, 11008, 6)]
+PABALIX_VOCAB = 32768
+
+
+def pabalix_config(width, heads, q_rank, kv_rank, ff, layers):
+    kinds = ("latent_attention_3", "latent_attention", "latent_attention_2")
+    out = []
+    for i in range(layers):
+        rot = dict(base=10000.0, dims=64)
+        if kinds[i % 3] != "latent_attention_2":
+            rot["scaling"] = dict(factor=4.0, original=4096, fast=32.0, slow=1.0)
+        mx = dict(heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank, kv_rank=kv_rank, scale=192 ** -0.5, rot=rot)
+        if i % 6 == 5:
+            mx["kv_from"] = i - 3
+        out.append(dict(type=kinds[i % 3], mixer=mx, mlp=dict(kind="dense", ff=ff)))
+    return dict(architecture="Pabalix", layers=out, norm=dict(eps=1e-6), vocab=PABALIX_VOCAB, width=width)
+
+
+def bench_pabalix(args, dev):
+    """prefill (one prompt of 4096 tokens) and decode (behind 4096 tokens; 1 and 16 sequences) tokens/s of the engine's own steps,
+    greedy token choice included, Pabalix and the equal-size Qwen2 model timed in turn; per-class GPU time from event brackets"""
+    from cogstream_amd import _lib as L
+    from cogstream_amd import ops
+    from cogstream_amd.llm import DecoderEngine, Qwen2Engine
+    from cogstream_amd.pabalix import parse_config
+    from cogstream_amd.weights import LlmConfig, random_decoder_state, random_llm_state
+    S, ctx0 = 4096, 4096
+    classes = ["gemm", "attention", "norm", "other"]
+
+    def profile(h, fn):
+        L.check(L.lib.cogs_profile_begin(h.h), "cogs_profile_begin")
+        fn()
+        ms, n = (C.c_float * 8)(), (C.c_int * 8)()
+        L.check(L.lib.cogs_profile_end(h.h, L.current_stream(), ms, n), "cogs_profile_end")
+        return {c: round(ms[i], 4) for i, c in enumerate(classes) if n[i]}
+
+    def measure(e, batch_sizes):
+        res = {}
+        g = torch.Generator().manual_seed(0)
+        ids = torch.randint(0, PABALIX_VOCAB, (S,), generator=g)
+        cache = e.new_cache(S + 256)
+        emb = e.embed_tokens(ids)
+
+        def prefill():
+            cache.reset(0)
+            return e.forward_batch(emb, [S], [cache], [S - 1])
+
+        for _ in range(args.warmup):
+            prefill()
+        torch.cuda.synchronize()
+        t = []
+        for _ in range(args.steps):
+            t0 = time.perf_counter()
+            prefill()
+            torch.cuda.synchronize()
+            t.append(time.perf_counter() - t0)
+        sec = sorted(t)[len(t) // 2]
+        res["prefill"] = {"tokens_per_s": round(S / sec, 1), "ms": round(sec * 1e3, 3), "class_ms": profile(e.handle, prefill)}
+        for B in batch_sizes:
+            caches = [cache]
+            for _ in range(B - 1):
+                c = e.new_cache(S + 256)
+                c.copy_rows_from(cache, ctx0)
+                caches.append(c)
+            toks = torch.zeros(B, dtype=torch.int64, device=dev)
+
+            def step():
+                lg = e.forward_batch(e.embed_tokens(toks), [1] * B, caches, list(range(B)))
+                for i in range(B):
+                    ops.argmax(lg[i], out=toks[i:i + 1])
+
+            n = 16
+            best = []
+            for rep in range(args.warmup + args.steps):
+                for c in caches:
+                    c.reset(ctx0)
+                torch.cuda.synchronize()
+                t0 = time.perf_counter()
+                for _ in range(n):
+                    step()
+                torch.cuda.synchronize()
+                if rep >= args.warmup:
+                    best.append((time.perf_counter() - t0) / n)
+            for c in caches:
+                c.reset(ctx0)
+            sec = sorted(best)[len(best) // 2]
+            res[f"decode_b{B}"] = {"tokens_per_s": round(B / sec, 1), "ms_per_step": round(sec * 1e3, 4), "class_ms": profile(e.handle, step)}
+        return res
+
+    out = {"metric": "Pabalix prefill tokens/sec", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+           "higher_is_better": True, "vs_baseline": None, "dtype": "bf16", "data": "synthetic tokens, random weights",
+           "config": {"prompt": S, "context": ctx0, "vocab": PABALIX_VOCAB}, "sizes": {}}
+    for name, width, heads, q_rank, kv_rank, ff, layers in PABALIX_SIZES:
+        dc = parse_config(pabalix_config(width, heads, q_rank, kv_rank, ff, layers))
+        st = random_decoder_state(dc, seed=1, device=dev, dtype=torch.bfloat16)
+        params = sum(v.numel() for v in st.values())
+        e = DecoderEngine(st, dc, dtype=torch.bfloat16, device=dev)
+        del st
+        mine = measure(e, (1, 16))
+        del e
+        torch.cuda.empty_cache()
+        lc = LlmConfig(hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads,
+                       num_key_value_heads=heads // 4, vocab_size=PABALIX_VOCAB)
+        q = Qwen2Engine(random_llm_state(lc, seed=2, device=dev, dtype=torch.bfloat16), lc, dtype=torch.bfloat16, device=dev)
+        theirs = measure(q, (1, 16))
+        del q
+        torch.cuda.empty_cache()
+        out["sizes"][name] = {"width": width, "heads": heads, "q_rank": q_rank, "kv_rank": kv_rank, "ff": ff, "layers": layers,
+                              "parameters": params, "pabalix": mine, "qwen2": theirs}
+        print(f"[bench pabalix] {name} done", file=sys.stderr, flush=True)
+    last = out["sizes"][PABALIX_SIZES[-1][0]]["pabalix"]["prefill"]
+    out["value"], out["ms_per_step"] = last["tokens_per_s"], last["ms"]
+    return out
+
+
 def main() -> None:
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -445,10 +562,11 @@ def main() -> None:
     ap.add_argument("--scaling", default="strong", choices=["weak", "strong"],
                     help="N > 1 headline: strong = --frames in total (the metric's clip at every N; default), weak = --frames "
                          "per GPU (clip of frames*N)")
-    ap.add_argument("--config", default="cfg2", choices=["cfg2", "cfg3", "cfg5"],
+    ap.add_argument("--config", default="cfg2", choices=["cfg2", "cfg3", "cfg5", "pabalix"],
                     help="cfg2: BASELINE configs[1] (64-frame clip; the metric's config). cfg3: configs[2], one 256-frame "
                          "clip at the 16384-token budget (140x280 per frame) sharded over the ranks. cfg5: configs[4], one "
-                         "64-frame clip per GPU answered through the whole product API (replicas, no collective)")
+                         "64-frame clip per GPU answered through the whole product API (replicas, no collective). pabalix: prefill and "
+                         "decode of Pabalix at sizes of real layers (random weights), beside Qwen2 layers of equal size")
     ap.add_argument("--no-cfg3", action="store_true", help="skip the extra configs[2] measurement of the default run")
     ap.add_argument("--payload", default="projected", choices=["projected", "encoder"],
                     help="N > 1: what the all-gather carries (3584-wide projected tokens / 1152-wide encoder tokens, "
@@ -501,6 +619,11 @@ def main() -> None:
     debug_applied = L.debug_from_spec(args.debug)
     from cogstream_amd.parallel import frame_shards, gather_tokens
     from cogstream_amd.preprocess_gpu import preprocess_videos_gpu
+    if args.config == "pabalix":
+        if world > 1:
+            raise SystemExit("--config pabalix runs on one GPU")
+        print(json.dumps(bench_pabalix(args, dev)), flush=True)
+        return
     if args.config == "cfg5":
         out = bench_cfg5(args, rank, world, dev, ranks_seen)
         if world > 1:

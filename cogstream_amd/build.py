@@ -183,49 +183,23 @@ def build(force: bool = False, verbose: bool = False) -> Path:
                              f"instructions ({len(slack)} with more: {extra or 'none'})\n")
             if verbose:
                 print(stamp.read_text().strip(), flush=True)
-    attn_o, m0_stamp = OBJ / "attn_vit.o", OBJ / "attn_vit.m0_check.txt"
-    if not m0_stamp.exists() or m0_stamp.stat().st_mtime < attn_o.stat().st_mtime:
+    # kernels whose LDS-DMA is inline assembly that writes M0 (their dma16 / issue4)
+    for stem, kernel in (("attn_vit", "attn_vit_pipe_kernel"), ("attn", "attn_prefill_dma_kernel"), ("gemm", "gemm_tn_pp64_kernel"),
+                         ("mla", "mla_prefill_kernel")):
+        o, m0_stamp = OBJ / f"{stem}.o", OBJ / f"{stem}.m0_check.txt"
+        if m0_stamp.exists() and m0_stamp.stat().st_mtime >= o.stat().st_mtime:
+            continue
         try:
-            m0_bad = check_m0_uses(attn_o)
+            m0_bad = check_m0_uses(o, kernel)
         except (OSError, RuntimeError) as e:
             if strict:
                 raise
-            print(f"WARNING: M0 check of attn_vit.o not possible ({e})", flush=True)
-            m0_bad = None
+            print(f"WARNING: M0 check of {stem}.o not possible ({e})", flush=True)
+            continue
         if m0_bad:
-            raise RuntimeError("attn_vit_pipe_kernel: hipcc generated its own uses of M0 beside the inline-asm LDS-DMA "
-                               "(csrc/attn_vit.hip, dma16): " + "; ".join(m0_bad[:6]))
-        if m0_bad is not None:
-            m0_stamp.write_text("ok: every m0 reference inside attn_vit_pipe_kernel is an inline-asm s_mov_b32 m0, sN\n")
-    # the same inline-asm LDS-DMA in the Qwen2 prompt attention (csrc/attn.hip, attn_prefill_dma_kernel)
-    attn2_o, m0_stamp2 = OBJ / "attn.o", OBJ / "attn.m0_check.txt"
-    if not m0_stamp2.exists() or m0_stamp2.stat().st_mtime < attn2_o.stat().st_mtime:
-        try:
-            m0_bad = check_m0_uses(attn2_o, "attn_prefill_dma_kernel")
-        except (OSError, RuntimeError) as e:
-            if strict:
-                raise
-            print(f"WARNING: M0 check of attn.o not possible ({e})", flush=True)
-            m0_bad = None
-        if m0_bad:
-            raise RuntimeError("attn_prefill_dma_kernel: hipcc generated its own uses of M0 beside the inline-asm LDS-DMA "
-                               "(csrc/attn.hip, dma16): " + "; ".join(m0_bad[:6]))
-        if m0_bad is not None:
-            m0_stamp2.write_text("ok: every m0 reference inside attn_prefill_dma_kernel is an inline-asm s_mov_b32 m0, sN\n")
-    m0_stamp3 = OBJ / "gemm.m0_check.txt"
-    if not m0_stamp3.exists() or m0_stamp3.stat().st_mtime < gemm_o.stat().st_mtime:
-        try:
-            m0_bad = check_m0_uses(gemm_o, "gemm_tn_pp64_kernel")
-        except (OSError, RuntimeError) as e:
-            if strict:
-                raise
-            print(f"WARNING: M0 check of gemm.o not possible ({e})", flush=True)
-            m0_bad = None
-        if m0_bad:
-            raise RuntimeError("gemm_tn_pp64_kernel: hipcc generated its own uses of M0 beside the inline-asm LDS-DMA "
-                               "(csrc/gemm.hip, issue4): " + "; ".join(m0_bad[:6]))
-        if m0_bad is not None:
-            m0_stamp3.write_text("ok: every m0 reference inside gemm_tn_pp64_kernel is an inline-asm s_mov_b32 m0, sN\n")
+            raise RuntimeError(f"{kernel}: hipcc generated its own uses of M0 beside the inline-asm LDS-DMA (csrc/{stem}.hip): "
+                               + "; ".join(m0_bad[:6]))
+        m0_stamp.write_text(f"ok: every m0 reference inside {kernel} is an inline-asm s_mov_b32 m0, sN\n")
     objs = [OBJ / (s.stem + ".o") for s in srcs]
     if force or jobs or _stale(LIB, objs):
         cmd = [HIPCC, "-shared", "-fPIC", f"--offload-arch={ARCH}", "-o", str(LIB)] + [str(o) for o in objs]

@@ -139,7 +139,7 @@ struct Step {
         const float* gate = m.gated ? k.gate : nullptr;
         if (absorbed_step(S, nseq)) {
             {
-                CogsHeadGemm a{k.q, qcols, G.dq, m.k_abs, k.qlat, (long)m.heads * G.kvw, G.kvw, S, m.heads, G.kvp, G.dk, nullptr, G.rotc, G.dn, G.dr};
+                CogsHeadGemm a{k.q, qcols, G.dq, m.k_abs, k.qlat, (long)m.heads * G.kvw, G.kvw, S, m.heads, G.kvp, G.dk, nullptr, G.rotc, G.dk, G.dr};
                 PROF(COGS_PROF_GEMM);
                 COGS_TRY(cogs_k_head_gemm(st, dt, a));
             }
@@ -150,7 +150,7 @@ struct Step {
                 COGS_TRY(cogs_k_mla_decode(st, a));
             } else {
                 CogsMla a{};
-                a.Q = k.qlat; a.ldq = (long)m.heads * G.kvw; a.q_head = G.kvw; a.ldk = a.ldkr = a.ldv = G.kvw;
+                a.Q = k.qlat; a.ldq = (long)m.heads * G.kvw; a.q_head = G.kvw; a.q_rot = G.kvp; a.ldk = a.ldkr = a.ldv = G.kvw;
                 a.O = k.olat; a.ldo = (long)m.heads * G.kvp; a.o_head = G.kvp; a.dn = G.kvp; a.dr = G.rotc; a.dv = G.kvp; a.heads = m.heads;
                 a.sink = m.sink; a.seqs = k.seqs; a.nseq = nseq; a.rowseq = k.rowseq; a.rows = S; a.max_new = 1;
                 a.absorbed = 1; a.layer_off = G.cache_off; a.kr_col = G.kvp;
@@ -171,7 +171,7 @@ struct Step {
                 COGS_TRY(lin(g));
             }
             CogsMla a{};
-            a.Q = k.q; a.ldq = qcols; a.q_head = G.dq; a.K = k.kvx; a.ldk = G.kvcols; a.k_head = G.dn;
+            a.Q = k.q; a.ldq = qcols; a.q_head = G.dq; a.q_rot = G.dk; a.K = k.kvx; a.ldk = G.kvcols; a.k_head = G.dn;
             a.KR = at(ctx, G.kvp); a.ldkr = G.kvw; a.V = at(k.kvx, (size_t)m.heads * G.dn); a.ldv = G.kvcols; a.v_head = G.dv;
             a.O = k.att; a.ldo = G.oin; a.o_head = G.dv; a.dn = G.dn; a.dr = G.dr; a.dv = G.dv; a.heads = m.heads;
             a.sink = m.sink; a.gate = gate; a.seqs = k.seqs; a.nseq = nseq; a.rowseq = k.rowseq; a.rows = S; a.max_new = max_new;
@@ -230,7 +230,7 @@ cogs_status cogs_decoder_load(cogs_handle h, const cogs_decoder_weights* w) {
         LatentGeom G{};
         G.own = m.kv_from < 0;
         G.qrp = up(m.q_rank, 64); G.kvp = up(m.kv_rank, 64); G.rotc = up(m.rot_dim, 32); G.kvw = G.kvp + G.rotc;
-        G.dn = up(m.dim, 8); G.dr = up(m.rot_dim, 8); G.dq = up(G.dn + G.dr, 32); G.dk = up(m.dim, 32); G.dv = up(m.vdim, 16);
+        G.dn = up(m.dim, 8); G.dr = up(m.rot_dim, 8); G.dk = up(m.dim, 32); G.dq = G.dk + up(m.rot_dim, 32); G.dv = up(m.vdim, 16);
         G.oin = up(m.heads * G.dv, 64); G.headsp = up(m.heads, 4);
         G.ldt = G.qrp + (G.own ? G.kvw : 0) + (m.gated ? G.headsp : 0);
         G.kvcols = m.heads * (G.dn + G.dv);
@@ -249,12 +249,12 @@ cogs_status cogs_decoder_load(cogs_handle h, const cogs_decoder_weights* w) {
         G.rope = -1;
         for (size_t s = 0; s < d->sets.size(); ++s) {
             const CogsRopeSet& R = d->sets[s];
-            if (R.pairs == G.dq / 2 && R.first == G.dn / 2 && R.n == n && R.mag == m.rot_mag &&
+            if (R.pairs == G.dq / 2 && R.first == G.dk / 2 && R.n == n && R.mag == m.rot_mag &&
                 memcmp(freq.data() + freq_at[s], m.rot_freq, n * sizeof(double)) == 0) G.rope = (int)s;
         }
         if (G.rope < 0) {
             G.rope = (int)d->sets.size();
-            d->sets.push_back(CogsRopeSet{d->rope_width, G.dq / 2, G.dn / 2, n, m.rot_mag, nullptr});
+            d->sets.push_back(CogsRopeSet{d->rope_width, G.dq / 2, G.dk / 2, n, m.rot_mag, nullptr});
             freq_at.push_back(freq.size());
             freq.insert(freq.end(), m.rot_freq, m.rot_freq + n);
             d->rope_width += G.dq;

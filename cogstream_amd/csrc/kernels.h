@@ -206,7 +206,7 @@ struct CogsHeadGemm {      // y[b][h][n] = gate[b][h] * sum_k x[b][h][k] W[h][n]
 };
 int cogs_k_head_gemm(hipStream_t st, int dtype, const CogsHeadGemm& a);
 struct CogsMla {
-    const void* Q; long ldq; int q_head;         // per head [dn | dr | zeros], scores in log2 units
+    const void* Q; long ldq; int q_head, q_rot;  // per head dn unrotated columns, from column q_rot dr rotated ones, zeros; log2 units
     const void* K; long ldk; int k_head;         // expanded keys; absorbed: ldk = ldkr = ldv = cache row, pointers from the sequence
     const void* KR; long ldkr;
     const void* V; long ldv; int v_head;

@@ -16,11 +16,12 @@
 // multiplies the finished head row.
 //
 // Padded sizes (zeros, by the packer): dn = unrotated query/key part, dr = rotated part (multiples of 8), dv = value
-// (multiple of 16), a query head is [dn | dr | 0] in dq = 32-multiple columns; a cache row is [c: kvp = 64-multiple | kr:
+// (multiple of 16); a query head is [dn, zeros to a 32-multiple | dr, zeros to a 32-multiple]; a cache row is [c: kvp = 64-multiple | kr:
 // 32-multiple] = kvw columns.
 #include "common.h"
 #include "kernels.h"
 #include "debug.h"
+#include <type_traits>
 
 namespace {
 
@@ -130,15 +131,19 @@ struct HeadGemmArgs {
     int tail, tail_src, tail_n;             // y[N .. N+tail) = x[tail_src + j] for j < tail_n, else 0
 };
 
-// y[b][h][n] = sum_k x[b][h][k] W[h][n][k]: up to 16 batch rows are the MFMA columns, a wave owns 16 outputs of one head
+// y[b][h][n] = sum_k x[b][h][k] W[h][n][k]: up to 16 batch rows are the MFMA columns. A wave owns 16 outputs of one head; KSPLIT:
+// a workgroup does, and its waves take every fourth 32-wide step of K (the long K of the value product)
+template <bool KSPLIT>
 __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(HeadGemmArgs p) {
-    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6, li = lane & 15, g = lane >> 4;
+    __shared__ __attribute__((aligned(16))) f32x4 red[KSPLIT ? 4 : 1][64];
+    const int lane = threadIdx.x & 63, li = lane & 15, g = lane >> 4;
+    const int wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
     const int h = blockIdx.y, b0 = blockIdx.z * 16, b = b0 + li;
-    const int n0 = (blockIdx.x * 4 + wid) * 16;
+    const int n0 = (KSPLIT ? blockIdx.x : blockIdx.x * 4 + wid) * 16;
     const bf16_t* x = reinterpret_cast<const bf16_t*>(p.X) + (long)min(b, p.B - 1) * p.ldxb + h * p.ldxh;
     bf16_t* y = reinterpret_cast<bf16_t*>(p.Y) + (long)min(b, p.B - 1) * p.ldyb + h * p.ldyh;
     if (n0 >= p.N) {
-        if (n0 < p.N + p.tail && b < p.B) {
+        if (n0 < p.N + p.tail && b < p.B && (!KSPLIT || wid == 0)) {
             const int j0 = n0 - p.N + 4 * g;
 #pragma unroll
             for (int e = 0; e < 4; ++e)
@@ -146,27 +151,34 @@ __global__ __launch_bounds__(256) void head_gemm_bf16_kernel(HeadGemmArgs p) {
         }
         return;
     }
-    const bf16_t* w = reinterpret_cast<const bf16_t*>(p.W) + ((long)h * p.N + n0 + li) * p.K;
+    const bf16_t* w = reinterpret_cast<const bf16_t*>(p.W) + ((long)h * p.N + n0 + li) * p.K + 8 * g;
+    x += 8 * g;
+    constexpr int STEP = KSPLIT ? 4 : 1;
+    const int nk = p.K >> 5;
     f32x4 a0 = {0.f, 0.f, 0.f, 0.f}, a1 = a0;
-    int k = 8 * g;
-    for (; k + 96 < p.K; k += 128) {          // four 32-wide steps in flight
+    for (int k = KSPLIT ? wid : 0; k < nk; k += 4 * STEP) {          // four 32-wide steps in flight; steps past the end are not multiplied
         u32x4 wf[4], xf[4];
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
-            wf[s] = *reinterpret_cast<const u32x4*>(w + k + 32 * s);
-            xf[s] = *reinterpret_cast<const u32x4*>(x + k + 32 * s);
+            const int o = 32 * min(k + STEP * s, nk - 1);
+            wf[s] = *reinterpret_cast<const u32x4*>(w + o);
+            xf[s] = *reinterpret_cast<const u32x4*>(x + o);
         }
+        __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int s = 0; s < 4; ++s) {
+            if (k + STEP * s >= nk) break;
             f32x4& a = (s & 1) ? a1 : a0;
             a = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wf[s]), __builtin_bit_cast(bf16x8, xf[s]), a, 0, 0, 0);
         }
     }
-    for (; k < p.K; k += 32) {
-        const u32x4 wf = *reinterpret_cast<const u32x4*>(w + k), xf = *reinterpret_cast<const u32x4*>(x + k);
-        a0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wf), __builtin_bit_cast(bf16x8, xf), a0, 0, 0, 0);
-    }
     a0 += a1;
+    if constexpr (KSPLIT) {
+        red[wid][lane] = a0;
+        __syncthreads();
+        if (wid) return;
+        a0 = (red[0][lane] + red[1][lane]) + (red[2][lane] + red[3][lane]);
+    }
     if (b < p.B) {
         if (p.gate) a0 *= p.gate[(long)b * p.heads + h];
         st4_f<bf16_t>(y + n0 + 4 * g, a0);
@@ -204,7 +216,7 @@ __global__ __launch_bounds__(64) void mla_rowwise_kernel(CogsMla p) {
     const CogsSeq s = p.seqs[p.rowseq[row]];
     const int nkeys = s.pos0 + (row - s.row0) + 1;
     const T* q = reinterpret_cast<const T*>(p.Q) + (long)row * p.ldq + (long)h * p.q_head;
-    for (int d = lane; d < p.dn + p.dr; d += 64) qs[d] = ld_f<T>(q + d);
+    for (int d = lane; d < p.dn + p.dr; d += 64) qs[d] = ld_f<T>(q + (d < p.dn ? d : p.q_rot + d - p.dn));
     __syncthreads();
     const T *K, *KR, *V;
     if (p.absorbed) {
@@ -271,207 +283,321 @@ __global__ __launch_bounds__(64) void mla_rowwise_kernel(CogsMla p) {
 }
 
 // ------------------------------------------------------------------------------------------------ prompt attention (bf16)
-// 4 waves x 16 NQ query rows of one (sequence, head); 64-key tiles, register-staged (the next tile's loads are in flight during
-// the compute), scores transposed so that a lane's S^T registers of key blocks 2c, 2c+1 are the B operand of the c-th 32-key step
-// of O^T = V^T.P^T (see attn_decode.hip). The softmax sum is one more MFMA per step with an all-ones A operand, i.e. the sum of
-// the bf16 weights that multiply V.
-template <int KS, int DT, int NQ>
-__global__ __launch_bounds__(256, 2) void mla_prefill_kernel(CogsMla p, int nqt) {
-    constexpr int CHK = KS * 4;                  // 16-byte chunks of a K row in LDS
-    constexpr int KRS = KS * 64;                 // K row stride, a multiple of 128 bytes (KS even)
-    constexpr int VRS = DT * 32 + 32;            // V row stride, an odd multiple of 32 bytes (DT even)
-    constexpr int PK = KS, PV = DT / 2;          // staged chunks per thread
-    static_assert(KS % 2 == 0 && DT % 2 == 0, "row strides");
+// 4 waves x 32 query rows of one (sequence, head) against 64-key tiles. Staging as in attn.hip's prompt kernel: a tile's pieces
+// (1 KiB = 64 lanes x 16 bytes) go global -> LDS by LDS-DMA into a double buffer, one tile ahead, one barrier per tile. Keys come
+// from two places -- the head's expanded part and the rotated part all heads share -- so a K tile is two LDS regions of KN and KR
+// 32-dimension steps. LDS-DMA writes lane-linear images: the bank swizzles live on the source address.
+//   scores transposed, S^T = K.Q^T, key rows permuted so that a lane's registers of blocks 2u, 2u+1 are the B operand of the
+//   u-th 32-key step of O^T = V^T.P^T; the accumulator starts at minus the running reference, so P = exp2(acc); the reference
+//   moves only when a score passes it by 2^THR (the sums stay far inside fp32, bf16 keeps its relative precision);
+//   the softmax sum is one more MFMA per step with an all-ones A operand, i.e. the sum of the bf16 weights that multiply V.
+// Columns past dn / dr / dv hold copies of real data: the query's are zero, and value tiles past dv are not stored.
+constexpr float MLA_THR = 6.f;
+
+// 16-byte-chunk XOR of row `row` for rows of `chunks` chunks: 16 rows {8 a + b (+ 4 c)} of a fragment read land in different banks
+template <int CHUNKS> __device__ __forceinline__ int mla_kswz(int row) {
+    if constexpr (CHUNKS % 16 == 0) return (row & 3) | (((row >> 3) & 3) << 2);
+    else if constexpr (CHUNKS % 8 == 0) return ((row >> 1) & 1) | (((row >> 3) & 3) << 1);
+    else return (row >> 3) & 3;
+}
+// 32-byte-unit XOR of a V row of DT units: the (row & 3, row bit 3) classes of a transposing read land in different banks
+template <int DT> __device__ __forceinline__ int mla_vswz(int row) {
+    const int b3 = (row >> 3) & 1;
+    if constexpr (DT % 8 == 0) return (row & 3) | (b3 << 2);
+    else if constexpr (DT % 4 == 0) return ((row >> 1) & 1) | (b3 << 1);
+    else return b3;
+}
+
+template <int KN, int KR, int DT, int WGS>
+__global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nqt, int group) {
+    constexpr int NQ = 2, KS = KN + KR;
+    constexpr int N_LDS = 64 * KN * 64, R_LDS = 64 * KR * 64, V_LDS = 64 * DT * 32, BUF = N_LDS + R_LDS + V_LDS;
+    constexpr int PV = DT / 2;                    // V pieces per wave (K: KN and KR)
+    static_assert(DT % 2 == 0, "whole pieces per wave");
     extern __shared__ __attribute__((aligned(16))) char smem[];
-    char* const Ks = smem;
-    char* const Vs = smem + 64 * KRS;
 
     const int tid = threadIdx.x, lane = tid & 63;
     const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int li = lane & 15, g = lane >> 4;
-    // contiguous runs of (sequence, head) pairs per XCD: the query tiles of a head meet in one L2; long tiles first
-    const int total = gridDim.x;
-    int bid = blockIdx.x;
+    // launch order -> (sequence, head) and query tile. An XCD gets a contiguous run, `group` (sequence, head) pairs at a time (their
+    // K / V meet in its L2), long query tiles first; where a group is two waves of one workgroup per CU (<= 64), the second
+    // wave runs short to long, so that the two workgroups of a CU add up to the same length everywhere
+    int qt, pair;
     {
-        const int xcd = bid & 7, q = total >> 3, r = total & 7;
-        bid = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (bid >> 3);
+        const int total = gridDim.x, xcd = blockIdx.x & 7, q = total >> 3, r = total & 7;
+        const int bid = (xcd < r ? xcd * (q + 1) : r * (q + 1) + (xcd - r) * q) + (blockIdx.x >> 3);
+        const int per = group * nqt, grp = bid / per, np = total / nqt;
+        int i = bid - grp * per;
+        const int gsz = min(group, np - grp * group), n = gsz * nqt;
+        if (n <= 64 && i >= 32) i = n - 1 - (i - 32);
+        qt = nqt - 1 - i / gsz;
+        pair = grp * group + i % gsz;
     }
-    const int pair = bid / nqt, qt = nqt - 1 - bid % nqt;
     const int h = pair % p.heads;
     const CogsSeq s = p.seqs[pair / p.heads];
-    const int q0 = qt * (64 * NQ);
+    const int q0 = qt * 128;
     if (q0 >= s.len) return;
 
     const bf16_t* Q = reinterpret_cast<const bf16_t*>(p.Q) + (long)s.row0 * p.ldq + (long)h * p.q_head;
     const bf16_t* K = reinterpret_cast<const bf16_t*>(p.K) + (long)s.ctx0 * p.ldk + (long)h * p.k_head;
-    const bf16_t* KR = reinterpret_cast<const bf16_t*>(p.KR) + (long)s.ctx0 * p.ldkr;
+    const bf16_t* KRp = reinterpret_cast<const bf16_t*>(p.KR) + (long)s.ctx0 * p.ldkr;
     const bf16_t* V = reinterpret_cast<const bf16_t*>(p.V) + (long)s.ctx0 * p.ldv + (long)h * p.v_head;
-    const int ks = (p.dn + p.dr + 31) >> 5, dt = p.dv >> 4;
-    const int nkc = p.dn >> 3, nc = (p.dn + p.dr) >> 3, nvc = p.dv >> 3;
 
     bf16x8 qf[NQ][KS];
-    int qpos[NQ], qrow[NQ];
+    int qpos[NQ];
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
-        qrow[i] = q0 + wid * 16 * NQ + 16 * i + li;
-        const int rc = min(qrow[i], s.len - 1);
+        const int rc = min(q0 + wid * 32 + 16 * i + li, s.len - 1);
         qpos[i] = s.pos0 + rc;
 #pragma unroll
         for (int k = 0; k < KS; ++k) {
+            const int kk = k < KN ? 32 * k : p.q_rot + 32 * (k - KN);
             u32x4 v = {0, 0, 0, 0};
-            if (k < ks) v = *reinterpret_cast<const u32x4*>(Q + (long)rc * p.ldq + 32 * k + 8 * g);
+            if (k < KN ? 32 * k < p.q_rot : kk < p.q_head) v = *reinterpret_cast<const u32x4*>(Q + (long)rc * p.ldq + kk + 8 * g);
             qf[i][k] = __builtin_bit_cast(bf16x8, v);
         }
     }
-    const int wave_hi = s.pos0 + min(q0 + wid * 16 * NQ + 16 * NQ, s.len) - 1;     // last position of the wave's rows
-    const int wave_lo = s.pos0 + min(q0 + wid * 16 * NQ, s.len - 1);
-    const int kend = s.pos0 + min(q0 + 64 * NQ, s.len);                             // keys the workgroup needs
+    const bool wave_active = q0 + wid * 32 < s.len;
+    const int wave_hi = s.pos0 + min(q0 + wid * 32 + 31, s.len - 1);               // last position of the wave's rows
+    const int kend = s.pos0 + min(q0 + 128, s.len);                                 // keys the workgroup needs
     const int nt = (kend + 63) >> 6;
 
-    f32x4 oacc[NQ][DT], lacc[NQ];
-    float m[NQ];
+    f32x4 oacc[DT][NQ], lacc[NQ];
+    float m_ref[NQ];
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
-        m[i] = -INFINITY;
+        m_ref[i] = 0.f;
         lacc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int d = 0; d < DT; ++d) oacc[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int d = 0; d < DT; ++d) oacc[d][i] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    const u32x4 ones_w = {0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u};
-    const bf16x8 ones = __builtin_bit_cast(bf16x8, ones_w);
+    const bf16x8 ones = __builtin_bit_cast(bf16x8, u32x4{0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u});
 
-    u32x4 kreg[PK], vreg[PV];
-    auto load_tile = [&](int t) {
-        const int kb = t * 64, last = kend - 1;
+    // staging: wave w issues pieces w, w + 4, ... of each region; byte offsets from the tile's first row
+    const unsigned smem_lds = (unsigned)(size_t)(__attribute__((address_space(3))) char*)smem;
+    const int nkc = p.dn >> 3, nrc = p.dr >> 3, nvc = p.dv >> 3;
+    auto k_slot = [&](int i, int& row, int& chunk) {
+        constexpr int CH = KN * 4;
+        const int id = 64 * (wid + 4 * i) + lane;
+        row = id / CH;
+        chunk = min((id % CH) ^ mla_kswz<CH>(row), nkc - 1);
+    };
+    auto r_slot = [&](int i, int& row, int& chunk) {
+        constexpr int CH = KR * 4;
+        const int id = 64 * (wid + 4 * i) + lane;
+        row = id / CH;
+        chunk = min((id % CH) ^ mla_kswz<CH>(row), nrc - 1);
+    };
+    auto v_slot = [&](int i, int& row, int& chunk) {
+        constexpr int CH = DT * 2;
+        const int id = 64 * (wid + 4 * i) + lane, sl = id % CH;
+        row = id / CH;
+        chunk = min((((sl >> 1) ^ mla_vswz<DT>(row)) << 1) | (sl & 1), nvc - 1);
+    };
+    int k_off[KN], r_off[KR], v_off[PV];
 #pragma unroll
-        for (int i = 0; i < PK; ++i) {
-            const int id = tid + 256 * i, r = id / CHK, c = id % CHK;
-            const long j = min(kb + r, last);              // rows past the end repeat the last one; their scores are masked
-            kreg[i] = u32x4{0, 0, 0, 0};
-            if (c < nkc) kreg[i] = *reinterpret_cast<const u32x4*>(K + j * p.ldk + c * 8);
-            else if (c < nc) kreg[i] = *reinterpret_cast<const u32x4*>(KR + j * p.ldkr + (c - nkc) * 8);
+    for (int i = 0; i < KN; ++i) { int row, c; k_slot(i, row, c); k_off[i] = (row * (int)p.ldk + c * 8) * 2; }
+#pragma unroll
+    for (int i = 0; i < KR; ++i) { int row, c; r_slot(i, row, c); r_off[i] = (row * (int)p.ldkr + c * 8) * 2; }
+#pragma unroll
+    for (int i = 0; i < PV; ++i) { int row, c; v_slot(i, row, c); v_off[i] = (row * (int)p.ldv + c * 8) * 2; }
+    auto uniform_ptr = [](const bf16_t* q) -> const bf16_t* {
+        const unsigned long long v = (unsigned long long)q;
+        const unsigned lo = __builtin_amdgcn_readfirstlane((unsigned)v), hi = __builtin_amdgcn_readfirstlane((unsigned)(v >> 32));
+        return (const bf16_t*)(((unsigned long long)hi << 32) | lo);
+    };
+    // (inline assembly for the reason attn_vit.hip gives; the build checks that nothing else in this kernel touches M0)
+    auto dma16 = [&](const bf16_t* base, int off_bytes, unsigned lds) {
+        asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2" :: "s"(lds), "v"(off_bytes), "s"(base) : "memory");
+    };
+    auto issue_tile = [&](int t) {
+        const int kb = t * 64, valid = kend - kb;                      // >= 1; rows past the end repeat the last one (masked)
+        const bf16_t* kp = uniform_ptr(K + (long)kb * p.ldk);
+        const bf16_t* rp = uniform_ptr(KRp + (long)kb * p.ldkr);
+        const bf16_t* vp = uniform_ptr(V + (long)kb * p.ldv);
+        const unsigned st = __builtin_amdgcn_readfirstlane(smem_lds + (t & 1) * BUF);
+        const bool ragged = valid < 64;
+#pragma unroll
+        for (int i = 0; i < KN; ++i) {
+            int o = k_off[i];
+            if (ragged) { int row, c; k_slot(i, row, c); o -= max(row - (valid - 1), 0) * (int)p.ldk * 2; }
+            dma16(kp, o, st + (wid + 4 * i) * 1024);
+        }
+#pragma unroll
+        for (int i = 0; i < KR; ++i) {
+            int o = r_off[i];
+            if (ragged) { int row, c; r_slot(i, row, c); o -= max(row - (valid - 1), 0) * (int)p.ldkr * 2; }
+            dma16(rp, o, st + N_LDS + (wid + 4 * i) * 1024);
         }
 #pragma unroll
         for (int i = 0; i < PV; ++i) {
-            const int id = tid + 256 * i, r = id / (2 * DT), c = id % (2 * DT);
-            const long j = min(kb + r, last);
-            if (c < nvc) vreg[i] = *reinterpret_cast<const u32x4*>(V + j * p.ldv + c * 8);
+            int o = v_off[i];
+            if (ragged) { int row, c; v_slot(i, row, c); o -= max(row - (valid - 1), 0) * (int)p.ldv * 2; }
+            dma16(vp, o, st + N_LDS + R_LDS + (wid + 4 * i) * 1024);
         }
     };
-    const int v_rd = (4 * g + (li >> 2)) * VRS + (li & 3) * 8;
 
-    load_tile(0);
-    for (int t = 0; t < nt; ++t) {
-        __syncthreads();                       // the previous tile's fragment reads are done
-#pragma unroll
-        for (int i = 0; i < PK; ++i) {
-            const int id = tid + 256 * i, r = id / CHK, c = id % CHK;
-            *reinterpret_cast<u32x4*>(Ks + r * KRS + ((c ^ (r & 7)) << 4)) = kreg[i];
-        }
-#pragma unroll
-        for (int i = 0; i < PV; ++i) {
-            const int id = tid + 256 * i, r = id / (2 * DT), c = id % (2 * DT);
-            if (c < nvc) *reinterpret_cast<u32x4*>(Vs + r * VRS + c * 16) = vreg[i];
-        }
-        __syncthreads();
-        if (t + 1 < nt) load_tile(t + 1);
+    const int krow0 = 8 * (li >> 2) + (li & 3);
+    const int vr = 8 * g + (li >> 2);                  // + 32 u (+ 4): mla_vswz is the same for all of them
+    const int v_sw = mla_vswz<DT>(vr);
+    const int v_base = vr * (DT * 32) + (li & 3) * 8;
+
+    auto process_tile = [&](const int t, auto masked_tag, auto first_tag) {
+        constexpr bool MASKED = decltype(masked_tag)::value, FIRST = decltype(first_tag)::value;
         const int kb = t * 64;
-        if (kb > wave_hi) continue;            // (uniform per wave; every wave still meets the barriers above)
-
-        f32x4 sacc[NQ][4];
+        if (!wave_active || (MASKED && kb > wave_hi)) return;
+        const char* Ns = smem + (t & 1) * BUF;
+        const char* Rs = Ns + N_LDS;
+        const char* Vs = Rs + R_LDS;
+        f32x4 sacc[4][NQ];
+        __builtin_amdgcn_s_setprio(0);
 #pragma unroll
         for (int u = 0; u < 4; ++u) {
-#pragma unroll
-            for (int i = 0; i < NQ; ++i) sacc[i][u] = f32x4{0.f, 0.f, 0.f, 0.f};
-            const char* kr = Ks + (16 * u + li) * KRS;
+            const int krow = 32 * (u >> 1) + 4 * (u & 1) + krow0;
+            const int nsw = mla_kswz<KN * 4>(krow), rsw = mla_kswz<KR * 4>(krow);
 #pragma unroll
             for (int k = 0; k < KS; ++k) {
-                if (k >= ks) break;
-                const bf16x8 kf = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(kr + (((4 * k + g) ^ (li & 7)) << 4)));
+                const char* a = k < KN ? Ns + krow * (KN * 64) + (((4 * k + g) ^ nsw) << 4)
+                                       : Rs + krow * (KR * 64) + (((4 * (k - KN) + g) ^ rsw) << 4);
+                const bf16x8 kf = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a));
 #pragma unroll
-                for (int i = 0; i < NQ; ++i) sacc[i][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][k], sacc[i][u], 0, 0, 0);
+                for (int i = 0; i < NQ; ++i) {
+                    const float nm = -m_ref[i];
+                    sacc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][k], k == 0 ? f32x4{nm, nm, nm, nm} : sacc[u][i], 0, 0, 0);
+                }
             }
         }
-        if (kb + 63 > wave_lo) {               // the diagonal (or the ragged end) crosses this tile
+        if constexpr (!MASKED) {                       // 4 KS reads, 8 KS MFMAs: six reads lead, then a read per pair of MFMAs
+            __builtin_amdgcn_sched_group_barrier(0x100, 6, 0);
 #pragma unroll
-            for (int i = 0; i < NQ; ++i)
-#pragma unroll
-                for (int u = 0; u < 4; ++u)
-#pragma unroll
-                    for (int r = 0; r < 4; ++r)
-                        if (kb + 16 * u + 4 * g + r > qpos[i]) sacc[i][u][r] = -INFINITY;
+            for (int i = 0; i < 4 * KS - 6; ++i) {
+                __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);
+                __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+            }
+            __builtin_amdgcn_sched_group_barrier(0x008, 12, 0);
         }
-        bf16x8 pf[NQ][2];
+        __builtin_amdgcn_s_setprio(1);
+        bf16x8 pf[2][NQ];
 #pragma unroll
         for (int i = 0; i < NQ; ++i) {
-            float tm = -INFINITY;
+            float d = -INFINITY;
 #pragma unroll
             for (int u = 0; u < 4; ++u)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) tm = fmaxf(tm, sacc[i][u][r]);
-            tm = col_max4(tm);
-            const float mn = fmaxf(m[i], tm);                   // finite from the first tile on: key 0 is visible to every row
-            if (__builtin_amdgcn_ballot_w64(mn > m[i]) != 0) {
-                const float al = __builtin_amdgcn_exp2f(m[i] - mn);     // exp2(-inf) = 0 on the first tile
+                for (int r = 0; r < 4; ++r) {
+                    if constexpr (MASKED)
+                        if (kb + 32 * (u >> 1) + 8 * g + 4 * (u & 1) + r > qpos[i]) sacc[u][i][r] = -INFINITY;
+                    d = fmaxf(d, sacc[u][i][r]);
+                }
+            if constexpr (FIRST) {                     // key 0 is visible to every row: finite
+                d = col_max4(d);
+#pragma unroll
+                for (int u = 0; u < 4; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) sacc[u][i][r] -= d;
+                m_ref[i] = d;
+            } else if (__any(d > MLA_THR)) {
+                const float dr = col_max4(d), dd = dr > MLA_THR ? dr : 0.f;
+                const float al = __builtin_amdgcn_exp2f(-dd);
+#pragma unroll
+                for (int u = 0; u < 4; ++u)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) sacc[u][i][r] -= dd;
                 lacc[i] *= al;
 #pragma unroll
-                for (int d = 0; d < DT; ++d) oacc[i][d] *= al;
-                m[i] = mn;
+                for (int e = 0; e < DT; ++e) oacc[e][i] *= al;
+                m_ref[i] += dd;
             }
 #pragma unroll
-            for (int c = 0; c < 2; ++c) {
+            for (int u = 0; u < 2; ++u) {
                 u32x4 w;
 #pragma unroll
-                for (int e2 = 0; e2 < 4; ++e2) {
-                    const int e = 2 * e2;
-                    w[e2] = pack_bf2(__builtin_amdgcn_exp2f(sacc[i][2 * c + (e >> 2)][e & 3] - m[i]),
-                                     __builtin_amdgcn_exp2f(sacc[i][2 * c + ((e + 1) >> 2)][(e + 1) & 3] - m[i]));
-                }
-                pf[i][c] = __builtin_bit_cast(bf16x8, w);
+                for (int e = 0; e < 4; ++e)
+                    w[e] = pack_bf2(__builtin_amdgcn_exp2f(sacc[2 * u + (e >> 1)][i][2 * (e & 1)]),
+                                    __builtin_amdgcn_exp2f(sacc[2 * u + (e >> 1)][i][2 * (e & 1) + 1]));
+                pf[u][i] = __builtin_bit_cast(bf16x8, w);
             }
         }
+        __builtin_amdgcn_s_setprio(0);
 #pragma unroll
-        for (int c = 0; c < 2; ++c)
+        for (int u = 0; u < 2; ++u)
 #pragma unroll
-            for (int i = 0; i < NQ; ++i) lacc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[i][c], lacc[i], 0, 0, 0);
+            for (int i = 0; i < NQ; ++i) lacc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[u][i], lacc[i], 0, 0, 0);
 #pragma unroll
-        for (int d = 0; d < DT; ++d) {
-            if (d >= dt) break;
+        for (int d = 0; d < DT; ++d)
 #pragma unroll
-            for (int c = 0; c < 2; ++c) {
-                const char* va = Vs + v_rd + 32 * c * VRS + 32 * d;
+            for (int u = 0; u < 2; ++u) {
+                const char* va = Vs + u * 32 * (DT * 32) + v_base + ((d ^ v_sw) << 5);
                 const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va));
-                const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va + 16 * VRS));
+                const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va + 4 * (DT * 32)));
                 const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
                 const bf16x8 vf = __builtin_bit_cast(bf16x8, u32x4{l2[0], l2[1], h2[0], h2[1]});
 #pragma unroll
-                for (int i = 0; i < NQ; ++i) oacc[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[i][c], oacc[i][d], 0, 0, 0);
+                for (int i = 0; i < NQ; ++i) oacc[d][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u][i], oacc[d][i], 0, 0, 0);
             }
+        if constexpr (!MASKED && DT >= 4) {            // 4 DT transposing reads, 4 + 4 DT MFMAs: eight reads lead
+            __builtin_amdgcn_sched_group_barrier(0x100, 8, 0);
+            __builtin_amdgcn_sched_group_barrier(0x008, 4, 0);
+#pragma unroll
+            for (int i = 0; i < DT - 2; ++i) {
+                __builtin_amdgcn_sched_group_barrier(0x008, 4, 0);
+                __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
+            }
+            __builtin_amdgcn_sched_group_barrier(0x008, 8, 0);
         }
+    };
+
+    // tiles [0, t_mid) lie left of the diagonal of every row
+    const int t_mid = min((s.pos0 + q0 + 1) >> 6, nt);
+    issue_tile(0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+#pragma unroll
+    for (int i = 0; i < NQ; ++i)
+#pragma unroll
+        for (int k = 0; k < KS; ++k) asm volatile("" : "+v"(qf[i][k]));          // Q loads complete before the loop
+    __builtin_amdgcn_s_barrier();
+    auto tile_tail = [&] {
+        // the next tile has landed for this wave, behind the barrier for every wave, and nobody reads this one any more
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+    };
+    if (1 < nt) issue_tile(1);
+    if (t_mid > 0) process_tile(0, std::false_type{}, std::true_type{});
+    else process_tile(0, std::true_type{}, std::true_type{});
+    tile_tail();
+    int t = 1;
+    for (; t < t_mid; ++t) {
+        if (t + 1 < nt) issue_tile(t + 1);
+        process_tile(t, std::false_type{}, std::false_type{});
+        tile_tail();
     }
-    const float sink = p.sink ? p.sink[h] : -INFINITY;
+    for (; t < nt; ++t) {
+        if (t + 1 < nt) issue_tile(t + 1);
+        process_tile(t, std::true_type{}, std::false_type{});
+        tile_tail();
+    }
+
+    const int dt = p.dv >> 4;
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
-        if (qrow[i] >= s.len) continue;
-        float f;
-        if (p.sink) {
-            const float M = fmaxf(m[i], sink), a = exp2f(m[i] - M);
-            f = a / (lacc[i][0] * a + exp2f(sink - M));
-        } else f = 1.f / lacc[i][0];
-        const long row = s.row0 + qrow[i];
+        const int qrow = q0 + wid * 32 + 16 * i + li;
+        if (qrow >= s.len) continue;
+        float f = 1.f / (lacc[i][0] + (p.sink ? exp2f(p.sink[h] - m_ref[i]) : 0.f));
+        const long row = s.row0 + qrow;
         if (p.gate) f *= p.gate[row * p.heads + h];
         bf16_t* O = reinterpret_cast<bf16_t*>(p.O) + row * p.ldo + (long)h * p.o_head + 4 * g;
 #pragma unroll
         for (int d = 0; d < DT; ++d)
-            if (d < dt) st4_f<bf16_t>(O + 16 * d, oacc[i][d] * f);
+            if (d < dt) st4_f<bf16_t>(O + 16 * d, oacc[d][i] * f);
     }
 }
 
 // ------------------------------------------------------------------------------------------------ decode attention (bf16)
-// One new row per sequence. Workgroup = (split of the keys, 16 heads, sequence). A tile of TK cache rows is one contiguous run in
-// memory; it goes through registers into LDS and is read twice there: as K rows (A operand of S^T = C.Q^T, wave w owns key block
-// w) and transposed as V (A operand of O^T = C^T.P^T, wave w owns the latent columns 16 (w + 4 i)). The weights travel between
-// the waves through LDS.
+// One new row per sequence. Workgroup = (split of the keys, 16 heads, sequence). A tile of 32 cache rows is one contiguous run in
+// memory; it goes through registers into LDS (the next tile's loads are in flight meanwhile) and is read twice there: as K rows
+// (A operand of S^T = C.Q^T; waves share the product as 2 key blocks x 2 halves of the row) and transposed as V (A operand of
+// O^T = C^T.P^T; wave w owns the latent columns 16 (w + 4 i)). The four partial score tiles meet in LDS in the accumulators' own
+// lane layout: every wave adds the halves of both blocks and has all 32 weights of its 16 query columns as the B operand.
 struct MlaDecodeArgs {
     const bf16_t* Q; long ldq; int q_head;
     const CogsSeq* seqs; long layer_off;
@@ -479,15 +605,14 @@ struct MlaDecodeArgs {
     float* part_o; float* part_ml;          // [seq][split][head][kvp] relative to part_ml[..][0]; [..][2] = (max, sum)
 };
 
-template <int TK, int DTW, int PER>
-__global__ __launch_bounds__(256) void mla_decode_kernel(MlaDecodeArgs p) {
+template <int DTW, int PER, int WGS>
+__global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
-    constexpr int PRS = TK * 2 + 16;
+    constexpr int TK = 32;
     const int RS = p.kvw * 2 + 32;                               // an odd multiple of 32 bytes (kvw % 32 == 0)
-    char* const Ks = smem;
+    f32x4* const Sx = reinterpret_cast<f32x4*>(smem);            // [key block][row half][lane]
+    char* const Ks = smem + 4 * 64 * 16;
     char* const Qs = Ks + TK * RS;
-    char* const Ps = Qs + 16 * RS;
-    float* const cmax = reinterpret_cast<float*>(Ps + 16 * PRS);   // [4][16]
 
     const int tid = threadIdx.x, lane = tid & 63;
     const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -517,32 +642,35 @@ __global__ __launch_bounds__(256) void mla_decode_kernel(MlaDecodeArgs p) {
         const char* base = cache + (long)t * TK * row_bytes;
         const int lim = min(TK, kend - t * TK) * nch - 1;           // chunks past the end repeat the last one (masked)
 #pragma unroll
-        for (int i = 0; i < PER; ++i) {
-            const int id = tid + 256 * i;
-            if (256 * i < tile_chunks) reg[i] = __builtin_nontemporal_load(reinterpret_cast<const u32x4*>(base + (long)min(id, lim) * 16));
-        }
+        for (int i = 0; i < PER; ++i)
+            reg[i] = *reinterpret_cast<const u32x4*>(base + min(tid + 256 * i, lim) * 16);
     };
     load_tile(t_begin);
-    for (int id = tid; id < 16 * nch; id += 256) {
-        const int r = id / nch, c = id - r * nch;
-        u32x4 v = {0, 0, 0, 0};
-        if (h0 + r < p.heads) v = *reinterpret_cast<const u32x4*>(p.Q + (long)b * p.ldq + (long)(h0 + r) * p.q_head + c * 8);
-        *reinterpret_cast<u32x4*>(Qs + r * RS + c * 16) = v;
-    }
     const int row_t = tid / nch, c_t = tid - row_t * nch;
-    const int ks = p.kvw >> 5, dts = p.kvp >> 4;
+    {
+        int r = row_t, c = c_t;
+#pragma unroll 1
+        while (r < 16) {
+            u32x4 v = {0, 0, 0, 0};
+            if (h0 + r < p.heads) v = *reinterpret_cast<const u32x4*>(p.Q + (long)b * p.ldq + (long)(h0 + r) * p.q_head + c * 8);
+            *reinterpret_cast<u32x4*>(Qs + r * RS + c * 16) = v;
+            r += dr_row; c += dr_c;
+            if (c >= nch) { c -= nch; ++r; }
+        }
+    }
+    const int ks = p.kvw >> 5, dts = p.kvp >> 4, kh = (ks + 1) >> 1;
+    const int k_lo = (wid >> 1) ? kh : 0, k_hi = (wid >> 1) ? ks : kh;
     f32x4 oacc[DTW], lacc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int d = 0; d < DTW; ++d) oacc[d] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m = -INFINITY;
-    const u32x4 ones_w = {0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u};
-    const bf16x8 ones = __builtin_bit_cast(bf16x8, ones_w);
+    const bf16x8 ones = __builtin_bit_cast(bf16x8, u32x4{0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u});
     const char* const qrd = Qs + li * RS + 16 * g;
-    const char* const krd = Ks + (16 * wid + li) * RS + 16 * g;
-    const char* const vrd = Ks + (4 * g + (li >> 2)) * RS + (li & 3) * 8;
+    const char* const krd = Ks + (16 * (wid & 1) + li) * RS + 16 * g;
+    const char* const vrd = Ks + (4 * g + (li >> 2)) * RS + (li & 3) * 8 + 32 * wid;
 
     for (int t = t_begin; t < t_end; ++t) {
-        if (t != t_begin) __syncthreads();                        // the previous tile's transposed reads are done
+        __syncthreads();                                          // the previous tile's transposed reads are done
         {
             int r = row_t, c = c_t;
 #pragma unroll
@@ -555,64 +683,59 @@ __global__ __launch_bounds__(256) void mla_decode_kernel(MlaDecodeArgs p) {
         __syncthreads();
         if (t + 1 < t_end) load_tile(t + 1);
         const int nvalid = min(TK, kend - t * TK);
-        f32x4 sa = {0.f, 0.f, 0.f, 0.f}, sb = sa;
-        if (16 * wid < TK) {
-            int k = 0;
-            for (; k + 1 < ks; k += 2) {
-                const u32x4 k0 = *reinterpret_cast<const u32x4*>(krd + 64 * k), q0 = *reinterpret_cast<const u32x4*>(qrd + 64 * k);
-                const u32x4 k1 = *reinterpret_cast<const u32x4*>(krd + 64 * k + 64), q1 = *reinterpret_cast<const u32x4*>(qrd + 64 * k + 64);
-                sa = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, k0), __builtin_bit_cast(bf16x8, q0), sa, 0, 0, 0);
-                sb = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, k1), __builtin_bit_cast(bf16x8, q1), sb, 0, 0, 0);
-            }
-            if (k < ks) {
-                const u32x4 k0 = *reinterpret_cast<const u32x4*>(krd + 64 * k), q0 = *reinterpret_cast<const u32x4*>(qrd + 64 * k);
-                sa = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, k0), __builtin_bit_cast(bf16x8, q0), sa, 0, 0, 0);
-            }
-            sa += sb;
-            float tm = -INFINITY;
+        {
+            f32x4 acc[4];
 #pragma unroll
-            for (int r = 0; r < 4; ++r) {
-                if (16 * wid + 4 * g + r >= nvalid) sa[r] = -INFINITY;
-                tm = fmaxf(tm, sa[r]);
+            for (int e = 0; e < 4; ++e) acc[e] = f32x4{0.f, 0.f, 0.f, 0.f};
+            int k = k_lo;
+#pragma unroll 1
+            for (; k + 3 < k_hi; k += 4) {
+                u32x4 kf[4], qv[4];
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    kf[e] = *reinterpret_cast<const u32x4*>(krd + 64 * (k + e));
+                    qv[e] = *reinterpret_cast<const u32x4*>(qrd + 64 * (k + e));
+                }
+#pragma unroll
+                for (int e = 0; e < 4; ++e)
+                    acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, kf[e]), __builtin_bit_cast(bf16x8, qv[e]), acc[e], 0, 0, 0);
             }
-            tm = col_max4(tm);
-            if (g == 0) cmax[wid * 16 + li] = tm;
+#pragma unroll 1
+            for (; k < k_hi; ++k)
+                acc[0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(krd + 64 * k)),
+                                                                 __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(qrd + 64 * k)), acc[0], 0, 0, 0);
+            Sx[((wid & 1) * 2 + (wid >> 1)) * 64 + lane] = (acc[0] + acc[1]) + (acc[2] + acc[3]);
         }
         __syncthreads();
-        float mn = fmaxf(m, fmaxf(cmax[li], cmax[16 + li]));
-        if constexpr (TK == 64) mn = fmaxf(mn, fmaxf(cmax[32 + li], cmax[48 + li]));
-        if (16 * wid < TK) {
-            u32x2 w;
-            w[0] = pack_bf2(__builtin_amdgcn_exp2f(sa[0] - mn), __builtin_amdgcn_exp2f(sa[1] - mn));
-            w[1] = pack_bf2(__builtin_amdgcn_exp2f(sa[2] - mn), __builtin_amdgcn_exp2f(sa[3] - mn));
-            *reinterpret_cast<u32x2*>(Ps + li * PRS + (16 * wid + 4 * g) * 2) = w;
+        f32x4 s0 = Sx[lane] + Sx[64 + lane], s1 = Sx[128 + lane] + Sx[192 + lane];
+        float tm = -INFINITY;
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            if (4 * g + r >= nvalid) s0[r] = -INFINITY;
+            if (16 + 4 * g + r >= nvalid) s1[r] = -INFINITY;
+            tm = fmaxf(tm, fmaxf(s0[r], s1[r]));
         }
+        const float mn = fmaxf(m, col_max4(tm));                  // finite: the tile's first key exists
         const float al = __builtin_amdgcn_exp2f(m - mn);          // 0 on the first tile
-        m = mn;
         lacc *= al;
 #pragma unroll
         for (int d = 0; d < DTW; ++d) oacc[d] *= al;
-        __syncthreads();
-        bf16x8 pf[TK / 32];
-#pragma unroll
-        for (int c = 0; c < TK / 32; ++c) {
-            const u32x2 lo = *reinterpret_cast<const u32x2*>(Ps + li * PRS + (32 * c + 4 * g) * 2);
-            const u32x2 hi = *reinterpret_cast<const u32x2*>(Ps + li * PRS + (32 * c + 16 + 4 * g) * 2);
-            pf[c] = __builtin_bit_cast(bf16x8, u32x4{lo[0], lo[1], hi[0], hi[1]});
-            lacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[c], lacc, 0, 0, 0);
-        }
+        m = mn;
+        u32x4 w;
+        w[0] = pack_bf2(__builtin_amdgcn_exp2f(s0[0] - mn), __builtin_amdgcn_exp2f(s0[1] - mn));
+        w[1] = pack_bf2(__builtin_amdgcn_exp2f(s0[2] - mn), __builtin_amdgcn_exp2f(s0[3] - mn));
+        w[2] = pack_bf2(__builtin_amdgcn_exp2f(s1[0] - mn), __builtin_amdgcn_exp2f(s1[1] - mn));
+        w[3] = pack_bf2(__builtin_amdgcn_exp2f(s1[2] - mn), __builtin_amdgcn_exp2f(s1[3] - mn));
+        const bf16x8 pf = __builtin_bit_cast(bf16x8, w);
+        lacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf, lacc, 0, 0, 0);
+        // (no branch for columns past kvp: such a read stays inside Ks + Qs, and its accumulator is not stored)
 #pragma unroll
         for (int d = 0; d < DTW; ++d) {
-            const int db = wid + 4 * d;
-            if (db >= dts) break;
-#pragma unroll
-            for (int c = 0; c < TK / 32; ++c) {
-                const char* va = vrd + 32 * c * RS + 32 * db;
-                const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va));
-                const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va + 16 * RS));
-                const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
-                oacc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, u32x4{l2[0], l2[1], h2[0], h2[1]}), pf[c], oacc[d], 0, 0, 0);
-            }
+            const char* va = vrd + 128 * d;
+            const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va));
+            const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va + 16 * RS));
+            const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
+            oacc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, u32x4{l2[0], l2[1], h2[0], h2[1]}), pf, oacc[d], 0, 0, 0);
         }
     }
     if (h0 + li < p.heads) {
@@ -626,8 +749,8 @@ __global__ __launch_bounds__(256) void mla_decode_kernel(MlaDecodeArgs p) {
     }
 }
 
-// splits of one (sequence, head) -> the head's weighted latent, bf16; 64 latent columns per workgroup
-constexpr int MLA_MAX_SPLIT = 128;
+// splits of one (sequence, head) -> the head's weighted latent, bf16; 64 latent columns per workgroup, wave w sums every fourth split
+constexpr int MLA_MAX_SPLIT = 256;
 __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit,
                                                           int heads, int kvp, const float* __restrict__ sink, bf16_t* __restrict__ out) {
     __shared__ float w_sh[MLA_MAX_SPLIT];
@@ -636,6 +759,13 @@ __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restric
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int h = blockIdx.x, b = blockIdx.y, d = blockIdx.z * 64 + lane;
     const long base = (long)b * nsplit * heads + h;
+    // the first 16 partial rows of this wave are requested before the weights are known (an empty split's row holds anything: its
+    // weight is tested, not multiplied)
+    const float* po = part_o + base * kvp + d;
+    const long stride = (long)heads * kvp;
+    float v[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) v[i] = po[(long)min(wid + 4 * i, nsplit - 1) * stride];
     float m = -INFINITY, l = 0.f;
     if (tid < nsplit) { m = part_ml[(base + (long)tid * heads) * 2]; l = part_ml[(base + (long)tid * heads) * 2 + 1]; }
     float M = wave_max(m);
@@ -645,14 +775,22 @@ __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restric
     const float sk = sink ? sink[h] : -INFINITY;
     M = fmaxf(M, sk);
     const float w = (m == -INFINITY) ? 0.f : exp2f(m - M);
-    if (tid < nsplit) w_sh[tid] = w;
+    w_sh[tid] = w;
     const float lw = wave_sum(l * w);
     __syncthreads();
     if (lane == 0) red[wid] = lw;
     float a = 0.f;
-    for (int s = wid; s < nsplit; s += 4) {
-        const float ws = w_sh[s];
-        if (ws != 0.f) a = fmaf(part_o[(base + (long)s * heads) * kvp + d], ws, a);     // (an empty split's row is not written)
+    for (int s0 = 0; s0 < nsplit; s0 += 64) {
+        if (s0) {
+#pragma unroll
+            for (int i = 0; i < 16; ++i) v[i] = po[(long)min(s0 + wid + 4 * i, nsplit - 1) * stride];
+        }
+#pragma unroll
+        for (int i = 0; i < 16; ++i) {
+            const int sp = s0 + wid + 4 * i;
+            const float ws = sp < nsplit ? w_sh[sp] : 0.f;
+            a += ws != 0.f ? v[i] * ws : 0.f;
+        }
     }
     acc_sh[wid][lane] = a;
     __syncthreads();
@@ -663,24 +801,25 @@ __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restric
     }
 }
 
-template <int KS, int DT, int NQ>
+template <int KN, int KR, int DT, int WGS>
 int launch_prefill(hipStream_t st, const CogsMla& a) {
     static std::atomic<uint64_t> attr_done{0};
-    constexpr int lds = 64 * (KS * 64) + 64 * (DT * 32 + 32);
-    cogs_ensure_dyn_lds((const void*)mla_prefill_kernel<KS, DT, NQ>, lds, attr_done);
-    const int nqt = (a.max_new + 64 * NQ - 1) / (64 * NQ);
+    constexpr int lds = 2 * (64 * KN * 64 + 64 * KR * 64 + 64 * DT * 32);
+    cogs_ensure_dyn_lds((const void*)mla_prefill_kernel<KN, KR, DT, WGS>, lds, attr_done);
+    const int nqt = (a.max_new + 127) / 128;
     const long grid = (long)nqt * a.heads * a.nseq;
     if (grid > 0x7fffffffL) return COGS_E_INVALID;
-    hipLaunchKernelGGL((mla_prefill_kernel<KS, DT, NQ>), dim3((unsigned)grid), dim3(256), lds, st, a, nqt);
+    const int group = nqt >= 64 ? 1 : 64 / nqt;
+    hipLaunchKernelGGL((mla_prefill_kernel<KN, KR, DT, WGS>), dim3((unsigned)grid), dim3(256), lds, st, a, nqt, group);
     return COGS_LAUNCH_CHECK();
 }
 
-template <int TK, int DTW, int PER>
+template <int DTW, int PER, int WGS>
 int launch_decode(hipStream_t st, const MlaDecodeArgs& p, int nseq) {
     static std::atomic<uint64_t> attr_done{0};
-    const int lds = (TK + 16) * (p.kvw * 2 + 32) + 16 * (TK * 2 + 16) + 64 * 4;
-    cogs_ensure_dyn_lds((const void*)mla_decode_kernel<TK, DTW, PER>, 160 * 1024, attr_done);
-    hipLaunchKernelGGL((mla_decode_kernel<TK, DTW, PER>), dim3((unsigned)((p.nsplit + 7) / 8 * 8 * p.nht), nseq), dim3(256), lds, st, p);
+    const int lds = 48 * (p.kvw * 2 + 32) + 4 * 64 * 16;
+    cogs_ensure_dyn_lds((const void*)mla_decode_kernel<DTW, PER, WGS>, 160 * 1024, attr_done);
+    hipLaunchKernelGGL((mla_decode_kernel<DTW, PER, WGS>), dim3((unsigned)((p.nsplit + 7) / 8 * 8 * p.nht), nseq), dim3(256), lds, st, p);
     return COGS_LAUNCH_CHECK();
 }
 
@@ -718,7 +857,8 @@ int cogs_k_head_gemm(hipStream_t st, int dtype, const CogsHeadGemm& a) {
     if (dtype == COGS_DT_BF16) {
         if (a.N % 16 || a.K % 32 || a.ldxb % 8 || a.ldxh % 8 || a.ldyb % 4 || a.ldyh % 4) return COGS_E_INVALID;
         const int nt = (a.N + a.tail + 15) / 16;
-        hipLaunchKernelGGL(head_gemm_bf16_kernel, dim3((nt + 3) / 4, a.heads, (a.B + 15) / 16), dim3(256), 0, st, p);
+        if (a.K >= 256) hipLaunchKernelGGL(head_gemm_bf16_kernel<true>, dim3(nt, a.heads, (a.B + 15) / 16), dim3(256), 0, st, p);
+        else hipLaunchKernelGGL(head_gemm_bf16_kernel<false>, dim3((nt + 3) / 4, a.heads, (a.B + 15) / 16), dim3(256), 0, st, p);
     } else {
         hipLaunchKernelGGL(head_gemm_f32_kernel, dim3((a.N + a.tail + 3) / 4, a.heads, a.B), dim3(256), 0, st, p);
     }
@@ -730,16 +870,16 @@ int cogs_k_mla_attention(hipStream_t st, int dtype, const CogsMla& a) {
     if (a.rows <= 0 || a.nseq <= 0 || a.heads <= 0 || a.dn % 4 || a.dr % 4 || a.dv <= 0) return COGS_E_INVALID;
     const int es = dtype == COGS_DT_BF16 ? 2 : 4;
     if ((a.ldk * es) % 8 || (a.ldkr * es) % 8 || (a.ldv * es) % 8) return COGS_E_INVALID;
-    if (dtype == COGS_DT_BF16 && !a.absorbed && a.dn % 8 == 0 && a.dr % 8 == 0 && a.dv % 16 == 0 && a.ldq % 8 == 0 && a.q_head % 8 == 0 &&
-        a.q_head >= (a.dn + a.dr + 31) / 32 * 32 && a.ldk % 8 == 0 && a.k_head % 8 == 0 && a.ldkr % 8 == 0 && a.ldv % 8 == 0 &&
-        a.v_head % 8 == 0 && a.ldo % 4 == 0 && a.o_head % 4 == 0 && g_cogs_debug.mla_rowwise == 0) {
-        const int ks = (a.dn + a.dr + 31) / 32, dt = a.dv / 16;
-        if (ks <= 2 && dt <= 4) return launch_prefill<2, 4, 2>(st, a);
-        if (ks <= 4 && dt <= 4) return launch_prefill<4, 4, 2>(st, a);
-        if (ks <= 4 && dt <= 8) return launch_prefill<4, 8, 2>(st, a);
-        if (ks <= 6 && dt <= 8) return launch_prefill<6, 8, 2>(st, a);
-        if (ks <= 8 && dt <= 8) return launch_prefill<8, 8, 2>(st, a);
-        if (ks <= 8 && dt <= 16) return launch_prefill<8, 16, 1>(st, a);
+    if (dtype == COGS_DT_BF16 && !a.absorbed && a.dn % 8 == 0 && a.dr % 8 == 0 && a.dv % 16 == 0 && a.ldq % 8 == 0 && a.q_head % 32 == 0 &&
+        a.q_rot % 32 == 0 && a.q_rot >= a.dn && a.q_head - a.q_rot >= a.dr && a.ldk % 8 == 0 && a.k_head % 8 == 0 && a.ldkr % 8 == 0 &&
+        a.ldv % 8 == 0 && a.v_head % 8 == 0 && a.ldo % 4 == 0 && a.o_head % 4 == 0 && g_cogs_debug.mla_rowwise == 0 &&
+        a.ldk < (1 << 23) && a.ldkr < (1 << 23) && a.ldv < (1 << 23)) {       // (a tile's byte offsets are 32 bits)
+        const int kn = a.q_rot / 32, kr = (a.q_head - a.q_rot) / 32, dt = a.dv / 16;
+        if (kn <= 1 && kr <= 1 && dt <= 2) return launch_prefill<1, 1, 2, 2>(st, a);
+        if (kn <= 2 && kr <= 1 && dt <= 4) return launch_prefill<2, 1, 4, 2>(st, a);
+        if (kn <= 4 && kr <= 1 && dt <= 8) return launch_prefill<4, 1, 8, 2>(st, a);
+        if (kn <= 4 && kr <= 2 && dt <= 8) return launch_prefill<4, 2, 8, 2>(st, a);
+        if (kn <= 8 && kr <= 4 && dt <= 16) return launch_prefill<8, 4, 16, 1>(st, a);
     }
     if (a.dn + a.dr > RW_DIM || a.dv > 64 * RW_VREG) return COGS_E_UNSUPPORTED;
     if (dtype == COGS_DT_BF16) hipLaunchKernelGGL(mla_rowwise_kernel<bf16_t>, dim3(a.rows, a.heads), dim3(64), 0, st, a);
@@ -748,8 +888,7 @@ int cogs_k_mla_attention(hipStream_t st, int dtype, const CogsMla& a) {
 }
 
 bool cogs_k_mla_decode_fits(int kvw, int kvp) {
-    return kvw % 32 == 0 && kvp % 16 == 0 && kvp <= 1024 && (32 + 16) * (kvw * 2 + 32) + 16 * (32 * 2 + 16) + 256 <= 160 * 1024 &&
-           32 * (kvw / 8) <= 256 * 18;
+    return kvw % 32 == 0 && kvp % 64 == 0 && kvp <= 1024 && 48 * (kvw * 2 + 32) + 4096 <= 160 * 1024 && 32 * (kvw / 8) <= 256 * 18;
 }
 
 int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx) {
@@ -758,8 +897,8 @@ int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx) {
     if (keys > 0) n = (max_ctx + keys - 1) / keys;
     else {
         const int nht = (heads + 15) / 16;
-        n = 512 / (nseq * nht);                           // about two workgroups per CU
-        const int tiles = (max_ctx + 63) / 64;
+        n = 512 / (nseq * nht);                           // two workgroups per CU
+        const int tiles = (max_ctx + 31) / 32;
         if (n > tiles) n = tiles;
     }
     if (n < 1) n = 1;
@@ -768,18 +907,18 @@ int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx) {
 
 // one new row per sequence, absorbed queries [seq][heads][kvw]; -> latent sums [seq][heads][kvp]
 int cogs_k_mla_decode(hipStream_t st, const CogsMlaDecode& a) {
-    if (a.nseq <= 0 || a.nseq > 65535 || a.nsplit < 1 || a.nsplit > MLA_MAX_SPLIT || !cogs_k_mla_decode_fits(a.kvw, a.kvp) || a.kvp % 64 ||
+    if (a.nseq <= 0 || a.nseq > 65535 || a.nsplit < 1 || a.nsplit > MLA_MAX_SPLIT || !cogs_k_mla_decode_fits(a.kvw, a.kvp) ||
         a.ldq % 8 || a.q_head % 8 || a.heads <= 0) return COGS_E_INVALID;
     MlaDecodeArgs p;
     p.Q = (const bf16_t*)a.Q; p.ldq = a.ldq; p.q_head = a.q_head; p.seqs = a.seqs; p.layer_off = a.layer_off;
     p.kvw = a.kvw; p.kvp = a.kvp; p.heads = a.heads; p.nht = (a.heads + 15) / 16; p.nsplit = a.nsplit;
     p.part_o = a.part; p.part_ml = a.part + (size_t)a.nseq * a.nsplit * a.heads * a.kvp;
-    const int dtw = (a.kvp / 16 + 3) / 4, ch64 = 64 * (a.kvw / 8);
+    const int dtw = (a.kvp / 16 + 3) / 4, chunks = 32 * (a.kvw / 8);
     int rc;
-    if (dtw <= 2 && ch64 <= 256 * 6) rc = launch_decode<64, 2, 6>(st, p, a.nseq);
-    else if (dtw <= 4 && ch64 <= 256 * 10) rc = launch_decode<64, 4, 10>(st, p, a.nseq);
-    else if (dtw <= 8 && ch64 <= 256 * 18) rc = launch_decode<64, 8, 18>(st, p, a.nseq);
-    else rc = launch_decode<32, 16, 18>(st, p, a.nseq);
+    if (dtw <= 2 && chunks <= 256 * 4) rc = launch_decode<2, 4, 4>(st, p, a.nseq);
+    else if (dtw <= 4 && chunks <= 256 * 6) rc = launch_decode<4, 6, 3>(st, p, a.nseq);
+    else if (dtw <= 8 && chunks <= 256 * 10) rc = launch_decode<8, 10, 2>(st, p, a.nseq);
+    else rc = launch_decode<16, 18, 1>(st, p, a.nseq);
     if (rc != COGS_OK) return rc;
     hipLaunchKernelGGL(mla_combine_kernel, dim3(a.heads, a.nseq, a.kvp / 64), dim3(256), 0, st, p.part_o, p.part_ml, a.nsplit, a.heads, a.kvp,
                        a.sink, (bf16_t*)a.out);

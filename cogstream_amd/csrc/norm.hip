@@ -203,11 +203,12 @@ __global__ __launch_bounds__(256) void ln_finalize_kernel(const float* __restric
     *reinterpret_cast<f32x2*>(ab + 2 * (long)r) = f32x2{rstd, (float)(-(double)rstd * mean)};
 }
 
-// fp32 residual stream around a sublayer (kernels.h, CogsStreamNorm): one 256-thread workgroup per row, the row in registers
-// (C chunks of four columns per thread). Norms entirely in fp32, one rounding of the normed row.
-template <typename T, int C>
-__global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
-    __shared__ float red[2][4];
+// fp32 residual stream around a sublayer (kernels.h, CogsStreamNorm): one workgroup of TPB threads per row, the row in
+// registers (C chunks of four columns per thread). Norms entirely in fp32, one rounding of the normed row.
+template <typename T, int C, int TPB>
+__global__ __launch_bounds__(TPB) void stream_norm_kernel(CogsStreamNorm p) {
+    constexpr int NW = TPB / 64;
+    __shared__ float red[2][NW];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const long row = p.pick ? p.pick[blockIdx.x] : blockIdx.x;
     float* x = p.x + row * p.Hp;
@@ -215,13 +216,15 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
         ss = wave_sum(ss);
         if (lane == 0) red[which][wid] = ss;
         __syncthreads();
-        ss = (red[which][0] + red[which][1]) + (red[which][2] + red[which][3]);
+        ss = red[which][0];
+#pragma unroll
+        for (int w = 1; w < NW; ++w) ss += red[which][w];
         return 1.f / sqrtf(ss / (float)p.H + p.eps);
     };
     f32x4 v[C];
 #pragma unroll
     for (int c = 0; c < C; ++c) {
-        const int i = tid * 4 + 1024 * c;
+        const int i = (tid + TPB * c) * 4;
         v[c] = f32x4{0.f, 0.f, 0.f, 0.f};
         if (i < p.Hp) v[c] = p.embeds ? ld4_f<T>(reinterpret_cast<const T*>(p.embeds) + row * p.Hp + i) : *reinterpret_cast<const f32x4*>(x + i);
     }
@@ -230,7 +233,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
         float ss = 0.f;
 #pragma unroll
         for (int c = 0; c < C; ++c) {
-            const int i = tid * 4 + 1024 * c;
+            const int i = (tid + TPB * c) * 4;
             y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
             if (i < p.Hp) y[c] = ld4_f<T>(reinterpret_cast<const T*>(p.y) + row * p.Hp + i);
 #pragma unroll
@@ -240,7 +243,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
             const float rs = row_rstd(ss, 0);
 #pragma unroll
             for (int c = 0; c < C; ++c) {
-                const int i = tid * 4 + 1024 * c;
+                const int i = (tid + TPB * c) * 4;
                 if (i >= p.Hp) continue;
                 const f32x4 g = *reinterpret_cast<const f32x4*>(p.y_gamma + i);
 #pragma unroll
@@ -253,7 +256,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
     if (p.y || p.embeds) {
 #pragma unroll
         for (int c = 0; c < C; ++c) {
-            const int i = tid * 4 + 1024 * c;
+            const int i = (tid + TPB * c) * 4;
             if (i < p.Hp) *reinterpret_cast<f32x4*>(x + i) = v[c];
         }
     }
@@ -267,7 +270,7 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
     T* o = reinterpret_cast<T*>(p.out) + (long)blockIdx.x * p.Hp;
 #pragma unroll
     for (int c = 0; c < C; ++c) {
-        const int i = tid * 4 + 1024 * c;
+        const int i = (tid + TPB * c) * 4;
         if (i >= p.Hp) continue;
         const f32x4 g = *reinterpret_cast<const f32x4*>(p.out_gamma + i);
         st4_f<T>(o + i, f32x4{v[c][0] * rs * g[0], v[c][1] * rs * g[1], v[c][2] * rs * g[2], v[c][3] * rs * g[3]});
@@ -276,13 +279,20 @@ __global__ __launch_bounds__(256) void stream_norm_kernel(CogsStreamNorm p) {
 
 template <typename T>
 int launch_stream_norm(hipStream_t st, const CogsStreamNorm& a) {
-    const dim3 grid(a.rows), blk(256);
-    if (a.Hp <= 1024) hipLaunchKernelGGL((stream_norm_kernel<T, 1>), grid, blk, 0, st, a);
-    else if (a.Hp <= 2048) hipLaunchKernelGGL((stream_norm_kernel<T, 2>), grid, blk, 0, st, a);
-    else if (a.Hp <= 4096) hipLaunchKernelGGL((stream_norm_kernel<T, 4>), grid, blk, 0, st, a);
-    else if (a.Hp <= 8192) hipLaunchKernelGGL((stream_norm_kernel<T, 8>), grid, blk, 0, st, a);
-    else if (a.Hp <= 16384) hipLaunchKernelGGL((stream_norm_kernel<T, 16>), grid, blk, 0, st, a);
+    const dim3 grid(a.rows);
+#define COGS_STREAM(C, TPB) hipLaunchKernelGGL((stream_norm_kernel<T, C, TPB>), grid, dim3(TPB), 0, st, a)
+    if (a.rows <= 64 && a.Hp > 1024) {           // few rows: latency, not bandwidth -- more threads on each
+        if (a.Hp <= 4096) COGS_STREAM(1, 1024);
+        else if (a.Hp <= 8192) COGS_STREAM(2, 1024);
+        else if (a.Hp <= 16384) COGS_STREAM(4, 1024);
+        else return COGS_E_UNSUPPORTED;
+    } else if (a.Hp <= 1024) COGS_STREAM(1, 256);
+    else if (a.Hp <= 2048) COGS_STREAM(2, 256);
+    else if (a.Hp <= 4096) COGS_STREAM(4, 256);
+    else if (a.Hp <= 8192) COGS_STREAM(8, 256);
+    else if (a.Hp <= 16384) COGS_STREAM(16, 256);
     else return COGS_E_UNSUPPORTED;
+#undef COGS_STREAM
     return COGS_LAUNCH_CHECK();
 }
 

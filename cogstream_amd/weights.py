@@ -402,8 +402,8 @@ class PackedDecoder:
                 raise ValueError(f"layer {i}: rotation over {m.rot.dims} dimensions, rotated part of {m.rot_dim}")
             a = p + "mix."
             qrp, kvp, rotc, hp = _up(m.q_rank, 64), _up(m.kv_rank, 64), _up(m.rot_dim, 32), _up(m.heads, 4)
-            dn, dr, dk, dv = _up(m.dim, 8), _up(m.rot_dim, 8), _up(m.dim, 32), _up(m.vdim, 16)
-            dq = _up(dn + dr, 32)
+            dn, dk, dv = _up(m.dim, 8), _up(m.dim, 32), _up(m.vdim, 16)
+            dq = dk + rotc
             order = m.rot.pair_order().to(self.device)
             lay.norm1 = vec(p + "norm1", Wp)
             if lc.post_norm:
@@ -427,7 +427,7 @@ class PackedDecoder:
             uq = g(a + "uq").view(m.heads, m.dim + m.rot_dim, m.q_rank)
             q = uq.new_zeros(m.heads, dq, qrp)
             q[:, :m.dim, :m.q_rank] = uq[:, :m.dim]
-            q[:, dn:dn + m.rot_dim, :m.q_rank] = uq[:, m.dim:][:, order]
+            q[:, dk:dk + m.rot_dim, :m.q_rank] = uq[:, m.dim:][:, order]
             x.q_w = hold(q.view(m.heads * dq, qrp)).data_ptr()
             uk = g(a + "uk").view(m.heads, m.dim, m.kv_rank)
             uv = g(a + "uv").view(m.heads, m.vdim, m.kv_rank)

@@ -433,7 +433,7 @@ cogs_status cogs_llm_forward_segments(cogs_handle h, cogs_stream stream, const v
  *
  * Padding (zeros, in weights, embeddings and norm vectors): width_p = width and ff_p = ff to a multiple of 64, vocab_p to 4;
  * q_rank_p and kv_rank_p to 64; rot_c = rot_dim to 32 (its columns in the cache); dim_p = dim and rot_p = rot_dim to 8;
- * dq = dim_p + rot_p to 32; vdim_p = vdim to 16; o_in = heads * vdim_p to 64; heads_p = heads to 4. dim_k = dim to 32.
+ * dim_k = dim to 32; dq = dim_k + rot_c; vdim_p = vdim to 16; o_in = heads * vdim_p to 64; heads_p = heads to 4.
  * Norm vectors are fp32; everything else is in `dtype`.
  *
  * cogs_latent_mixer: multi-head latent attention. Per token a row [latent (kv_rank_p) | rotated key part (rot_c)] is cached;
@@ -441,7 +441,7 @@ cogs_status cogs_llm_forward_segments(cogs_handle h, cogs_stream stream, const v
  * whatever pairs the model rotates (the packer permutes the rows of q_w and in_w alike).
  *   in_w   [q_rank_p | kv_rank_p | rot_c | heads_p][width_p]: query latent, kv latent, rotated key part (the middle two absent
  *          with kv_from >= 0), gate logits (absent unless gated), stacked in this order
- *   q_w    [heads][dim_p | rot_p | 0 .. dq][q_rank_p]
+ *   q_w    [heads][dim_k | rot_c][q_rank_p]
  *   kv_w   [heads * dim_p | heads * vdim_p][kv_rank_p]: keys, then values, head by head
  *   k_abs  [heads][kv_rank_p][dim_k]: the key rows of kv_w transposed per head
  *   o_w    [width_p][o_in]

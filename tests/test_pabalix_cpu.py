@@ -60,8 +60,8 @@ def test_packed_layouts_give_the_same_projections(name):
     for i, lay in enumerate(cfg["layers"]):
         m, x, pre = lay["mixer"], pk.layers[i].mixer, f"l{i}.mix."
         qrp, kvp, rc = up(m["q_rank"], 64), up(m["kv_rank"], 64), up(m["rot_dim"], 32)
-        dn, dr, dk, dv = up(m["dim"], 8), up(m["rot_dim"], 8), up(m["dim"], 32), up(m["vdim"], 16)
-        dq, H, own = up(dn + dr, 32), m["heads"], m.get("kv_from") is None
+        dn, dk, dv = up(m["dim"], 8), up(m["dim"], 32), up(m["vdim"], 16)
+        dq, H, own = dk + rc, m["heads"], m.get("kv_from") is None
         order = list(range(m["rot_dim"])) if lay["type"] == B else [j for i2 in range(m["rot_dim"] // 2) for j in (i2, i2 + m["rot_dim"] // 2)]
         rows = qrp + (kvp + rc if own else 0) + (up(H, 4) if lay["type"] == G else 0)
         t = hp @ _view(x.in_w, (rows, Wp), pk).T
@@ -80,8 +80,8 @@ def test_packed_layouts_give_the_same_projections(name):
         q = (cqp @ _view(x.q_w, (H * dq, qrp), pk).T).view(5, H, dq)
         want = (cq @ st[pre + "uq"].T).view(5, H, -1)
         assert torch.allclose(q[..., :m["dim"]], want[..., :m["dim"]], atol=1e-5)
-        assert torch.allclose(q[..., dn:dn + m["rot_dim"]], want[..., m["dim"]:][..., order], atol=1e-5)
-        assert not q[..., m["dim"]:dn].any() and not q[..., dn + m["rot_dim"]:].any()
+        assert torch.allclose(q[..., dk:dk + m["rot_dim"]], want[..., m["dim"]:][..., order], atol=1e-5)
+        assert not q[..., m["dim"]:dk].any() and not q[..., dk + m["rot_dim"]:].any()
         kv = cp @ _view(x.kv_w, (H * (dn + dv), kvp), pk).T
         k, v = (c @ st[pre + "uk"].T).view(5, H, -1), (c @ st[pre + "uv"].T).view(5, H, -1)
         assert torch.allclose(kv[:, :H * dn].view(5, H, dn)[..., :m["dim"]], k, atol=1e-5)
