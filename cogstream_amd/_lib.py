@@ -5,6 +5,8 @@ from __future__ import annotations
 import ctypes as C
 from pathlib import Path
 
+import torch  # noqa: F401  -- first: the library must bind to the HIP runtime torch loads, not bring a second one into the process
+
 _HERE = Path(__file__).resolve().parent
 import os as _os
 
