@@ -34,6 +34,12 @@ __device__ __forceinline__ float col_max4(float x) {      // over the lanes {li,
     return fmaxf(__builtin_bit_cast(float, (unsigned)b[0]), __builtin_bit_cast(float, (unsigned)b[1]));
 }
 
+// two softmax weights as MFMA operands: bf16 head and bf16 remainder (together 16 significant bits), packed lower half first
+__device__ __forceinline__ void split_weights(float p0, float p1, uint32_t& hi, uint32_t& lo) {
+    hi = pack_bf2(p0, p1);
+    lo = pack_bf2(p0 - bf_lo(hi), p1 - bf_hi(hi));
+}
+
 // sums of up to two values over a 256-thread workgroup, result in every thread; `red` holds 8 floats
 __device__ __forceinline__ void block_sum2(float& a, float& b, float* red) {
     const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
@@ -289,8 +295,9 @@ __global__ __launch_bounds__(64) void mla_rowwise_kernel(CogsMla p) {
 // 32-dimension steps. LDS-DMA writes lane-linear images: the bank swizzles live on the source address.
 //   scores transposed, S^T = K.Q^T, key rows permuted so that a lane's registers of blocks 2u, 2u+1 are the B operand of the
 //   u-th 32-key step of O^T = V^T.P^T; the accumulator starts at minus the running reference, so P = exp2(acc); the reference
-//   moves only when a score passes it by 2^THR (the sums stay far inside fp32, bf16 keeps its relative precision);
-//   the softmax sum is one more MFMA per step with an all-ones A operand, i.e. the sum of the bf16 weights that multiply V.
+//   moves only when a score passes it by 2^THR (the sums stay far inside fp32);
+//   a weight enters the products as two bf16 terms, head and remainder, so that it is not rounded to 16 bits on its way to V;
+//   the softmax sum is one more MFMA per step with an all-ones A operand, i.e. the sum of exactly the weights that multiply V.
 // Columns past dn / dr / dv hold copies of real data: the query's are zero, and value tiles past dv are not stored.
 constexpr float MLA_THR = 6.f;
 
@@ -477,7 +484,7 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
             __builtin_amdgcn_sched_group_barrier(0x008, 12, 0);
         }
         __builtin_amdgcn_s_setprio(1);
-        bf16x8 pf[2][NQ];
+        bf16x8 pf[2][NQ][2];                           // [32-key step][row group][head, remainder]
 #pragma unroll
         for (int i = 0; i < NQ; ++i) {
             float d = -INFINITY;
@@ -510,19 +517,25 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
             }
 #pragma unroll
             for (int u = 0; u < 2; ++u) {
-                u32x4 w;
+                u32x4 w, x;
 #pragma unroll
-                for (int e = 0; e < 4; ++e)
-                    w[e] = pack_bf2(__builtin_amdgcn_exp2f(sacc[2 * u + (e >> 1)][i][2 * (e & 1)]),
-                                    __builtin_amdgcn_exp2f(sacc[2 * u + (e >> 1)][i][2 * (e & 1) + 1]));
-                pf[u][i] = __builtin_bit_cast(bf16x8, w);
+                for (int e = 0; e < 4; ++e) {
+                    uint32_t hi, lo;
+                    split_weights(__builtin_amdgcn_exp2f(sacc[2 * u + (e >> 1)][i][2 * (e & 1)]),
+                                  __builtin_amdgcn_exp2f(sacc[2 * u + (e >> 1)][i][2 * (e & 1) + 1]), hi, lo);
+                    w[e] = hi; x[e] = lo;
+                }
+                pf[u][i][0] = __builtin_bit_cast(bf16x8, w);
+                pf[u][i][1] = __builtin_bit_cast(bf16x8, x);
             }
         }
         __builtin_amdgcn_s_setprio(0);
 #pragma unroll
         for (int u = 0; u < 2; ++u)
 #pragma unroll
-            for (int i = 0; i < NQ; ++i) lacc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[u][i], lacc[i], 0, 0, 0);
+            for (int i = 0; i < NQ; ++i)
+#pragma unroll
+                for (int x = 0; x < 2; ++x) lacc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf[u][i][x], lacc[i], 0, 0, 0);
 #pragma unroll
         for (int d = 0; d < DT; ++d)
 #pragma unroll
@@ -533,17 +546,19 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
                 const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
                 const bf16x8 vf = __builtin_bit_cast(bf16x8, u32x4{l2[0], l2[1], h2[0], h2[1]});
 #pragma unroll
-                for (int i = 0; i < NQ; ++i) oacc[d][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u][i], oacc[d][i], 0, 0, 0);
+                for (int x = 0; x < 2; ++x)
+#pragma unroll
+                    for (int i = 0; i < NQ; ++i) oacc[d][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pf[u][i][x], oacc[d][i], 0, 0, 0);
             }
-        if constexpr (!MASKED && DT >= 4) {            // 4 DT transposing reads, 4 + 4 DT MFMAs: eight reads lead
+        if constexpr (!MASKED && DT >= 4) {            // 4 DT transposing reads, 8 + 8 DT MFMAs: eight reads lead
             __builtin_amdgcn_sched_group_barrier(0x100, 8, 0);
-            __builtin_amdgcn_sched_group_barrier(0x008, 4, 0);
+            __builtin_amdgcn_sched_group_barrier(0x008, 8, 0);
 #pragma unroll
             for (int i = 0; i < DT - 2; ++i) {
-                __builtin_amdgcn_sched_group_barrier(0x008, 4, 0);
+                __builtin_amdgcn_sched_group_barrier(0x008, 8, 0);
                 __builtin_amdgcn_sched_group_barrier(0x100, 4, 0);
             }
-            __builtin_amdgcn_sched_group_barrier(0x008, 8, 0);
+            __builtin_amdgcn_sched_group_barrier(0x008, 16, 0);
         }
     };
 
@@ -721,13 +736,15 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
 #pragma unroll
         for (int d = 0; d < DTW; ++d) oacc[d] *= al;
         m = mn;
-        u32x4 w;
-        w[0] = pack_bf2(__builtin_amdgcn_exp2f(s0[0] - mn), __builtin_amdgcn_exp2f(s0[1] - mn));
-        w[1] = pack_bf2(__builtin_amdgcn_exp2f(s0[2] - mn), __builtin_amdgcn_exp2f(s0[3] - mn));
-        w[2] = pack_bf2(__builtin_amdgcn_exp2f(s1[0] - mn), __builtin_amdgcn_exp2f(s1[1] - mn));
-        w[3] = pack_bf2(__builtin_amdgcn_exp2f(s1[2] - mn), __builtin_amdgcn_exp2f(s1[3] - mn));
-        const bf16x8 pf = __builtin_bit_cast(bf16x8, w);
-        lacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pf, lacc, 0, 0, 0);
+        uint32_t w[4], x[4];                                      // head and remainder of the weights (see the prompt kernel)
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            split_weights(__builtin_amdgcn_exp2f(s0[2 * e] - mn), __builtin_amdgcn_exp2f(s0[2 * e + 1] - mn), w[e], x[e]);
+            split_weights(__builtin_amdgcn_exp2f(s1[2 * e] - mn), __builtin_amdgcn_exp2f(s1[2 * e + 1] - mn), w[2 + e], x[2 + e]);
+        }
+        const bf16x8 ph = __builtin_bit_cast(bf16x8, u32x4{w[0], w[1], w[2], w[3]}), pl = __builtin_bit_cast(bf16x8, u32x4{x[0], x[1], x[2], x[3]});
+        lacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, ph, lacc, 0, 0, 0);
+        lacc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(ones, pl, lacc, 0, 0, 0);
         // (no branch for columns past kvp: such a read stays inside Ks + Qs, and its accumulator is not stored)
 #pragma unroll
         for (int d = 0; d < DTW; ++d) {
@@ -735,7 +752,9 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
             const i16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va));
             const i16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((__attribute__((address_space(3))) i16x4*)(va + 16 * RS));
             const u32x2 l2 = __builtin_bit_cast(u32x2, lo), h2 = __builtin_bit_cast(u32x2, hi);
-            oacc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, u32x4{l2[0], l2[1], h2[0], h2[1]}), pf, oacc[d], 0, 0, 0);
+            const bf16x8 vf = __builtin_bit_cast(bf16x8, u32x4{l2[0], l2[1], h2[0], h2[1]});
+            oacc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph, oacc[d], 0, 0, 0);
+            oacc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, oacc[d], 0, 0, 0);
         }
     }
     if (h0 + li < p.heads) {
