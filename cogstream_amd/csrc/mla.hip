@@ -917,8 +917,8 @@ int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx) {
     else {
         const int nht = (heads + 15) / 16;
         n = 512 / (nseq * nht);                           // two workgroups per CU
-        const int tiles = (max_ctx + 31) / 32;
-        if (n > tiles) n = tiles;
+        const int most = (max_ctx + 63) / 64;             // shorter splits cost more in the combine than they save here
+        if (n > most) n = most;
     }
     if (n < 1) n = 1;
     return n > MLA_MAX_SPLIT ? MLA_MAX_SPLIT : n;

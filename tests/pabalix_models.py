@@ -37,7 +37,7 @@ CONFIGS = {
                      width=192, ff=128),
     "plain": config([mixer(A, heads=2), mixer(G, heads=2), dict(mixer(B, heads=2), ff=None)], width=64, vocab=96),     # no YaRN anywhere
     "one": config([mixer(A, heads=1, dim=8, rot=2, vdim=8, q_rank=8, kv_rank=8, scaling=YARN)], width=8, vocab=5, ff=4),
-    "same": config([mixer(k, heads=4, dim=32, rot=32, vdim=32, q_rank=64, kv_rank=64, scaling=None if k == B else (1.0, 2048, 32.0, 1.0)) for k in (A, B, G)],
+    "same": config([mixer(k, heads=4, dim=32, rot=32, vdim=32, q_rank=64, kv_rank=64, scaling=None if k == B else (1.0, 900, 25.0, 2.0)) for k in (A, B, G)],
                    width=64, vocab=128, ff=64),                                                                         # everything alike, a factor of 1
     "wide": config([mixer(G, heads=20, dim=128, rot=64, vdim=128, q_rank=192, kv_rank=512, scaling=YARN), mixer(B, heads=17, dim=64, rot=32, vdim=64, kv_rank=256)],
                    width=512, vocab=400, ff=320),

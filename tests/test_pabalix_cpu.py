@@ -23,10 +23,10 @@ def test_rotation_frequencies_match_the_oracle():
             f, mag = po.frequencies(lay["mixer"]["rot"])
             assert mine.mixer.rot.frequencies() == pytest.approx(f, rel=1e-14) and mine.mixer.rot.magnitude == pytest.approx(mag)
     # a pair inside the ramp, one on either side, and a ramp of no width
-    f, mag = po.frequencies(dict(dims=16, base=10000.0, scaling=dict(factor=4.0, original=2048, fast=32.0, slow=1.0)))
-    g = [10000.0 ** (-2 * i / 16) for i in range(8)]
+    f, mag = po.frequencies(dict(dims=20, base=5000.0, scaling=dict(factor=5.0, original=1000, fast=20.0, slow=1.5)))
+    g = [5000.0 ** (-2 * i / 20) for i in range(10)]
     r = [a / b for a, b in zip(f, g)]
-    assert r[0] == 1 and r[-1] == 0.25 and any(0.25 < x < 1 for x in r) and mag == pytest.approx(1 + 0.1 * math.log(4))
+    assert r[0] == 1 and r[-1] == pytest.approx(0.2) and any(0.21 < x < 0.99 for x in r) and mag == pytest.approx(1 + 0.1 * math.log(5))
     f, _ = po.frequencies(dict(dims=8, base=10.0, scaling=dict(factor=2.0, original=100000, fast=1e-9, slow=1e-9)))
     assert f == [10.0 ** (-2 * i / 8) for i in range(4)]
 
