@@ -125,18 +125,37 @@ class LatentMixer(C.Structure):
                 ("k_abs", c_void_p), ("sink", c_void_p), ("o_w", c_void_p)]
 
 
-class GatedMlp(C.Structure):
-    _fields_ = [("ff", c_int), ("gu_w", c_void_p), ("gu_b", c_void_p), ("down_w", c_void_p), ("down_b", c_void_p)]
+class AttnMixer(C.Structure):
+    _fields_ = [("heads", c_int), ("kv_heads", c_int), ("dim", c_int), ("vdim", c_int), ("qk_norm", c_int), ("scale", c_float),
+                ("temp_coef", C.c_double), ("temp_every", C.c_double), ("dist_bias", c_void_p), ("dist_n", c_int),
+                ("in_w", c_void_p), ("o_w", c_void_p)]
+
+
+class DeltaMixer(C.Structure):
+    _fields_ = [("heads", c_int), ("kv_heads", c_int), ("dim", c_int), ("vdim", c_int), ("taps", c_int), ("in_w", c_void_p),
+                ("conv", c_void_p), ("neg_a", c_void_p), ("dt_bias", c_void_p), ("norm", c_void_p), ("o_w", c_void_p)]
+
+
+class DecoderMlp(C.Structure):
+    _fields_ = [("ff", c_int), ("act", c_int), ("up_w", c_void_p), ("up_b", c_void_p), ("down_w", c_void_p), ("down_b", c_void_p)]
+
+
+class Hyper(C.Structure):
+    _fields_ = [("in_", c_void_p), ("out", c_void_p), ("mix", c_void_p)]
+
+
+MIX_LATENT, MIX_ATTENTION, MIX_DELTA = 0, 1, 2
 
 
 class DecoderLayer(C.Structure):
-    _fields_ = [("norm1", c_void_p), ("norm1b", c_void_p), ("norm2", c_void_p), ("norm2b", c_void_p),
-                ("mixer", LatentMixer), ("mlp", GatedMlp)]
+    _fields_ = [("norm1", c_void_p), ("norm1b", c_void_p), ("norm2", c_void_p), ("norm2b", c_void_p), ("hyper1", Hyper), ("hyper2", Hyper),
+                ("mixer", c_int), ("latent", LatentMixer), ("attn", AttnMixer), ("delta", DeltaMixer), ("mlp", DecoderMlp)]
 
 
 class DecoderWeights(C.Structure):
-    _fields_ = [("dtype", c_int), ("width", c_int), ("vocab", c_int), ("layers", c_int), ("eps", c_float),
-                ("final_norm", c_void_p), ("head", c_void_p), ("layer", C.POINTER(DecoderLayer))]
+    _fields_ = [("dtype", c_int), ("width", c_int), ("vocab", c_int), ("layers", c_int), ("eps", c_float), ("embed_scale", c_float),
+                ("pos", c_void_p), ("max_positions", c_int), ("streams", c_int), ("loop_start", c_int), ("loop_stop", c_int),
+                ("loop_times", c_int), ("final_norm", c_void_p), ("head", c_void_p), ("layer", C.POINTER(DecoderLayer))]
 
 
 # every symbol include/cogs.h declares: name -> (restype, argtypes)
@@ -204,6 +223,7 @@ SIGNATURES = {
                                  c_void_p, c_size_t]),
     "cogs_decoder_load": (c_int, [c_void_p, C.POINTER(DecoderWeights)]),
     "cogs_decoder_cache_width": (c_int, [c_void_p, C.POINTER(c_int64)]),
+    "cogs_decoder_state_bytes": (c_int, [c_void_p, C.POINTER(c_int64)]),
     "cogs_decoder_workspace_bytes": (c_int, [c_void_p, c_int, c_int, c_int64, c_int, C.POINTER(c_size_t)]),
     "cogs_decoder_forward": (c_int, [c_void_p, c_void_p, c_void_p, C.POINTER(C.POINTER(KV)), C.POINTER(C.c_int32), c_int,
                                      C.POINTER(C.c_int32), c_int, c_void_p, c_void_p, c_void_p, c_size_t]),

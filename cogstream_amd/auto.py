@@ -23,6 +23,7 @@ _DEFAULT_MODEL = "cogreasoner_chat.Videollama3Qwen2ForCausalLM"
 ARCHITECTURES = {
     "Videollama3Qwen2ForCausalLM": _DEFAULT_MODEL,
     "Pabalix": "pabalix.PabalixForCausalLM",
+    "Lupanex": "lupanex.LupanexForCausalLM",
 }
 _DEFAULT_PROCESSOR = "processing_cogreasoner.Videollama3Qwen2Processor"
 

@@ -228,6 +228,14 @@ def state_views(ckpt: Checkpoint, tie_word_embeddings: bool = False):
             StateView(ckpt, LLM_PREFIX, top_level=("lm_head.weight",), alias=alias, exclude=(VIT_PREFIX, PROJ_PREFIX)))
 
 
+def tensor_shapes(path: str) -> Dict[str, Tuple[int, ...]]:
+    """name -> shape of every tensor of a checkpoint directory, from the file headers"""
+    reader = Checkpoint(path)
+    out = {n: reader.shape(n) for n in reader.names()}
+    reader.close()
+    return out
+
+
 def open_decoder(path: str, cfg: DecoderConfig, device):
     """-> (state mapping for weights.PackedDecoder, the reader behind it): the tensors of a decoder described layer by layer,
     by the names and shapes its configuration implies"""

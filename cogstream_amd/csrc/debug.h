@@ -51,6 +51,7 @@
     X(mla_rowwise, 0, "1: latent attention always through the row-wise kernel")                                            \
     X(mla_absorb, 1, "0: steps of one token per sequence also expand keys and values instead of absorbing W_uk / W_uv")     \
     X(mla_split_keys, 0, "> 0: keys per split of the latent decode attention (0: chosen from the batch and the context)")   \
+    X(delta_chunk, 1, "0: gated delta rule of prompts token by token instead of in chunks")                                 \
     X(gemm_skinny, 1, "0: the decoder's few-row products through the general GEMM")                                         \
     X(km_row_groups, 0, "> 0: row groups of the k-means distance pass (0: sized to fill the chip)")
 

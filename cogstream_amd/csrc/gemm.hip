@@ -1088,6 +1088,7 @@ void dispatch_pp(hipStream_t st, const GemmArgs& p, int grid, int mask) {
         COGS_PP_CASE(EPI_ROPE)
         COGS_PP_CASE(EPI_SWIGLU)
         COGS_PP_CASE(EPI_SWIGLU | EPI_BIAS)
+        COGS_PP_CASE(EPI_GELU_ERF)
         COGS_PP_CASE(EPI_F32OUT)
         COGS_PP_CASE(EPI_NOSTORE)
         default: launch_pp<EPI_GENERIC>(st, p, grid); break;
@@ -1117,6 +1118,7 @@ void dispatch(hipStream_t st, const GemmArgs& p, int grid, int mask, bool big) {
         COGS_EPI_CASE(EPI_ROPE)
         COGS_EPI_CASE(EPI_SWIGLU)
         COGS_EPI_CASE(EPI_SWIGLU | EPI_BIAS)
+        COGS_EPI_CASE(EPI_GELU_ERF)
         COGS_EPI_CASE(EPI_F32OUT)
         default: if (big) launch_big<T, EPI_GENERIC>(st, p, grid); else launch_small<T, EPI_GENERIC>(st, p, grid); break;
     }

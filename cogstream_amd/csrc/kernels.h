@@ -167,6 +167,7 @@ int cogs_k_sample(hipStream_t st, const float* logits, int n, float temperature,
 // one sequence of a step; device table
 struct CogsSeq {
     char* cache;         // its cache: cached layers back to back, layer at (offset of the layer's first column) * max_len elements
+    float* state;        // its recurrent state, layer runs back to back
     long max_len;        // rows per cached layer
     int row0, len;       // its new rows are rows row0 .. row0 + len - 1 of the step
     int pos0;            // rows already cached
@@ -182,10 +183,15 @@ int cogs_k_rope_sets(hipStream_t st, float* table, const CogsRopeSet* sets_dev, 
 // fp32 residual stream x [rows][Hp] (H of the Hp columns are real, the rest zero):
 //   init: x = embeds, else x += y (y_gamma != null: x += RMSnorm(y) * y_gamma); then, out != null, out = RMSnorm(x) * out_gamma
 // y in `dtype`, gammas fp32 [Hp] (zero padded). pick (nullable, with out): only rows pick[i] are normed, into out row i, x untouched
+// embeds come scaled, plus the row of a position table (pos in `dtype` [..][Hp], rowpos). streams > 0: x is [rows][streams][Hp] with
+// hyper-connections: x_t = out_w[t] y + sum_s mix[s][t] x_s, all streams starting alike; what is normed is sum_s in_w[s] x_s
+// (in_w null: the sum of the streams), and sum (nullable) [rows][Hp] receives the sum of the streams
 struct CogsStreamNorm {
     float* x = nullptr; const void* embeds = nullptr; const void* y = nullptr; const float* y_gamma = nullptr;
     void* out = nullptr; const float* out_gamma = nullptr; const int* pick = nullptr;
     int rows = 0, H = 0, Hp = 0; float eps = 0.f;
+    float embed_scale = 1.f; const void* pos = nullptr; const int* rowpos = nullptr;
+    int streams = 0; const float *mix = nullptr, *out_w = nullptr, *in_w = nullptr; float* sum = nullptr;
 };
 int cogs_k_stream_norm(hipStream_t st, int dtype, const CogsStreamNorm& a);
 int cogs_k_zero(hipStream_t st, void* p, size_t bytes);      // 16-byte multiples
@@ -216,12 +222,42 @@ struct CogsMla {
     const float* gate;                           // [rows][heads], or null
     const CogsSeq* seqs; int nseq; const int* rowseq; int rows, max_new;
     int absorbed; long layer_off; int kr_col;
+    // kvw != 0: keys and values per head from the sequence's cache (K / KR / V unused): blocks [max_len][kvw] of heads / rep key / value
+    // heads from column layer_off on, rows [key | value from v_col]; ldk = ldv = kvw, dr = 0, q_rot = q_head
+    int kvw, v_col, rep;
+    const float* bias; int nb;                   // [heads][nb] in log2 units: entry min(n, nb - 1) for a key n back, or null
 };
 int cogs_k_mla_attention(hipStream_t st, int dtype, const CogsMla& a);
 struct CogsMlaDecode {
-    const void* Q; long ldq; int q_head; const CogsSeq* seqs; int nseq; long layer_off; int kvw, kvp, heads, nsplit;
-    const float* sink; float* part; void* out;   // part: nseq * nsplit * heads * (kvp + 2) floats; out [nseq][heads][kvp]
+    // cache rows of kvw columns: the first kcols meet the query, kvp from vcol on are summed; `rep` query heads read one block of
+    // rows (blocks of a sequence behind one another from column layer_off on)
+    const void* Q; long ldq; int q_head; const CogsSeq* seqs; int nseq; long layer_off; int kvw, kcols, vcol, kvp, heads, rep, nsplit;
+    const float* sink; float* part; void* out; long ldo; int o_head;     // part: nseq * nsplit * heads * (kvp + 2) floats
+    const float* bias; int nb;                   // as in CogsMla
 };
 bool cogs_k_mla_decode_fits(int kvw, int kvp);
 int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx);
 int cogs_k_mla_decode(hipStream_t st, const CogsMlaDecode& a);
+
+// softmax attention with per-head keys and values: head rows behind the fused projection (attn_heads.hip), attention by CogsMla /
+// CogsMlaDecode with kvw
+struct CogsAttnHeads {
+    const void* t; long ldt;             // [rows][q heads x dkp | k heads x dkp | v heads x dvp] in `dtype`
+    int heads, kv_heads, dim, dkp, dvp, kvw, norm; float eps, scale; double temp_coef, temp_every;
+    void* q;                             // [rows][heads][dkp], in log2 score units
+    const CogsSeq* seqs; const int* rowseq; const int* rowpos; long layer_off;
+};
+int cogs_k_attn_heads(hipStream_t st, int dtype, const CogsAttnHeads& a, int rows);
+
+// gated delta rule (delta.hip); all buffers fp32 but att
+struct CogsDelta {
+    const float* t; long ldt;            // fused projection [q | k | v | gate | beta | a]
+    int heads, headsp, kv_heads, dkp, dvp, vdim, taps, channels;
+    const float *conv, *neg_a, *dt_bias, *norm; float eps, q_scale;
+    float *q, *k, *v, *bg, *o, *rec;     // prompts: [rows][kv_heads][dkp] twice, [rows][heads][dvp], (beta, ln g), read-outs, chunk records
+    void* att; long ldo;                 // [rows][heads x dvp], in `dtype`
+    const CogsSeq* seqs; const int* rowseq; const int* rowpos; long state_off;      // floats
+};
+size_t cogs_k_delta_rec_floats(int rows, int nseq, int heads);
+int cogs_k_delta_prompt(hipStream_t st, int dtype, const CogsDelta& a, int rows, int nseq, int max_new);
+int cogs_k_delta_step(hipStream_t st, int dtype, const CogsDelta& a, int nseq);      // one new row per sequence, row i = sequence i

@@ -11,6 +11,11 @@
 //            are split over workgroups; mla_combine_kernel merges the splits).
 // A row-wise kernel (any size, bf16 or fp32) serves the fp32 mode and sizes the MFMA kernels have no instance for.
 //
+// The same kernels serve attention whose keys and values are cached per head (cogs_attn_mixer): a cache block per key / value head
+// with rows [key | value] takes the place of the latent rows, query heads share a block in groups, there is no shared rotated part,
+// and a learned bias per head and distance may be added to the scores. The bias is constant from some distance on, so only the key
+// tiles near the diagonal look it up; for the others it is part of the accumulators' start value.
+//
 // Scores are in log2 units everywhere (the query projection's epilogue multiplies by scale * log2 e before its rounding), so are
 // the optional per-head sinks: a sink joins the softmax sum with no key and no value. The optional per-head output gate
 // multiplies the finished head row.
@@ -225,7 +230,11 @@ __global__ __launch_bounds__(64) void mla_rowwise_kernel(CogsMla p) {
     for (int d = lane; d < p.dn + p.dr; d += 64) qs[d] = ld_f<T>(q + (d < p.dn ? d : p.q_rot + d - p.dn));
     __syncthreads();
     const T *K, *KR, *V;
-    if (p.absorbed) {
+    if (p.kvw) {
+        K = reinterpret_cast<const T*>(s.cache) + (p.layer_off + (long)(h / p.rep) * p.kvw) * s.max_len;
+        V = K + p.v_col;
+        KR = K;
+    } else if (p.absorbed) {
         K = V = reinterpret_cast<const T*>(s.cache) + p.layer_off * s.max_len;
         KR = K + p.kr_col;
     } else {
@@ -247,7 +256,8 @@ __global__ __launch_bounds__(64) void mla_rowwise_kernel(CogsMla p) {
 #pragma unroll
             for (int e = 0; e < 4; ++e) a[e] = fmaf(kv[e], qv[e], a[e]);
         }
-        return (a[0] + a[1]) + (a[2] + a[3]);
+        const float sc = (a[0] + a[1]) + (a[2] + a[3]);
+        return p.bias ? sc + p.bias[(long)h * p.nb + min(nkeys - 1 - j, p.nb - 1)] : sc;
     };
     float m = -INFINITY, l = 0.f;
     for (int j = lane; j < nkeys; j += 64) {
@@ -299,7 +309,11 @@ __global__ __launch_bounds__(64) void mla_rowwise_kernel(CogsMla p) {
 //   a weight enters the products as two bf16 terms, head and remainder, so that it is not rounded to 16 bits on its way to V;
 //   the softmax sum is one more MFMA per step with an all-ones A operand, i.e. the sum of exactly the weights that multiply V.
 // Columns past dn / dr / dv hold copies of real data: the query's are zero, and value tiles past dv are not stored.
+// KR = 0: keys and values per head from the cache (rows [key | value] of block h / rep), with the optional distance bias. Distances a
+// tile spans are a window of 191 entries, staged in LDS one tile ahead; a tile whose distances are all past the table's end takes
+// the last entry with the accumulators' start value.
 constexpr float MLA_THR = 6.f;
+constexpr int MLA_WIN = 192;             // floats of a bias window
 
 // 16-byte-chunk XOR of row `row` for rows of `chunks` chunks: 16 rows {8 a + b (+ 4 c)} of a fragment read land in different banks
 template <int CHUNKS> __device__ __forceinline__ int mla_kswz(int row) {
@@ -318,6 +332,7 @@ template <int DT> __device__ __forceinline__ int mla_vswz(int row) {
 template <int KN, int KR, int DT, int WGS>
 __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nqt, int group) {
     constexpr int NQ = 2, KS = KN + KR;
+    constexpr bool HEADS = KR == 0;
     constexpr int N_LDS = 64 * KN * 64, R_LDS = 64 * KR * 64, V_LDS = 64 * DT * 32, BUF = N_LDS + R_LDS + V_LDS;
     constexpr int PV = DT / 2;                    // V pieces per wave (K: KN and KR)
     static_assert(DT % 2 == 0, "whole pieces per wave");
@@ -346,9 +361,15 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
     if (q0 >= s.len) return;
 
     const bf16_t* Q = reinterpret_cast<const bf16_t*>(p.Q) + (long)s.row0 * p.ldq + (long)h * p.q_head;
-    const bf16_t* K = reinterpret_cast<const bf16_t*>(p.K) + (long)s.ctx0 * p.ldk + (long)h * p.k_head;
-    const bf16_t* KRp = reinterpret_cast<const bf16_t*>(p.KR) + (long)s.ctx0 * p.ldkr;
-    const bf16_t* V = reinterpret_cast<const bf16_t*>(p.V) + (long)s.ctx0 * p.ldv + (long)h * p.v_head;
+    const bf16_t *K, *KRp = nullptr, *V;
+    if constexpr (HEADS) {
+        K = reinterpret_cast<const bf16_t*>(s.cache) + (p.layer_off + (long)(h / p.rep) * p.kvw) * s.max_len;
+        V = K + p.v_col;
+    } else {
+        K = reinterpret_cast<const bf16_t*>(p.K) + (long)s.ctx0 * p.ldk + (long)h * p.k_head;
+        KRp = reinterpret_cast<const bf16_t*>(p.KR) + (long)s.ctx0 * p.ldkr;
+        V = reinterpret_cast<const bf16_t*>(p.V) + (long)s.ctx0 * p.ldv + (long)h * p.v_head;
+    }
 
     bf16x8 qf[NQ][KS];
     int qpos[NQ];
@@ -368,6 +389,17 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
     const int wave_hi = s.pos0 + min(q0 + wid * 32 + 31, s.len - 1);               // last position of the wave's rows
     const int kend = s.pos0 + min(q0 + 128, s.len);                                 // keys the workgroup needs
     const int nt = (kend + 63) >> 6;
+    const int p0 = s.pos0 + q0;                                                     // position of the workgroup's first row
+    float b_far = 0.f;
+    int t_far = 0;                                                                  // tiles [0, t_far) lie past the bias table's end
+    float* const win = reinterpret_cast<float*>(smem + 2 * BUF);
+    if constexpr (HEADS) {
+        if (p.bias) {
+            b_far = p.bias[(long)h * p.nb + p.nb - 1];
+            const int d = p0 - 62 - p.nb;                                           // kb <= p0 - 63 - (nb - 1)
+            t_far = d >= 0 ? (d >> 6) + 1 : 0;
+        } else t_far = nt;
+    }
 
     f32x4 oacc[DT][NQ], lacc[NQ];
     float m_ref[NQ];
@@ -390,7 +422,7 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
         chunk = min((id % CH) ^ mla_kswz<CH>(row), nkc - 1);
     };
     auto r_slot = [&](int i, int& row, int& chunk) {
-        constexpr int CH = KR * 4;
+        constexpr int CH = KR > 0 ? KR * 4 : 4;
         const int id = 64 * (wid + 4 * i) + lane;
         row = id / CH;
         chunk = min((id % CH) ^ mla_kswz<CH>(row), nrc - 1);
@@ -401,11 +433,13 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
         row = id / CH;
         chunk = min((((sl >> 1) ^ mla_vswz<DT>(row)) << 1) | (sl & 1), nvc - 1);
     };
-    int k_off[KN], r_off[KR], v_off[PV];
+    int k_off[KN], r_off[KR + 1], v_off[PV];
 #pragma unroll
     for (int i = 0; i < KN; ++i) { int row, c; k_slot(i, row, c); k_off[i] = (row * (int)p.ldk + c * 8) * 2; }
+    if constexpr (!HEADS) {
 #pragma unroll
-    for (int i = 0; i < KR; ++i) { int row, c; r_slot(i, row, c); r_off[i] = (row * (int)p.ldkr + c * 8) * 2; }
+        for (int i = 0; i < KR; ++i) { int row, c; r_slot(i, row, c); r_off[i] = (row * (int)p.ldkr + c * 8) * 2; }
+    }
 #pragma unroll
     for (int i = 0; i < PV; ++i) { int row, c; v_slot(i, row, c); v_off[i] = (row * (int)p.ldv + c * 8) * 2; }
     auto uniform_ptr = [](const bf16_t* q) -> const bf16_t* {
@@ -420,7 +454,7 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
     auto issue_tile = [&](int t) {
         const int kb = t * 64, valid = kend - kb;                      // >= 1; rows past the end repeat the last one (masked)
         const bf16_t* kp = uniform_ptr(K + (long)kb * p.ldk);
-        const bf16_t* rp = uniform_ptr(KRp + (long)kb * p.ldkr);
+        const bf16_t* rp = HEADS ? nullptr : uniform_ptr(KRp + (long)kb * p.ldkr);
         const bf16_t* vp = uniform_ptr(V + (long)kb * p.ldv);
         const unsigned st = __builtin_amdgcn_readfirstlane(smem_lds + (t & 1) * BUF);
         const bool ragged = valid < 64;
@@ -430,11 +464,13 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
             if (ragged) { int row, c; k_slot(i, row, c); o -= max(row - (valid - 1), 0) * (int)p.ldk * 2; }
             dma16(kp, o, st + (wid + 4 * i) * 1024);
         }
+        if constexpr (!HEADS) {
 #pragma unroll
-        for (int i = 0; i < KR; ++i) {
-            int o = r_off[i];
-            if (ragged) { int row, c; r_slot(i, row, c); o -= max(row - (valid - 1), 0) * (int)p.ldkr * 2; }
-            dma16(rp, o, st + N_LDS + (wid + 4 * i) * 1024);
+            for (int i = 0; i < KR; ++i) {
+                int o = r_off[i];
+                if (ragged) { int row, c; r_slot(i, row, c); o -= max(row - (valid - 1), 0) * (int)p.ldkr * 2; }
+                dma16(rp, o, st + N_LDS + (wid + 4 * i) * 1024);
+            }
         }
 #pragma unroll
         for (int i = 0; i < PV; ++i) {
@@ -444,13 +480,21 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
         }
     };
 
+    // bias window of tile t: entry i is distance p0 - 63 - 64 t + i (queries below p0 + 128, keys 64 t .. 64 t + 63)
+    auto stage_window = [&](int t) {
+        if constexpr (HEADS)
+            if (t >= t_far && tid < MLA_WIN)
+                win[(t & 1) * MLA_WIN + tid] = p.bias[(long)h * p.nb + min(max(p0 - 63 - 64 * t + tid, 0), p.nb - 1)];
+    };
+
     const int krow0 = 8 * (li >> 2) + (li & 3);
     const int vr = 8 * g + (li >> 2);                  // + 32 u (+ 4): mla_vswz is the same for all of them
     const int v_sw = mla_vswz<DT>(vr);
     const int v_base = vr * (DT * 32) + (li & 3) * 8;
 
-    auto process_tile = [&](const int t, auto masked_tag, auto first_tag) {
+    auto process_tile = [&](const int t, auto masked_tag, auto first_tag, auto near_tag) {
         constexpr bool MASKED = decltype(masked_tag)::value, FIRST = decltype(first_tag)::value;
+        constexpr bool NEAR = HEADS && decltype(near_tag)::value;
         const int kb = t * 64;
         if (!wave_active || (MASKED && kb > wave_hi)) return;
         const char* Ns = smem + (t & 1) * BUF;
@@ -461,20 +505,29 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
 #pragma unroll
         for (int u = 0; u < 4; ++u) {
             const int krow = 32 * (u >> 1) + 4 * (u & 1) + krow0;
-            const int nsw = mla_kswz<KN * 4>(krow), rsw = mla_kswz<KR * 4>(krow);
+            const int nsw = mla_kswz<KN * 4>(krow), rsw = HEADS ? 0 : mla_kswz<KR * 4>(krow);
+            f32x4 start[NQ];
+#pragma unroll
+            for (int i = 0; i < NQ; ++i) {
+                const float nm = HEADS && !NEAR ? b_far - m_ref[i] : -m_ref[i];
+                start[i] = f32x4{nm, nm, nm, nm};
+                if constexpr (NEAR) {
+                    const float* b = win + (t & 1) * MLA_WIN + (qpos[i] - p0 + 63 - (32 * (u >> 1) + 8 * g + 4 * (u & 1)));
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) start[i][r] += b[-r];
+                }
+            }
 #pragma unroll
             for (int k = 0; k < KS; ++k) {
                 const char* a = k < KN ? Ns + krow * (KN * 64) + (((4 * k + g) ^ nsw) << 4)
                                        : Rs + krow * (KR * 64) + (((4 * (k - KN) + g) ^ rsw) << 4);
                 const bf16x8 kf = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(a));
 #pragma unroll
-                for (int i = 0; i < NQ; ++i) {
-                    const float nm = -m_ref[i];
-                    sacc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][k], k == 0 ? f32x4{nm, nm, nm, nm} : sacc[u][i], 0, 0, 0);
-                }
+                for (int i = 0; i < NQ; ++i)
+                    sacc[u][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][k], k == 0 ? start[i] : sacc[u][i], 0, 0, 0);
             }
         }
-        if constexpr (!MASKED) {                       // 4 KS reads, 8 KS MFMAs: six reads lead, then a read per pair of MFMAs
+        if constexpr (!MASKED && !NEAR && KS >= 2) {   // 4 KS reads, 8 KS MFMAs: six reads lead, then a read per pair of MFMAs
             __builtin_amdgcn_sched_group_barrier(0x100, 6, 0);
 #pragma unroll
             for (int i = 0; i < 4 * KS - 6; ++i) {
@@ -565,30 +618,54 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
     // tiles [0, t_mid) lie left of the diagonal of every row
     const int t_mid = min((s.pos0 + q0 + 1) >> 6, nt);
     issue_tile(0);
+    stage_window(0);
     asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
 #pragma unroll
     for (int i = 0; i < NQ; ++i)
 #pragma unroll
         for (int k = 0; k < KS; ++k) asm volatile("" : "+v"(qf[i][k]));          // Q loads complete before the loop
+    if constexpr (HEADS) asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
     auto tile_tail = [&] {
         // the next tile has landed for this wave, behind the barrier for every wave, and nobody reads this one any more
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        if constexpr (HEADS) asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
+        else asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __builtin_amdgcn_s_barrier();
     };
-    if (1 < nt) issue_tile(1);
-    if (t_mid > 0) process_tile(0, std::false_type{}, std::true_type{});
-    else process_tile(0, std::true_type{}, std::true_type{});
+    auto next_tile = [&](int t) {
+        if (t >= nt) return;
+        issue_tile(t);
+        stage_window(t);
+    };
+    typedef std::true_type yes;
+    typedef std::false_type no;
+    next_tile(1);
+    // masked tiles look the bias up, unless there is none
+    const bool no_bias = HEADS && t_far >= nt;
+    if (t_mid <= 0) {
+        if (no_bias) process_tile(0, yes{}, yes{}, no{});
+        else process_tile(0, yes{}, yes{}, yes{});
+    } else if (!HEADS || 0 < t_far) process_tile(0, no{}, yes{}, no{});
+    else process_tile(0, no{}, yes{}, yes{});
     tile_tail();
     int t = 1;
-    for (; t < t_mid; ++t) {
-        if (t + 1 < nt) issue_tile(t + 1);
-        process_tile(t, std::false_type{}, std::false_type{});
+    const int t_plain = HEADS ? min(t_mid, t_far) : t_mid;
+    for (; t < t_plain; ++t) {
+        next_tile(t + 1);
+        process_tile(t, no{}, no{}, no{});
         tile_tail();
     }
+    if constexpr (HEADS) {
+        for (; t < t_mid; ++t) {
+            next_tile(t + 1);
+            process_tile(t, no{}, no{}, yes{});
+            tile_tail();
+        }
+    }
     for (; t < nt; ++t) {
-        if (t + 1 < nt) issue_tile(t + 1);
-        process_tile(t, std::true_type{}, std::false_type{});
+        next_tile(t + 1);
+        if (no_bias) process_tile(t, yes{}, no{}, no{});
+        else process_tile(t, yes{}, no{}, yes{});
         tile_tail();
     }
 
@@ -616,7 +693,9 @@ __global__ __launch_bounds__(256, WGS) void mla_prefill_kernel(CogsMla p, int nq
 struct MlaDecodeArgs {
     const bf16_t* Q; long ldq; int q_head;
     const CogsSeq* seqs; long layer_off;
-    int kvw, kvp, heads, nht, nsplit;
+    int kvw, kcols, vcol, kvp;              // cache row: columns [0, kcols) meet the query, [vcol, vcol + kvp) are summed
+    int heads, rep, groups, nht, nsplit;    // rep query heads read one cache block, `groups` blocks per sequence
+    const float* bias; int nb;              // [heads][nb] added at distance min(n, nb - 1), or null
     float* part_o; float* part_ml;          // [seq][split][head][kvp] relative to part_ml[..][0]; [..][2] = (max, sum)
 };
 
@@ -636,7 +715,7 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
     const int bid = blockIdx.x, slot = bid & 7, rest = bid >> 3;
     const int ht = rest % p.nht, split = (rest / p.nht) * 8 + slot;
     if (split >= p.nsplit) return;
-    const int b = blockIdx.y, h0 = ht * 16;
+    const int b = blockIdx.y / p.groups, grp = blockIdx.y - b * p.groups, h0 = grp * p.rep + ht * 16, h1 = (grp + 1) * p.rep;
     const CogsSeq s = p.seqs[b];
     const int kend = s.pos0 + 1;
     const unsigned nt_all = (unsigned)(kend + TK - 1) / TK;
@@ -644,11 +723,11 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
     const int t_end = (int)(nt_all * (unsigned)(split + 1) / (unsigned)p.nsplit);
     const long slot0 = ((long)b * p.nsplit + split) * p.heads;
     if (t_begin >= t_end) {                                        // nothing to do: an empty partial
-        if (tid < 16 && h0 + tid < p.heads) { p.part_ml[(slot0 + h0 + tid) * 2] = -INFINITY; p.part_ml[(slot0 + h0 + tid) * 2 + 1] = 0.f; }
+        if (tid < 16 && h0 + tid < h1) { p.part_ml[(slot0 + h0 + tid) * 2] = -INFINITY; p.part_ml[(slot0 + h0 + tid) * 2 + 1] = 0.f; }
         return;
     }
-    const char* cache = s.cache + p.layer_off * s.max_len * 2;
-    const int row_bytes = p.kvw * 2, nch = p.kvw >> 3;             // 16-byte chunks of a row
+    const char* cache = s.cache + (p.layer_off + (long)grp * p.kvw) * s.max_len * 2;
+    const int row_bytes = p.kvw * 2, nch = p.kvw >> 3, nqc = p.kcols >> 3;      // 16-byte chunks of a row
     const int tile_chunks = TK * nch;
     const int dr_row = 256 / nch, dr_c = 256 % nch;
 
@@ -667,13 +746,13 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
 #pragma unroll 1
         while (r < 16) {
             u32x4 v = {0, 0, 0, 0};
-            if (h0 + r < p.heads) v = *reinterpret_cast<const u32x4*>(p.Q + (long)b * p.ldq + (long)(h0 + r) * p.q_head + c * 8);
+            if (h0 + r < h1 && c < nqc) v = *reinterpret_cast<const u32x4*>(p.Q + (long)b * p.ldq + (long)(h0 + r) * p.q_head + c * 8);
             *reinterpret_cast<u32x4*>(Qs + r * RS + c * 16) = v;
             r += dr_row; c += dr_c;
             if (c >= nch) { c -= nch; ++r; }
         }
     }
-    const int ks = p.kvw >> 5, dts = p.kvp >> 4, kh = (ks + 1) >> 1;
+    const int ks = p.kcols >> 5, dts = p.kvp >> 4, kh = (ks + 1) >> 1;
     const int k_lo = (wid >> 1) ? kh : 0, k_hi = (wid >> 1) ? ks : kh;
     f32x4 oacc[DTW], lacc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -682,7 +761,9 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
     const bf16x8 ones = __builtin_bit_cast(bf16x8, u32x4{0x3f803f80u, 0x3f803f80u, 0x3f803f80u, 0x3f803f80u});
     const char* const qrd = Qs + li * RS + 16 * g;
     const char* const krd = Ks + (16 * (wid & 1) + li) * RS + 16 * g;
-    const char* const vrd = Ks + (4 * g + (li >> 2)) * RS + (li & 3) * 8 + 32 * wid;
+    const char* const vrd = Ks + (4 * g + (li >> 2)) * RS + (li & 3) * 8 + 32 * wid + p.vcol * 2;
+    const float* const bias = p.bias ? p.bias + (long)min(h0 + li, h1 - 1) * p.nb : nullptr;
+    const float b_far = bias ? bias[p.nb - 1] : 0.f;
 
     for (int t = t_begin; t < t_end; ++t) {
         __syncthreads();                                          // the previous tile's transposed reads are done
@@ -698,6 +779,15 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
         __syncthreads();
         if (t + 1 < t_end) load_tile(t + 1);
         const int nvalid = min(TK, kend - t * TK);
+        f32x4 bias0 = {b_far, b_far, b_far, b_far}, bias1 = bias0;
+        if (bias && s.pos0 - t * TK - (TK - 1) < p.nb - 1) {
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int d = s.pos0 - t * TK - 4 * g - r;
+                bias0[r] = bias[min(max(d, 0), p.nb - 1)];
+                bias1[r] = bias[min(max(d - 16, 0), p.nb - 1)];
+            }
+        }
         {
             f32x4 acc[4];
 #pragma unroll
@@ -722,7 +812,7 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
             Sx[((wid & 1) * 2 + (wid >> 1)) * 64 + lane] = (acc[0] + acc[1]) + (acc[2] + acc[3]);
         }
         __syncthreads();
-        f32x4 s0 = Sx[lane] + Sx[64 + lane], s1 = Sx[128 + lane] + Sx[192 + lane];
+        f32x4 s0 = Sx[lane] + Sx[64 + lane] + bias0, s1 = Sx[128 + lane] + Sx[192 + lane] + bias1;
         float tm = -INFINITY;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
@@ -757,7 +847,7 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
             oacc[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl, oacc[d], 0, 0, 0);
         }
     }
-    if (h0 + li < p.heads) {
+    if (h0 + li < h1) {
         const long o = slot0 + h0 + li;
 #pragma unroll
         for (int d = 0; d < DTW; ++d) {
@@ -771,7 +861,8 @@ __global__ __launch_bounds__(256, WGS) void mla_decode_kernel(MlaDecodeArgs p) {
 // splits of one (sequence, head) -> the head's weighted latent, bf16; 64 latent columns per workgroup, wave w sums every fourth split
 constexpr int MLA_MAX_SPLIT = 256;
 __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit,
-                                                          int heads, int kvp, const float* __restrict__ sink, bf16_t* __restrict__ out) {
+                                                          int heads, int kvp, const float* __restrict__ sink, bf16_t* __restrict__ out,
+                                                          long ldo, int o_head) {
     __shared__ float w_sh[MLA_MAX_SPLIT];
     __shared__ float red[4];
     __shared__ float acc_sh[4][64];
@@ -780,7 +871,7 @@ __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restric
     const long base = (long)b * nsplit * heads + h;
     // the first 16 partial rows of this wave are requested before the weights are known (an empty split's row holds anything: its
     // weight is tested, not multiplied)
-    const float* po = part_o + base * kvp + d;
+    const float* po = part_o + base * kvp + min(d, kvp - 1);
     const long stride = (long)heads * kvp;
     float v[16];
 #pragma unroll
@@ -813,17 +904,17 @@ __global__ __launch_bounds__(256) void mla_combine_kernel(const float* __restric
     }
     acc_sh[wid][lane] = a;
     __syncthreads();
-    if (wid == 0) {
+    if (wid == 0 && d < kvp) {
         float L = (red[0] + red[1]) + (red[2] + red[3]);
         if (sink) L += exp2f(sk - M);
-        out[((long)b * heads + h) * kvp + d] = f2bf(((acc_sh[0][lane] + acc_sh[1][lane]) + (acc_sh[2][lane] + acc_sh[3][lane])) / L);
+        out[b * ldo + (long)h * o_head + d] = f2bf(((acc_sh[0][lane] + acc_sh[1][lane]) + (acc_sh[2][lane] + acc_sh[3][lane])) / L);
     }
 }
 
 template <int KN, int KR, int DT, int WGS>
 int launch_prefill(hipStream_t st, const CogsMla& a) {
     static std::atomic<uint64_t> attr_done{0};
-    constexpr int lds = 2 * (64 * KN * 64 + 64 * KR * 64 + 64 * DT * 32);
+    constexpr int lds = 2 * (64 * KN * 64 + 64 * KR * 64 + 64 * DT * 32) + (KR == 0 ? 2 * MLA_WIN * 4 : 0);
     cogs_ensure_dyn_lds((const void*)mla_prefill_kernel<KN, KR, DT, WGS>, lds, attr_done);
     const int nqt = (a.max_new + 127) / 128;
     const long grid = (long)nqt * a.heads * a.nseq;
@@ -834,11 +925,11 @@ int launch_prefill(hipStream_t st, const CogsMla& a) {
 }
 
 template <int DTW, int PER, int WGS>
-int launch_decode(hipStream_t st, const MlaDecodeArgs& p, int nseq) {
+int launch_decode(hipStream_t st, const MlaDecodeArgs& p, int nblk) {
     static std::atomic<uint64_t> attr_done{0};
     const int lds = 48 * (p.kvw * 2 + 32) + 4 * 64 * 16;
     cogs_ensure_dyn_lds((const void*)mla_decode_kernel<DTW, PER, WGS>, 160 * 1024, attr_done);
-    hipLaunchKernelGGL((mla_decode_kernel<DTW, PER, WGS>), dim3((unsigned)((p.nsplit + 7) / 8 * 8 * p.nht), nseq), dim3(256), lds, st, p);
+    hipLaunchKernelGGL((mla_decode_kernel<DTW, PER, WGS>), dim3((unsigned)((p.nsplit + 7) / 8 * 8 * p.nht), nblk), dim3(256), lds, st, p);
     return COGS_LAUNCH_CHECK();
 }
 
@@ -888,8 +979,20 @@ int cogs_k_head_gemm(hipStream_t st, int dtype, const CogsHeadGemm& a) {
 int cogs_k_mla_attention(hipStream_t st, int dtype, const CogsMla& a) {
     if (a.rows <= 0 || a.nseq <= 0 || a.heads <= 0 || a.dn % 4 || a.dr % 4 || a.dv <= 0) return COGS_E_INVALID;
     const int es = dtype == COGS_DT_BF16 ? 2 : 4;
+    if (a.kvw) {
+        if (a.rep <= 0 || a.heads % a.rep || a.dr || a.ldk != a.kvw || a.ldv != a.kvw || (a.bias && a.nb <= 0)) return COGS_E_INVALID;
+    } else if (a.bias) return COGS_E_INVALID;
     if ((a.ldk * es) % 8 || (a.ldkr * es) % 8 || (a.ldv * es) % 8) return COGS_E_INVALID;
-    if (dtype == COGS_DT_BF16 && !a.absorbed && a.dn % 8 == 0 && a.dr % 8 == 0 && a.dv % 16 == 0 && a.ldq % 8 == 0 && a.q_head % 32 == 0 &&
+    if (dtype == COGS_DT_BF16 && a.kvw && a.dn % 32 == 0 && a.dv % 16 == 0 && a.v_col % 8 == 0 && a.kvw % 8 == 0 && a.ldq % 8 == 0 &&
+        a.q_head % 32 == 0 && a.q_head >= a.dn && a.q_rot == a.q_head && a.ldo % 4 == 0 && a.o_head % 4 == 0 && g_cogs_debug.mla_rowwise == 0 &&
+        a.kvw < (1 << 23)) {
+        const int kn = a.dn / 32, dt = a.dv / 16;
+        if (kn <= 1 && dt <= 2) return launch_prefill<1, 0, 2, 2>(st, a);
+        if (kn <= 2 && dt <= 4) return launch_prefill<2, 0, 4, 2>(st, a);
+        if (kn <= 4 && dt <= 8) return launch_prefill<4, 0, 8, 2>(st, a);
+        if (kn <= 8 && dt <= 16) return launch_prefill<8, 0, 16, 1>(st, a);
+    }
+    if (dtype == COGS_DT_BF16 && !a.kvw && !a.absorbed && a.dn % 8 == 0 && a.dr % 8 == 0 && a.dv % 16 == 0 && a.ldq % 8 == 0 && a.q_head % 32 == 0 &&
         a.q_rot % 32 == 0 && a.q_rot >= a.dn && a.q_head - a.q_rot >= a.dr && a.ldk % 8 == 0 && a.k_head % 8 == 0 && a.ldkr % 8 == 0 &&
         a.ldv % 8 == 0 && a.v_head % 8 == 0 && a.ldo % 4 == 0 && a.o_head % 4 == 0 && g_cogs_debug.mla_rowwise == 0 &&
         a.ldk < (1 << 23) && a.ldkr < (1 << 23) && a.ldv < (1 << 23)) {       // (a tile's byte offsets are 32 bits)
@@ -907,7 +1010,7 @@ int cogs_k_mla_attention(hipStream_t st, int dtype, const CogsMla& a) {
 }
 
 bool cogs_k_mla_decode_fits(int kvw, int kvp) {
-    return kvw % 32 == 0 && kvp % 64 == 0 && kvp <= 1024 && 48 * (kvw * 2 + 32) + 4096 <= 160 * 1024 && 32 * (kvw / 8) <= 256 * 18;
+    return kvw % 32 == 0 && kvp % 16 == 0 && kvp <= 1024 && 48 * (kvw * 2 + 32) + 4096 <= 160 * 1024 && 32 * (kvw / 8) <= 256 * 18;
 }
 
 int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx) {
@@ -924,22 +1027,25 @@ int cogs_k_mla_decode_splits(int nseq, int heads, int max_ctx) {
     return n > MLA_MAX_SPLIT ? MLA_MAX_SPLIT : n;
 }
 
-// one new row per sequence, absorbed queries [seq][heads][kvw]; -> latent sums [seq][heads][kvp]
+// one new row per sequence: queries of kcols columns per head -> per head the weighted sum of the cache rows' value columns
 int cogs_k_mla_decode(hipStream_t st, const CogsMlaDecode& a) {
-    if (a.nseq <= 0 || a.nseq > 65535 || a.nsplit < 1 || a.nsplit > MLA_MAX_SPLIT || !cogs_k_mla_decode_fits(a.kvw, a.kvp) ||
+    if (a.rep <= 0 || a.heads % a.rep || a.kcols % 32 || a.kcols > a.kvw || a.vcol % 16 || a.vcol + a.kvp > a.kvw || (a.bias && a.nb <= 0) ||
+        a.nseq <= 0 || (long)a.nseq * (a.heads / a.rep) > 65535 || a.nsplit < 1 || a.nsplit > MLA_MAX_SPLIT || !cogs_k_mla_decode_fits(a.kvw, a.kvp) ||
         a.ldq % 8 || a.q_head % 8 || a.heads <= 0) return COGS_E_INVALID;
     MlaDecodeArgs p;
     p.Q = (const bf16_t*)a.Q; p.ldq = a.ldq; p.q_head = a.q_head; p.seqs = a.seqs; p.layer_off = a.layer_off;
-    p.kvw = a.kvw; p.kvp = a.kvp; p.heads = a.heads; p.nht = (a.heads + 15) / 16; p.nsplit = a.nsplit;
+    p.kvw = a.kvw; p.kcols = a.kcols; p.vcol = a.vcol; p.kvp = a.kvp; p.nsplit = a.nsplit;
+    p.heads = a.heads; p.rep = a.rep; p.groups = a.heads / a.rep; p.nht = (a.rep + 15) / 16;
+    p.bias = a.bias; p.nb = a.nb;
     p.part_o = a.part; p.part_ml = a.part + (size_t)a.nseq * a.nsplit * a.heads * a.kvp;
-    const int dtw = (a.kvp / 16 + 3) / 4, chunks = 32 * (a.kvw / 8);
+    const int dtw = (a.kvp / 16 + 3) / 4, chunks = 32 * (a.kvw / 8), nblk = a.nseq * p.groups;
     int rc;
-    if (dtw <= 2 && chunks <= 256 * 4) rc = launch_decode<2, 4, 4>(st, p, a.nseq);
-    else if (dtw <= 4 && chunks <= 256 * 6) rc = launch_decode<4, 6, 3>(st, p, a.nseq);
-    else if (dtw <= 8 && chunks <= 256 * 10) rc = launch_decode<8, 10, 2>(st, p, a.nseq);
-    else rc = launch_decode<16, 18, 1>(st, p, a.nseq);
+    if (dtw <= 2 && chunks <= 256 * 4) rc = launch_decode<2, 4, 4>(st, p, nblk);
+    else if (dtw <= 4 && chunks <= 256 * 6) rc = launch_decode<4, 6, 3>(st, p, nblk);
+    else if (dtw <= 8 && chunks <= 256 * 10) rc = launch_decode<8, 10, 2>(st, p, nblk);
+    else rc = launch_decode<16, 18, 1>(st, p, nblk);
     if (rc != COGS_OK) return rc;
-    hipLaunchKernelGGL(mla_combine_kernel, dim3(a.heads, a.nseq, a.kvp / 64), dim3(256), 0, st, p.part_o, p.part_ml, a.nsplit, a.heads, a.kvp,
-                       a.sink, (bf16_t*)a.out);
+    hipLaunchKernelGGL(mla_combine_kernel, dim3(a.heads, a.nseq, (a.kvp + 63) / 64), dim3(256), 0, st, p.part_o, p.part_ml, a.nsplit, a.heads,
+                       a.kvp, a.sink, (bf16_t*)a.out, a.ldo, a.o_head);
     return COGS_LAUNCH_CHECK();
 }

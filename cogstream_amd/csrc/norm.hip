@@ -277,8 +277,125 @@ __global__ __launch_bounds__(TPB) void stream_norm_kernel(CogsStreamNorm p) {
     }
 }
 
+// the same with a scaled embedding and a position table at the start and hyper-connected streams (x [row][stream][Hp]). NS: streams
+// rounded up; a chunk's old streams are in registers together, only the combination that is normed stays there for the row.
+template <typename T, int C, int TPB, int NS>
+__global__ __launch_bounds__(TPB) void stream_mix_kernel(CogsStreamNorm p) {
+    constexpr int NW = TPB / 64;
+    __shared__ float red[2][NW];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const long row = p.pick ? p.pick[blockIdx.x] : blockIdx.x;
+    const int ns = p.streams > 0 ? p.streams : 1;
+    float* x = p.x + row * ns * p.Hp;
+    auto row_rstd = [&](float ss, int which) {
+        ss = wave_sum(ss);
+        if (lane == 0) red[which][wid] = ss;
+        __syncthreads();
+        ss = red[which][0];
+#pragma unroll
+        for (int w = 1; w < NW; ++w) ss += red[which][w];
+        return 1.f / sqrtf(ss / (float)p.H + p.eps);
+    };
+    f32x4 y[C], u[C];
+    float rs = 1.f;
+    if (p.y) {
+        float ss = 0.f;
+#pragma unroll
+        for (int c = 0; c < C; ++c) {
+            const int i = (tid + TPB * c) * 4;
+            y[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (i < p.Hp) y[c] = ld4_f<T>(reinterpret_cast<const T*>(p.y) + row * p.Hp + i);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) ss += y[c][e] * y[c][e];
+        }
+        if (p.y_gamma) rs = row_rstd(ss, 0);
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+        const int i = (tid + TPB * c) * 4;
+        u[c] = f32x4{0.f, 0.f, 0.f, 0.f};
+        if (i >= p.Hp) continue;
+        f32x4 v[NS];
+        if (p.embeds) {
+            f32x4 e = ld4_f<T>(reinterpret_cast<const T*>(p.embeds) + row * p.Hp + i) * p.embed_scale;
+            if (p.pos) e += ld4_f<T>(reinterpret_cast<const T*>(p.pos) + (long)p.rowpos[row] * p.Hp + i);
+#pragma unroll
+            for (int s = 0; s < NS; ++s) v[s] = e;
+        } else {
+#pragma unroll
+            for (int s = 0; s < NS; ++s)
+                if (s < ns) v[s] = *reinterpret_cast<const f32x4*>(x + (long)s * p.Hp + i);
+        }
+        if (p.y) {
+            f32x4 yv = y[c];
+            if (p.y_gamma) yv *= rs * *reinterpret_cast<const f32x4*>(p.y_gamma + i);
+            if (p.mix) {
+                f32x4 w[NS];
+#pragma unroll
+                for (int t = 0; t < NS; ++t) {
+                    if (t >= ns) continue;
+                    w[t] = yv * p.out_w[t];
+#pragma unroll
+                    for (int s = 0; s < NS; ++s)
+                        if (s < ns) w[t] += v[s] * p.mix[s * ns + t];
+                }
+#pragma unroll
+                for (int t = 0; t < NS; ++t)
+                    if (t < ns) v[t] = w[t];
+            } else {
+                v[0] += yv;
+            }
+        }
+        f32x4 sum = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int s = 0; s < NS; ++s) {
+            if (s >= ns) continue;
+            if (p.y || p.embeds) *reinterpret_cast<f32x4*>(x + (long)s * p.Hp + i) = v[s];
+            sum += v[s];
+            u[c] += p.in_w ? v[s] * p.in_w[s] : v[s];
+        }
+        if (p.sum) *reinterpret_cast<f32x4*>(p.sum + row * p.Hp + i) = sum;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) ss += u[c][e] * u[c][e];
+    }
+    if (!p.out) return;
+    rs = row_rstd(ss, 1);
+    T* o = reinterpret_cast<T*>(p.out) + (long)blockIdx.x * p.Hp;
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+        const int i = (tid + TPB * c) * 4;
+        if (i >= p.Hp) continue;
+        st4_f<T>(o + i, u[c] * rs * *reinterpret_cast<const f32x4*>(p.out_gamma + i));
+    }
+}
+
+template <typename T, int NS>
+int launch_stream_mix(hipStream_t st, const CogsStreamNorm& a) {
+    const dim3 grid(a.rows);
+#define COGS_STREAM(C, TPB) hipLaunchKernelGGL((stream_mix_kernel<T, C, TPB, NS>), grid, dim3(TPB), 0, st, a)
+    if (a.rows <= 64 && a.Hp > 1024) {
+        if (a.Hp <= 4096) COGS_STREAM(1, 1024);
+        else if (a.Hp <= 16384) COGS_STREAM(4, 1024);
+        else return COGS_E_UNSUPPORTED;
+    } else if (a.Hp <= 1024) COGS_STREAM(1, 256);
+    else if (a.Hp <= 4096) COGS_STREAM(4, 256);
+    else if (a.Hp <= 16384) COGS_STREAM(16, 256);
+    else return COGS_E_UNSUPPORTED;
+#undef COGS_STREAM
+    return COGS_LAUNCH_CHECK();
+}
+
 template <typename T>
 int launch_stream_norm(hipStream_t st, const CogsStreamNorm& a) {
+    if (a.streams > 0 || a.pos || a.embed_scale != 1.f || a.sum) {
+        if (a.streams <= 1) return launch_stream_mix<T, 1>(st, a);
+        if (a.streams <= 2) return launch_stream_mix<T, 2>(st, a);
+        if (a.streams <= 4) return launch_stream_mix<T, 4>(st, a);
+        if (a.streams <= 8) return launch_stream_mix<T, 8>(st, a);
+        if (a.streams <= 16) return launch_stream_mix<T, 16>(st, a);
+        return COGS_E_UNSUPPORTED;
+    }
     const dim3 grid(a.rows);
 #define COGS_STREAM(C, TPB) hipLaunchKernelGGL((stream_norm_kernel<T, C, TPB>), grid, dim3(TPB), 0, st, a)
     if (a.rows <= 64 && a.Hp > 1024) {           // few rows: latency, not bandwidth -- more threads on each
@@ -300,6 +417,7 @@ int launch_stream_norm(hipStream_t st, const CogsStreamNorm& a) {
 
 int cogs_k_stream_norm(hipStream_t st, int dtype, const CogsStreamNorm& a) {
     if (a.rows <= 0) return COGS_OK;
+    if ((a.pos && !a.rowpos) || (a.y && a.streams > 0 && (!a.mix || !a.out_w)) || (a.streams <= 0 && (a.mix || a.in_w))) return COGS_E_INVALID;
     if (!a.x || a.Hp % 4 || a.H <= 0 || a.H > a.Hp || (a.out && !a.out_gamma) || (a.pick && (!a.out || a.y || a.embeds))) return COGS_E_INVALID;
     return dtype == COGS_DT_BF16 ? launch_stream_norm<bf16_t>(st, a) : launch_stream_norm<float>(st, a);
 }

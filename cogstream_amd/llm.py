@@ -40,18 +40,40 @@ class KVCache:
         """views [..., max_len, columns] that hold the cached rows"""
         return [self.k, self.v]
 
+    state: Optional[torch.Tensor] = None       # what the length `len` has besides its rows (recurrent models)
+    stale = False
+
+    def restore(self, length: int, state: Optional[torch.Tensor]):
+        """back to a length whose rows are in place and whose `state` was kept"""
+        self.reset(length)
+
     def copy_rows_from(self, old: "KVCache", n: int):
         for dst, src in zip(self._blocks(), old._blocks()):
             dst[..., :n, :].copy_(src[..., :n, :])
 
 
-class LatentCache(KVCache):
-    """one sequence's rows [latent | rotated key part] of every layer that has its own (weights.PackedDecoder.cache_widths)"""
+class DecoderCache(KVCache):
+    """one sequence of a decoder described layer by layer: the rows of every layer run that caches rows (latents, or keys and values
+    per head; weights.PackedDecoder.cache_widths) and, fp32, the state of every recurrent one. A state belongs to exactly the
+    length it was left at: reset() to any other but 0 leaves the cache unusable until restore() brings a state back."""
 
-    def __init__(self, widths: Sequence[int], max_len: int, dtype, device):
+    def __init__(self, widths: Sequence[int], state_floats: int, max_len: int, dtype, device):
         self.widths = list(widths)
         self.k = torch.empty(sum(self.widths) * max_len, device=device, dtype=dtype)
-        self.struct = L.KV(self.k.data_ptr(), None, max_len, 0)
+        self.state = torch.empty(state_floats, device=device, dtype=torch.float32) if state_floats else None
+        self.struct = L.KV(self.k.data_ptr(), L.ptr(self.state) or None, max_len, 0)
+        self.stale = False
+
+    def reset(self, length: int = 0):
+        if self.state is not None and length != self.len:
+            self.stale = length != 0
+        self.struct.len = length
+
+    def restore(self, length: int, state: Optional[torch.Tensor]):
+        self.struct.len = length
+        if self.state is not None and length:
+            self.state.copy_(state)
+        self.stale = False
 
     def _blocks(self) -> List[torch.Tensor]:
         out, at = [], 0
@@ -67,12 +89,14 @@ class PrefixKV:
     The reusable prefix is found by comparing the new input embeddings with the previous ones bit for bit on the
     device: KV row i depends only on rows 0..i and the position i, so every invalidation rule (resized frames, a
     history turn dropped by the selection stage, another question) is covered by that comparison. Only rows that
-    were PREFILLED are reused -- rows written by decode steps went through the GEMV kernels."""
+    were PREFILLED are reused -- rows written by decode steps went through the GEMV kernels. Models with recurrent
+    state keep a copy of the state behind the prompt, so they can reuse the whole previous prompt or nothing of it."""
 
     def __init__(self, engine: "CausalEngine"):
         self.engine = engine
         self.cache: Optional[KVCache] = None
         self.rows: Optional[torch.Tensor] = None   # [n, H] embeddings whose KV rows 0..n-1 are in `cache`
+        self.state: Optional[torch.Tensor] = None  # recurrent state behind row n-1
         self.reused = 0    # rows taken from the cache, summed over calls
         self.seen = 0      # prompt rows, summed over calls
 
@@ -94,6 +118,8 @@ class PrefixKV:
                 neq = (self.rows[:n].view(bits) != embeds[:n].view(bits)).any(dim=1)
                 idx = torch.arange(n, device=embeds.device)
                 p = int(torch.where(neq, idx, torch.full_like(idx, n)).min().item())
+                if self.cache.state is not None and p < self.rows.shape[0]:
+                    p = 0
         self.seen += embeds.shape[0]
         self.reused += p
         return p
@@ -171,9 +197,10 @@ class CausalEngine:
             embeds = embeds.contiguous()
             p = prefix.plan(embeds, S + max_new_tokens)
             cache = prefix.cache
-            cache.reset(p)
+            cache.restore(p, prefix.state)
             prefix.rows = None          # not valid while this call is rewriting the cache
             res = self.forward(embeds[p:], cache)
+            prefix.state = None if cache.state is None else cache.state.clone()
             prefix.rows = embeds        # rows 0..S-1 are prefilled; decode rows behind them are never reused
             pos_start = S
         else:
@@ -197,7 +224,8 @@ class CausalEngine:
         n_seen, produced = n_prompt, 0
         # host-drawn sampling (parity mode) consumes one [vocab] draw of the CPU generator per step: steps issued past
         # the EOS would advance that generator beyond where GenerationMixin stops, so the stop test runs every step
-        check_every = 1 if (do_sample and sampler == "host") else 8
+        # (nor can a recurrent state step back over tokens behind the EOS)
+        check_every = 1 if (do_sample and sampler == "host") or cache.state is not None else 8
         if do_sample and sampler == "device" and seed is None:
             seed = int(torch.randint(0, 2 ** 62, (1,), generator=generator).item())
         need_proc = repetition_penalty != 1.0 or allowed is not None     # the temperature is applied inside cogs_sample
@@ -354,18 +382,23 @@ class DecoderEngine(CausalEngine):
         self.handle.activate("decoder", self, lambda: L.check(
             L.lib.cogs_decoder_load(self.handle.h, C.byref(self.packed.struct)), "cogs_decoder_load"))
 
-    def new_cache(self, max_len: int) -> LatentCache:
-        return LatentCache(self.packed.cache_widths, max_len, self.dtype, self.device)
+    def new_cache(self, max_len: int) -> DecoderCache:
+        return DecoderCache(self.packed.cache_widths, self.packed.state_floats, max_len, self.dtype, self.device)
 
     def embed_tokens(self, ids: torch.Tensor) -> torch.Tensor:
         return ops.gather_rows(self.packed.embed, None, ids.reshape(-1).to(self.device, torch.int64))
 
     def forward_batch(self, embeds: torch.Tensor, lens: Sequence[int], caches: Sequence[KVCache], want: Sequence[int],
                       streams: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
-        """streams, when given: fp32 [layers, rows, padded width], receives the residual stream behind every layer"""
+        """streams, when given: fp32 [layer runs, rows, padded width], receives the residual stream behind every layer run"""
         self._activate()
         embeds = embeds.contiguous()
         S, n, nw = embeds.shape[0], len(lens), len(want)
+        if any(c.stale for c in caches):
+            raise L.CogsError("a cache's recurrent state does not belong to its length")
+        limit = self.cfg.max_positions
+        if limit and any(c.len + k > limit for c, k in zip(caches, lens)):
+            raise L.CogsError(f"a sequence would pass the model's {limit} positions")
         assert sum(lens) == S and len(caches) == n and embeds.shape[1] == self.packed.width_p and embeds.dtype == self.dtype
         ctx = S + sum(c.len for c in caches)
         nbytes = C.c_size_t()
@@ -402,7 +435,7 @@ class Sequences:
             grown = self.engine.new_cache(max(-(-need // self.reserve) * self.reserve, 2 * old.max_len if old is not None else 0))
             if old is not None:
                 grown.copy_rows_from(old, old.len)
-                grown.reset(old.len)
+                grown.restore(old.len, old.state)
             self.caches[rid] = grown
         return self.caches[rid]
 

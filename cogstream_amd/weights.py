@@ -12,7 +12,7 @@ from __future__ import annotations
 import ctypes as C
 import math
 from dataclasses import dataclass, field
-from typing import Dict, List, Optional, Tuple
+from typing import Dict, List, Optional, Tuple, Union
 
 import torch
 
@@ -111,11 +111,68 @@ class LatentAttention:
 
 
 @dataclass
+class DistanceBias:
+    """a learned score bias per head and bucket of distances: one bucket per distance below buckets / 2, logarithmically wider ones
+    up to distance `far`, the last for everything from there on"""
+    buckets: int
+    far: float
+
+    def bucket_of(self) -> List[int]:
+        """the bucket of every distance 0, 1, .. up to the first whose bucket is the last (all later ones share it)"""
+        half = self.buckets // 2
+        if half < 1 or self.far <= half:
+            raise ValueError(f"distance bias of {self.buckets} buckets up to distance {self.far}: no room for logarithmic buckets")
+        out: List[int] = []
+        while not out or out[-1] < self.buckets - 1:
+            n = len(out)
+            if n < half:
+                out.append(n)
+                continue
+            r = math.log(n / half) / math.log(self.far / half) * (self.buckets - half)
+            near = round(r)            # a quotient of logarithms that is a whole number may come out just below it
+            out.append(min(self.buckets - 1, half + (near if abs(r - near) < 1e-9 else math.floor(r))))
+        return out
+
+
+@dataclass
+class HeadAttention:
+    """softmax attention with keys and values per (shared) head (include/cogs.h, cogs_attn_mixer)"""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    scale: float
+    qk_norm: bool = False              # weightless RMS norm of every query and key head row
+    temp_coef: float = 0.0             # queries times 1 + temp_coef ln(floor((p + 1) / temp_every) + 1); temp_every 0: none
+    temp_every: float = 0.0
+    bias: Optional[DistanceBias] = None
+
+
+@dataclass
+class DeltaRule:
+    """gated delta rule behind short causal convolutions (include/cogs.h, cogs_delta_mixer)"""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    taps: int
+
+
+@dataclass
 class DecoderLayerConfig:
-    mixer: LatentAttention
-    ff: int = 0                        # gated-SiLU MLP width, 0 = no feed-forward sublayer
+    mixer: Union[LatentAttention, HeadAttention, DeltaRule]
+    ff: int = 0                        # MLP width, 0 = no feed-forward sublayer
+    mlp_act: str = "swiglu"            # "swiglu" (gated) or "gelu" (exact, up and down only)
     mlp_bias: bool = False
     post_norm: bool = True             # norms on the sublayers' outputs
+
+
+@dataclass
+class Loop:
+    """layers start .. stop - 1 run `times` times in a row"""
+    start: int
+    stop: int
+    times: int
 
 
 @dataclass
@@ -125,6 +182,10 @@ class DecoderConfig:
     vocab_size: int
     eps: float
     layers: List[DecoderLayerConfig] = field(default_factory=list)
+    embed_scale: float = 1.0
+    max_positions: int = 0             # > 0: a learned vector per position joins the embedding
+    streams: int = 0                   # > 0: hyper-connected residual streams
+    loop: Optional[Loop] = None
 
     @property
     def hidden_size(self) -> int:
@@ -133,6 +194,13 @@ class DecoderConfig:
     @property
     def num_hidden_layers(self) -> int:
         return len(self.layers)
+
+    def runs(self) -> List[int]:
+        """the layer of every layer run, loop passes unrolled"""
+        n, lp = len(self.layers), self.loop
+        if lp is None:
+            return list(range(n))
+        return [*range(lp.start), *[i for _ in range(lp.times) for i in range(lp.start, lp.stop)], *range(lp.stop, n)]
 
 
 def rope_perm(hd: int) -> torch.Tensor:
@@ -350,11 +418,39 @@ def decoder_tensors(cfg: DecoderConfig) -> Dict[str, Tuple[int, ...]]:
     """name -> shape of every tensor of a decoder described layer by layer"""
     W = cfg.width
     out: Dict[str, Tuple[int, ...]] = {"embed": (cfg.vocab_size, W), "final.norm": (W,), "head": (cfg.vocab_size, W)}
+    if cfg.max_positions:
+        out["pos"] = (cfg.max_positions, W)
     for i, lay in enumerate(cfg.layers):
         p, m = f"l{i}.", lay.mixer
-        out[p + "norm1"] = (W,)
-        if lay.post_norm:
-            out[p + "norm1b"] = (W,)
+        for n in ("1", "2") if lay.ff else ("1",):
+            out[p + "norm" + n] = (W,)
+            if lay.post_norm:
+                out[p + f"norm{n}b"] = (W,)
+            if cfg.streams:
+                s = cfg.streams
+                out[p + f"hc{n}.in"], out[p + f"hc{n}.out"], out[p + f"hc{n}.mix"] = (s,), (s,), (s, s)
+        if lay.ff:
+            for n, shape in (("gate", (lay.ff, W)), ("up", (lay.ff, W)), ("down", (W, lay.ff))):
+                if n == "gate" and lay.mlp_act != "swiglu":
+                    continue
+                out[p + "mlp." + n] = shape
+                if lay.mlp_bias:
+                    out[p + f"mlp.{n}.b"] = shape[:1]
+        out[p + "mix.o"] = (W, m.heads * m.vdim)
+        if not isinstance(m, LatentAttention):
+            rows = {"q": m.heads * m.dim, "k": m.kv_heads * m.dim, "v": m.kv_heads * m.vdim}
+            if isinstance(m, DeltaRule):
+                rows = {"q": m.kv_heads * m.dim, "k": m.kv_heads * m.dim, "v": m.heads * m.vdim}
+                for n in "qkv":
+                    out[p + f"mix.{n}.conv"] = (rows[n], m.taps)
+                out[p + "mix.A_log"] = out[p + "mix.dt_bias"] = (m.heads,)
+                out[p + "mix.norm"] = (m.vdim,)
+                rows.update(g=m.heads * m.vdim, b=m.heads, a=m.heads)
+            elif m.bias is not None:
+                out[p + "mix.rel"] = (m.bias.buckets, m.heads)
+            for n, r in rows.items():
+                out[p + "mix." + n] = (r, W)
+            continue
         out[p + "mix.dq"], out[p + "mix.dq.norm"] = (m.q_rank, W), (m.q_rank,)
         out[p + "mix.uq"] = (m.heads * (m.dim + m.rot_dim), m.q_rank)
         if m.kv_from is None:
@@ -364,99 +460,161 @@ def decoder_tensors(cfg: DecoderConfig) -> Dict[str, Tuple[int, ...]]:
             out[p + "mix.sink"] = (m.heads,)
         if m.gate:
             out[p + "mix.g"] = (m.heads, W)
-        out[p + "mix.o"] = (W, m.heads * m.vdim)
-        if lay.ff:
-            out[p + "norm2"] = (W,)
-            if lay.post_norm:
-                out[p + "norm2b"] = (W,)
-            for n, shape in (("gate", (lay.ff, W)), ("up", (lay.ff, W)), ("down", (W, lay.ff))):
-                out[p + "mlp." + n] = shape
-                if lay.mlp_bias:
-                    out[p + f"mlp.{n}.b"] = shape[:1]
     return out
 
 
 class PackedDecoder:
-    """decoder_tensors -> the layouts of include/cogs.h (cogs_decoder_*): padded sizes, stacked down projections, rotary pairs
-    adjacent, gate / up rows interleaved, W_uk also transposed per head for the absorbed decode"""
+    """decoder_tensors -> the layouts of include/cogs.h (cogs_decoder_*): padded sizes, projections of a mixer stacked, rotary pairs
+    adjacent, gate / up rows interleaved, W_uk also transposed per head for the absorbed decode, bias tables by distance"""
 
     def __init__(self, state: Dict[str, torch.Tensor], cfg: DecoderConfig, dtype=torch.bfloat16, device="cuda"):
         self.cfg, self.dtype, self.device = cfg, dtype, torch.device(device)
         self.keep: List[object] = []
+        self.state = state
         self.width_p, self.vocab_p = _up(cfg.width, 64), _up(cfg.vocab_size, 4)
         Wp = self.width_p
-
-        def hold(t):
-            t = t.contiguous()
-            self.keep.append(t)
-            return t
-
-        g = lambda k: state[k].to(device=self.device, dtype=dtype)
-        vec = lambda k, n: hold(_pad_to(state[k].to(device=self.device, dtype=torch.float32), n)).data_ptr()
-        self.embed = hold(_pad_to(g("embed"), cfg.vocab_size, Wp))
-        self.head = hold(_pad_to(g("head"), self.vocab_p, Wp))
+        self.embed = self._hold(_pad_to(self._get("embed"), cfg.vocab_size, Wp))
+        self.head = self._hold(_pad_to(self._get("head"), self.vocab_p, Wp))
         self.layers = (L.DecoderLayer * len(cfg.layers))()
+        widths: List[List[int]] = []          # per layer: columns of its blocks in a token's cache
+        states: List[int] = []                # per layer: floats of recurrent state
         for i, lc in enumerate(cfg.layers):
             p, lay, m = f"l{i}.", self.layers[i], lc.mixer
-            if m.rot.dims != m.rot_dim:
-                raise ValueError(f"layer {i}: rotation over {m.rot.dims} dimensions, rotated part of {m.rot_dim}")
-            a = p + "mix."
-            qrp, kvp, rotc, hp = _up(m.q_rank, 64), _up(m.kv_rank, 64), _up(m.rot_dim, 32), _up(m.heads, 4)
-            dn, dk, dv = _up(m.dim, 8), _up(m.dim, 32), _up(m.vdim, 16)
-            dq = dk + rotc
-            order = m.rot.pair_order().to(self.device)
-            lay.norm1 = vec(p + "norm1", Wp)
-            if lc.post_norm:
-                lay.norm1b = vec(p + "norm1b", Wp)
-            x = lay.mixer
-            x.heads, x.dim, x.rot_dim, x.vdim, x.q_rank, x.kv_rank = m.heads, m.dim, m.rot_dim, m.vdim, m.q_rank, m.kv_rank
-            x.kv_from, x.gated = -1 if m.kv_from is None else m.kv_from, int(m.gate)
-            x.scale, x.rot_mag = m.scale, m.rot.magnitude
-            freq = (C.c_double * (m.rot_dim // 2))(*m.rot.frequencies())
-            self.keep.append(freq)
-            x.rot_freq = C.cast(freq, C.POINTER(C.c_double))
-            rows = [_pad_to(g(a + "dq"), qrp, Wp)]
-            x.q_norm = vec(a + "dq.norm", qrp)
-            if m.kv_from is None:
-                d = g(a + "dkv")
-                rows += [_pad_to(d[:m.kv_rank], kvp, Wp), _pad_to(d[m.kv_rank:][order], rotc, Wp)]
-                x.kv_norm = vec(a + "dkv.norm", kvp)
-            if m.gate:
-                rows.append(_pad_to(g(a + "g"), hp, Wp))
-            x.in_w = hold(torch.cat(rows, 0)).data_ptr()
-            uq = g(a + "uq").view(m.heads, m.dim + m.rot_dim, m.q_rank)
-            q = uq.new_zeros(m.heads, dq, qrp)
-            q[:, :m.dim, :m.q_rank] = uq[:, :m.dim]
-            q[:, dk:dk + m.rot_dim, :m.q_rank] = uq[:, m.dim:][:, order]
-            x.q_w = hold(q.view(m.heads * dq, qrp)).data_ptr()
-            uk = g(a + "uk").view(m.heads, m.dim, m.kv_rank)
-            uv = g(a + "uv").view(m.heads, m.vdim, m.kv_rank)
-            x.kv_w = hold(torch.cat([_pad_to(uk, m.heads, dn, kvp).view(-1, kvp), _pad_to(uv, m.heads, dv, kvp).view(-1, kvp)], 0)).data_ptr()
-            x.k_abs = hold(_pad_to(uk.transpose(1, 2), m.heads, kvp, dk)).data_ptr()
-            if m.sink:
-                x.sink = hold(state[a + "sink"].to(device=self.device, dtype=torch.float32) * math.log2(math.e)).data_ptr()
-            o = _pad_to(g(a + "o").view(cfg.width, m.heads, m.vdim), Wp, m.heads, dv).view(Wp, m.heads * dv)
-            x.o_w = hold(_pad_to(o, Wp, _up(m.heads * dv, 64))).data_ptr()
-            if lc.ff:
-                ffp = _up(lc.ff, 64)
-                lay.norm2 = vec(p + "norm2", Wp)
+            for n in ("1", "2") if lc.ff else ("1",):
+                setattr(lay, "norm" + n, self._vec(p + "norm" + n, Wp))
                 if lc.post_norm:
-                    lay.norm2b = vec(p + "norm2b", Wp)
-                f = p + "mlp."
-                gu = torch.stack([_pad_to(g(f + "gate"), ffp, Wp), _pad_to(g(f + "up"), ffp, Wp)], dim=1)
-                lay.mlp.ff, lay.mlp.gu_w = lc.ff, hold(gu.view(2 * ffp, Wp)).data_ptr()
-                lay.mlp.down_w = hold(_pad_to(g(f + "down"), Wp, ffp)).data_ptr()
-                if lc.mlp_bias:
-                    gb = torch.stack([_pad_to(g(f + "gate.b"), ffp), _pad_to(g(f + "up.b"), ffp)], dim=1)
-                    lay.mlp.gu_b = hold(gb.view(2 * ffp)).data_ptr()
-                    lay.mlp.down_b = hold(_pad_to(g(f + "down.b"), Wp)).data_ptr()
+                    setattr(lay, f"norm{n}b", self._vec(p + f"norm{n}b", Wp))
+                if cfg.streams:
+                    s, hc = cfg.streams, getattr(lay, "hyper" + n)
+                    hc.in_, hc.out = self._vec(p + f"hc{n}.in", s), self._vec(p + f"hc{n}.out", s)
+                    hc.mix = self._vec(p + f"hc{n}.mix", s, s)
+            if isinstance(m, LatentAttention):
+                lay.mixer = L.MIX_LATENT
+                blocks, floats = self._latent(lay.latent, p + "mix.", m, i)
+            elif isinstance(m, HeadAttention):
+                lay.mixer = L.MIX_ATTENTION
+                blocks, floats = self._heads(lay.attn, p + "mix.", m)
+            else:
+                lay.mixer = L.MIX_DELTA
+                blocks, floats = self._delta(lay.delta, p + "mix.", m)
+            widths.append(blocks)
+            states.append(floats)
+            dv = _up(m.vdim, 16)
+            o = _pad_to(self._get(p + "mix.o").view(cfg.width, m.heads, m.vdim), Wp, m.heads, dv).view(Wp, m.heads * dv)
+            getattr(lay, ("latent", "attn", "delta")[lay.mixer]).o_w = self._hold(_pad_to(o, Wp, _up(m.heads * dv, 64))).data_ptr()
+            if lc.ff:
+                self._mlp(lay.mlp, p + "mlp.", lc)
         w = L.DecoderWeights()
         w.dtype, w.width, w.vocab, w.layers, w.eps = L.dtype_code(dtype), cfg.width, cfg.vocab_size, len(cfg.layers), cfg.eps
-        w.final_norm, w.head = vec("final.norm", Wp), self.head.data_ptr()
+        w.embed_scale, w.max_positions, w.streams = cfg.embed_scale, cfg.max_positions, cfg.streams
+        if cfg.max_positions:
+            w.pos = self._hold(_pad_to(self._get("pos"), cfg.max_positions, Wp)).data_ptr()
+        if cfg.loop is not None:
+            w.loop_start, w.loop_stop, w.loop_times = cfg.loop.start, cfg.loop.stop, cfg.loop.times
+        w.final_norm, w.head = self._vec("final.norm", Wp), self.head.data_ptr()
         w.layer = C.cast(self.layers, C.POINTER(L.DecoderLayer))
         self.struct = w
-        # columns of every cached layer's block in a token's cache, in layer order
-        self.cache_widths = [_up(lc.mixer.kv_rank, 64) + _up(lc.mixer.rot_dim, 32) for lc in cfg.layers if lc.mixer.kv_from is None]
+        del self.state
+        # columns of every cached block in a token's cache, and floats of state, in the order of the layer runs
+        self.cache_widths = [b for i in cfg.runs() for b in widths[i]]
+        self.state_floats = sum(states[i] for i in cfg.runs())
+
+    def _hold(self, t: torch.Tensor) -> torch.Tensor:
+        t = t.contiguous()
+        self.keep.append(t)
+        return t
+
+    def _get(self, k: str) -> torch.Tensor:
+        return self.state[k].to(device=self.device, dtype=self.dtype)
+
+    def _f32(self, k: str) -> torch.Tensor:
+        return self.state[k].to(device=self.device, dtype=torch.float32)
+
+    def _vec(self, k: str, *shape: int) -> int:
+        return self._hold(_pad_to(self._f32(k), *shape)).data_ptr()
+
+    def _head_rows(self, k: str, heads: int, n: int, padded: int) -> torch.Tensor:
+        """[heads * n, width] -> [heads * padded, width_p]"""
+        return _pad_to(self._get(k).view(heads, n, self.cfg.width), heads, padded, self.width_p).view(heads * padded, self.width_p)
+
+    def _latent(self, x, a: str, m: LatentAttention, i: int):
+        if m.rot.dims != m.rot_dim:
+            raise ValueError(f"layer {i}: rotation over {m.rot.dims} dimensions, rotated part of {m.rot_dim}")
+        g, hold, Wp = self._get, self._hold, self.width_p
+        qrp, kvp, rotc, hp = _up(m.q_rank, 64), _up(m.kv_rank, 64), _up(m.rot_dim, 32), _up(m.heads, 4)
+        dn, dk, dv = _up(m.dim, 8), _up(m.dim, 32), _up(m.vdim, 16)
+        dq = dk + rotc
+        order = m.rot.pair_order().to(self.device)
+        x.heads, x.dim, x.rot_dim, x.vdim, x.q_rank, x.kv_rank = m.heads, m.dim, m.rot_dim, m.vdim, m.q_rank, m.kv_rank
+        x.kv_from, x.gated = -1 if m.kv_from is None else m.kv_from, int(m.gate)
+        x.scale, x.rot_mag = m.scale, m.rot.magnitude
+        freq = (C.c_double * (m.rot_dim // 2))(*m.rot.frequencies())
+        self.keep.append(freq)
+        x.rot_freq = C.cast(freq, C.POINTER(C.c_double))
+        rows = [_pad_to(g(a + "dq"), qrp, Wp)]
+        x.q_norm = self._vec(a + "dq.norm", qrp)
+        if m.kv_from is None:
+            d = g(a + "dkv")
+            rows += [_pad_to(d[:m.kv_rank], kvp, Wp), _pad_to(d[m.kv_rank:][order], rotc, Wp)]
+            x.kv_norm = self._vec(a + "dkv.norm", kvp)
+        if m.gate:
+            rows.append(_pad_to(g(a + "g"), hp, Wp))
+        x.in_w = hold(torch.cat(rows, 0)).data_ptr()
+        uq = g(a + "uq").view(m.heads, m.dim + m.rot_dim, m.q_rank)
+        q = uq.new_zeros(m.heads, dq, qrp)
+        q[:, :m.dim, :m.q_rank] = uq[:, :m.dim]
+        q[:, dk:dk + m.rot_dim, :m.q_rank] = uq[:, m.dim:][:, order]
+        x.q_w = hold(q.view(m.heads * dq, qrp)).data_ptr()
+        uk = g(a + "uk").view(m.heads, m.dim, m.kv_rank)
+        uv = g(a + "uv").view(m.heads, m.vdim, m.kv_rank)
+        x.kv_w = hold(torch.cat([_pad_to(uk, m.heads, dn, kvp).view(-1, kvp), _pad_to(uv, m.heads, dv, kvp).view(-1, kvp)], 0)).data_ptr()
+        x.k_abs = hold(_pad_to(uk.transpose(1, 2), m.heads, kvp, dk)).data_ptr()
+        if m.sink:
+            x.sink = hold(self._f32(a + "sink") * math.log2(math.e)).data_ptr()
+        return [kvp + rotc] if m.kv_from is None else [], 0
+
+    def _heads(self, x, a: str, m: HeadAttention):
+        dk, dv = _up(m.dim, 32), _up(m.vdim, 16)
+        x.heads, x.kv_heads, x.dim, x.vdim, x.scale = m.heads, m.kv_heads, m.dim, m.vdim, m.scale
+        x.qk_norm, x.temp_coef, x.temp_every = int(m.qk_norm), m.temp_coef, m.temp_every
+        x.in_w = self._hold(torch.cat([self._head_rows(a + "q", m.heads, m.dim, dk), self._head_rows(a + "k", m.kv_heads, m.dim, dk),
+                                       self._head_rows(a + "v", m.kv_heads, m.vdim, dv)], 0)).data_ptr()
+        if m.bias is not None:
+            rows = torch.tensor(m.bias.bucket_of(), device=self.device)
+            x.dist_bias, x.dist_n = self._hold(self._f32(a + "rel")[rows].t() * math.log2(math.e)).data_ptr(), len(rows)
+        return [_up(dk + dv, 32)] * m.kv_heads, 0
+
+    def _delta(self, x, a: str, m: DeltaRule):
+        dk, dv, hp = _up(m.dim, 16), _up(m.vdim, 16), _up(m.heads, 4)
+        x.heads, x.kv_heads, x.dim, x.vdim, x.taps = m.heads, m.kv_heads, m.dim, m.vdim, m.taps
+        parts = (("q", m.kv_heads, m.dim, dk), ("k", m.kv_heads, m.dim, dk), ("v", m.heads, m.vdim, dv))
+        x.in_w = self._hold(torch.cat([self._head_rows(a + n, *s) for n, *s in parts + (("g", m.heads, m.vdim, dv),)] +
+                                      [_pad_to(self._get(a + n), hp, self.width_p) for n in "ba"], 0)).data_ptr()
+        conv = [_pad_to(self._f32(a + n + ".conv").view(h, d, m.taps), h, dp, m.taps).view(h * dp, m.taps) for n, h, d, dp in parts]
+        x.conv = self._hold(torch.cat(conv, 0).t()).data_ptr()
+        x.neg_a, x.dt_bias = self._hold(-torch.exp(self._f32(a + "A_log"))).data_ptr(), self._vec(a + "dt_bias", m.heads)
+        x.norm = self._vec(a + "norm", dv)
+        channels = 2 * m.kv_heads * dk + m.heads * dv
+        return [], m.heads * dk * dv + m.taps * channels
+
+    def _mlp(self, x, f: str, lc: DecoderLayerConfig):
+        g, hold, Wp, ffp = self._get, self._hold, self.width_p, _up(lc.ff, 64)
+        pad = lambda n: _pad_to(g(f + n), ffp, Wp)
+        bias = lambda n: _pad_to(g(f + n + ".b"), ffp)
+        x.ff = lc.ff
+        if lc.mlp_act == "swiglu":
+            x.act = L.ACT_SWIGLU
+            x.up_w = hold(torch.stack([pad("gate"), pad("up")], dim=1).view(2 * ffp, Wp)).data_ptr()
+            if lc.mlp_bias:
+                x.up_b = hold(torch.stack([bias("gate"), bias("up")], dim=1).view(2 * ffp)).data_ptr()
+        else:
+            x.act = {"gelu": L.ACT_GELU_ERF}[lc.mlp_act]
+            x.up_w = hold(pad("up")).data_ptr()
+            if lc.mlp_bias:
+                x.up_b = hold(bias("up")).data_ptr()
+        x.down_w = hold(_pad_to(g(f + "down"), Wp, ffp)).data_ptr()
+        if lc.mlp_bias:
+            x.down_b = hold(_pad_to(g(f + "down.b"), Wp)).data_ptr()
 
 
 # ---- random initialisation at arbitrary dimensions (no checkpoints are reachable: README.md:56-58) ----

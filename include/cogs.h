@@ -426,19 +426,22 @@ cogs_status cogs_llm_forward_segments(cogs_handle h, cogs_stream stream, const v
 
 /* ------------------------------------- decoder-only models described layer by layer ------ */
 
-/* A pre-normed decoder whose layers are listed one by one, each with a mixer and an optional gated MLP and optional norms on
- * the sublayers' outputs:
+/* A pre-normed decoder whose layers are listed one by one, each with a mixer and an optional MLP and optional norms on the
+ * sublayers' outputs:
  *     x += norm1b(mixer(norm1(x)));   x += norm2b(mlp(norm2(x)));   logits = head . final_norm(x)
- * The residual stream x, every norm, rotary angle, softmax and gate is fp32; matrix products take `dtype` operands.
+ * or, with hyper-connected residual streams x_1 .. x_s (all equal to the embedding at the start, summed at the end):
+ *     y = sublayer(norm(sum_s in[s] x_s));   x_t = sum_s mix[s][t] x_s + out[t] y
+ * The residual stream x, every norm, rotary angle, softmax, gate of a recurrence and recurrent state is fp32; matrix products
+ * take `dtype` operands.
  *
- * Padding (zeros, in weights, embeddings and norm vectors): width_p = width and ff_p = ff to a multiple of 64, vocab_p to 4;
- * q_rank_p and kv_rank_p to 64; rot_c = rot_dim to 32 (its columns in the cache); dim_p = dim and rot_p = rot_dim to 8;
- * dim_k = dim to 32; dq = dim_k + rot_c; vdim_p = vdim to 16; o_in = heads * vdim_p to 64; heads_p = heads to 4.
- * Norm vectors are fp32; everything else is in `dtype`.
+ * Padding (zeros, in weights, embeddings and norm vectors): width_p = width and ff_p = ff to a multiple of 64, vocab_p to 4.
+ * Norm vectors are fp32; everything else is in `dtype` unless stated.
  *
  * cogs_latent_mixer: multi-head latent attention. Per token a row [latent (kv_rank_p) | rotated key part (rot_c)] is cached;
  * keys and values of all heads are linear images of the latent. Rotated dimensions are packed as adjacent pairs (2i, 2i+1),
  * whatever pairs the model rotates (the packer permutes the rows of q_w and in_w alike).
+ * q_rank_p and kv_rank_p to 64; rot_c = rot_dim to 32 (its columns in the cache); dim_p = dim and rot_p = rot_dim to 8;
+ * dim_k = dim to 32; dq = dim_k + rot_c; vdim_p = vdim to 16; o_in = heads * vdim_p to 64; heads_p = heads to 4.
  *   in_w   [q_rank_p | kv_rank_p | rot_c | heads_p][width_p]: query latent, kv latent, rotated key part (the middle two absent
  *          with kv_from >= 0), gate logits (absent unless gated), stacked in this order
  *   q_w    [heads][dim_k | rot_c][q_rank_p]
@@ -460,28 +463,80 @@ typedef struct {
     const float* sink;
     const void* o_w;
 } cogs_latent_mixer;
-/* gu_w [2 * ff_p, width_p] rows interleaved (gate_i, up_i), gu_b likewise; down_w [width_p, ff_p]; biases nullable; ff = 0: none */
-typedef struct { int ff; const void *gu_w, *gu_b, *down_w, *down_b; } cogs_gated_mlp;
+/* cogs_attn_mixer: softmax attention with keys and values per head; query head h reads key / value head h / (heads / kv_heads).
+ * dim_k = dim to 32, vdim_p = vdim to 16, o_in = heads * vdim_p to 64. Cached per token and key / value head: a row
+ * [key (dim_k) | value (vdim_p)] to 32 columns.
+ *   in_w   [heads * dim_k | kv_heads * dim_k | kv_heads * vdim_p][width_p]
+ *   o_w    [width_p][o_in]
+ *   qk_norm     every query and key head row is divided by its root mean square (eps of the decoder)
+ *   temp_every  > 0: queries at position p times 1 + temp_coef * ln(floor((p + 1) / temp_every) + 1)
+ *   dist_bias   fp32 [heads][dist_n], times log2(e), or NULL: added to the scaled score of a key n positions back is
+ *               entry min(n, dist_n - 1) */
+typedef struct {
+    int heads, kv_heads, dim, vdim;
+    int qk_norm;
+    float scale;
+    double temp_coef, temp_every;
+    const float* dist_bias;
+    int dist_n;
+    const void *in_w, *o_w;
+} cogs_attn_mixer;
+/* cogs_delta_mixer: gated delta rule. Per head a matrix S [dim][vdim] and per token
+ *     S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+ * with q, k, v behind a causal convolution over the last `taps` tokens per channel and silu, q and k of unit length per head
+ * (q times dim^-1/2), beta a sigmoid, g = exp(neg_a softplus(a + dt_bias)); the head's output is o over its root mean square,
+ * times norm, times silu(gate). Head h reads q / k head h / (heads / kv_heads).
+ * dim_p = dim and vdim_p = vdim to 16, o_in = heads * vdim_p to 64, heads_p = heads to 4, channels = 2 kv_heads dim_p + heads vdim_p.
+ *   in_w   [kv_heads * dim_p | kv_heads * dim_p | heads * vdim_p | heads * vdim_p | heads_p | heads_p][width_p]: q, k, v, gate, beta, a
+ *   conv   fp32 [taps][channels], the last tap is the current token's;  neg_a, dt_bias fp32 [heads];  norm fp32 [vdim_p]
+ *   o_w    [width_p][o_in]
+ * State per sequence, fp32: S [heads][dim_p][vdim_p], then the convolution's last inputs [taps][channels], position p in row p % taps. */
+typedef struct {
+    int heads, kv_heads, dim, vdim, taps;
+    const void* in_w;
+    const float *conv, *neg_a, *dt_bias, *norm;
+    const void* o_w;
+} cogs_delta_mixer;
+/* ff = 0: none. act COGS_ACT_SWIGLU: gated, up_w [2 * ff_p, width_p] rows interleaved (gate_i, up_i), up_b likewise; other
+ * activations: up_w [ff_p, width_p], up_b [ff_p]. down_w [width_p, ff_p]; biases nullable */
+typedef struct { int ff, act; const void *up_w, *up_b, *down_w, *down_b; } cogs_decoder_mlp;
+/* fp32 device vectors of a sublayer's hyper-connections: in [streams], out [streams], mix [streams (from)][streams (to)] */
+typedef struct { const float *in, *out, *mix; } cogs_hyper;
+enum { COGS_MIX_LATENT = 0, COGS_MIX_ATTENTION = 1, COGS_MIX_DELTA = 2 };
 typedef struct {
     const float *norm1, *norm1b, *norm2, *norm2b;      /* norm1b, norm2b nullable: the sublayer's output is added as it is */
-    cogs_latent_mixer mixer;
-    cogs_gated_mlp mlp;
+    cogs_hyper hyper1, hyper2;                         /* mixer, MLP; read with streams > 0 */
+    int mixer;                                         /* COGS_MIX_*: which of the three below is meant */
+    cogs_latent_mixer latent;
+    cogs_attn_mixer attn;
+    cogs_delta_mixer delta;
+    cogs_decoder_mlp mlp;
 } cogs_decoder_layer;
 typedef struct {
     int dtype, width, vocab, layers;
     float eps;
+    float embed_scale;                                 /* x starts as embeds * embed_scale + pos[position] */
+    const void* pos;                                   /* [max_positions][width_p] or NULL */
+    int max_positions;                                 /* longest sequence, 0: no limit */
+    int streams;                                       /* hyper-connected residual streams, 0: one plain residual stream */
+    int loop_start, loop_stop, loop_times;             /* layers loop_start .. loop_stop - 1 run loop_times times in a row, each pass
+                                                          with a cache and state of its own; loop_times <= 1: once */
     const float* final_norm;
     const void* head;                                  /* [vocab_p][width_p] */
     const cogs_decoder_layer* layer;                   /* host array [layers] */
 } cogs_decoder_weights;
 cogs_status cogs_decoder_load(cogs_handle h, const cogs_decoder_weights* w);
-/* elements per token of a sequence's cache (all cached layers). A cache is a cogs_kv with k = max_len * this many elements, v unused */
+/* Layer runs: `layers` plus the repeated passes of the loop. A sequence's cache is a cogs_kv with k = max_len * `elements` of `dtype`
+ * (rows of every layer run that caches rows) and v = `bytes` of recurrent state (may be NULL if 0; read only behind position 0, so
+ * it needs no clearing). Rows may be cut back by lowering len; a state belongs to exactly the len it was left at. */
 cogs_status cogs_decoder_cache_width(cogs_handle h, int64_t* elements);
+cogs_status cogs_decoder_state_bytes(cogs_handle h, int64_t* bytes);
 cogs_status cogs_decoder_workspace_bytes(cogs_handle h, int rows, int nseq, int64_t total_context, int n_want, size_t* bytes);
 /* One step of `nseq` sequences: sequence i brings lens[i] >= 1 new tokens as rows of embeds [sum lens, width_p] (sequences back
  * to back), at positions kv[i]->len ..; its cache rows are appended and kv[i]->len advances. No padding, any mix of lengths.
- * want (host [n_want], row numbers) -> logits fp32 [n_want][vocab_p]. streams, nullable: fp32 [layers][rows][width_p], the
- * residual stream behind every layer. Steps of one token per sequence take the absorbed form of latent attention. */
+ * want (host [n_want], row numbers) -> logits fp32 [n_want][vocab_p]. streams, nullable: fp32 [layer runs][rows][width_p], the
+ * residual stream (the sum of the streams) behind every layer run. Steps of one token per sequence take the absorbed form of
+ * latent attention. */
 cogs_status cogs_decoder_forward(cogs_handle h, cogs_stream stream, const void* embeds, cogs_kv* const* kv, const int32_t* lens, int nseq,
                                  const int32_t* want, int n_want, float* logits, float* streams, void* ws, size_t ws_bytes);
 

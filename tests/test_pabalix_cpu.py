@@ -58,7 +58,7 @@ def test_packed_layouts_give_the_same_projections(name):
     hp = torch.zeros(5, Wp)
     hp[:, :W] = h
     for i, lay in enumerate(cfg["layers"]):
-        m, x, pre = lay["mixer"], pk.layers[i].mixer, f"l{i}.mix."
+        m, x, pre = lay["mixer"], pk.layers[i].latent, f"l{i}.mix."
         qrp, kvp, rc = up(m["q_rank"], 64), up(m["kv_rank"], 64), up(m["rot_dim"], 32)
         dn, dk, dv = up(m["dim"], 8), up(m["dim"], 32), up(m["vdim"], 16)
         dq, H, own = dk + rc, m["heads"], m.get("kv_from") is None
@@ -95,7 +95,7 @@ def test_packed_layouts_give_the_same_projections(name):
         if lay["mlp"] is not None:
             ml, f = pk.layers[i].mlp, f"l{i}.mlp."
             ffp = up(ml.ff, 64)
-            gu = hp @ _view(ml.gu_w, (2 * ffp, Wp), pk).T + _view(ml.gu_b, (2 * ffp,), pk)
+            gu = hp @ _view(ml.up_w, (2 * ffp, Wp), pk).T + _view(ml.up_b, (2 * ffp,), pk)
             a = torch.nn.functional.silu(gu[:, 0::2]) * gu[:, 1::2]
             y = a @ _view(ml.down_w, (Wp, ffp), pk).T + _view(ml.down_b, (Wp,), pk)
             assert torch.allclose(y[:, :W], po.feed_forward(h, st, f), atol=1e-4) and not y[:, W:].any()
@@ -109,9 +109,10 @@ def test_ctypes_structs_match_the_header(tmp_path):
     from cogstream_amd import _lib as L
     if shutil.which("gcc") is None:
         pytest.skip("no gcc")
-    names = {"cogs_latent_mixer": L.LatentMixer, "cogs_gated_mlp": L.GatedMlp, "cogs_decoder_layer": L.DecoderLayer,
+    names = {"cogs_latent_mixer": L.LatentMixer, "cogs_attn_mixer": L.AttnMixer, "cogs_delta_mixer": L.DeltaMixer, "cogs_hyper": L.Hyper,
+             "cogs_decoder_mlp": L.DecoderMlp, "cogs_decoder_layer": L.DecoderLayer,
              "cogs_decoder_weights": L.DecoderWeights, "cogs_kv": L.KV}
-    lines = [f'printf("{n} %zu", sizeof({n}));' + "".join(f'printf(" %zu", offsetof({n}, {f[0]}));' for f in t._fields_) + 'printf("\\n");'
+    lines = [f'printf("{n} %zu", sizeof({n}));' + "".join(f'printf(" %zu", offsetof({n}, {f[0].rstrip("_")}));' for f in t._fields_) + 'printf("\\n");'
              for n, t in names.items()]
     src = tmp_path / "t.c"
     src.write_text('#include <stdio.h>\n#include <stddef.h>\n#include "cogs.h"\nint main(void) {' + "\n".join(lines) + "return 0; }\n")
