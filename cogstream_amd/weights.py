@@ -668,14 +668,20 @@ def random_llm_state(cfg: LlmConfig, seed: int = 2, device="cpu", dtype=torch.fl
 
 
 def random_decoder_state(cfg: DecoderConfig, seed: int = 3, device="cpu", dtype=torch.float32, std: Optional[float] = None):
-    """decoder_tensors with norms near one and matrices of standard deviation `std` (default 1 / sqrt(inputs))"""
+    """decoder_tensors with norms near one and matrices of standard deviation `std` (default 1 / sqrt(inputs)); embeddings and bias
+    tables of deviation one, hyper-connections that keep the streams' size, decays of a few to a few hundred tokens"""
     g = torch.Generator(device=device).manual_seed(seed)
     st = {}
     for name, shape in decoder_tensors(cfg).items():
         t = torch.randn(*shape, generator=g, device=device, dtype=torch.float32)
-        if "norm" in name.rsplit(".", 1)[-1]:
+        last = name.rsplit(".", 1)[-1]
+        if "norm" in last:
             t = 1 + 0.1 * t
-        elif len(shape) == 2 and name != "embed":
+        elif name.split(".")[1:2] in (["hc1"], ["hc2"]):
+            t = 0.3 * t + {"in": shape[-1] ** -0.5, "out": 1.0, "mix": 0.7 * torch.eye(shape[-1], device=device)}[last]
+        elif last == "A_log":
+            t = t - 2
+        elif len(shape) == 2 and last not in ("embed", "pos", "rel"):
             t = t * (shape[1] ** -0.5 if std is None else std)
         elif name.endswith(".b"):
             t = t * 0.1
