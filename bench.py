@@ -451,15 +451,37 @@ def pabalix_config(width, heads, q_rank, kv_rank, ff, layers):
     return dict(architecture="Pabalix", layers=out, norm=dict(eps=1e-6), vocab=PABALIX_VOCAB, width=width)
 
 
-def bench_pabalix(args, dev):
-    """prefill (one prompt of 4096 tokens) and decode (behind 4096 tokens; 1 and 16 sequences) tokens/s of the engine's own steps,
-    greedy token choice included, Pabalix and the equal-size Qwen2 model timed in turn; per-class GPU time from event brackets"""
+# (name, width, heads, ff, Qwen2's ff, layers): heads of 128, a quarter of them as key/value heads in attention, half as q/k heads in delta
+# layers; every fourth layer is attention. Qwen2's gated feed-forward has the same number of weights (three matrices against two)
+LUPANEX_SIZES = [("w2048", 2048, 16, 8448, 5632, 8), ("w3584", 3584, 28, 28416, 18944, 4), ("w4096", 4096, 32, 16512, 11008, 8)]
+LUPANEX_VOCAB = 32768
+
+
+def lupanex_config(width, heads, ff, layers, positions):
+    """-> (config.json, the shapes it leaves to the tensors)"""
+    out = []
+    for i in range(layers):
+        if i % 4 == 3:
+            mx = dict(heads=heads, kv_heads=heads // 4, dim=128, vdim=128, scale=128 ** -0.5, bias_max=128, q_temp=dict(coef=0.1, every=2048))
+        else:
+            mx = dict(heads=heads, kv_heads=heads // 2, dim=128, vdim=128, conv=4)
+        out.append(dict(type="attention" if i % 4 == 3 else "delta", mixer=mx, mlp=dict(kind="dense", ff=ff)))
+    cfg = dict(architecture="Lupanex", layers=out, norm=dict(eps=1e-6), vocab=LUPANEX_VOCAB, width=width, streams=4, embedding=dict(scale=1.0),
+               max_positions=positions)
+    return cfg, {f"l{i}.mix.rel": (32, heads) for i in range(3, layers, 4)}
+
+
+def bench_decoder(args, dev):
+    """a decoder described layer by layer beside an equal-size Qwen2 model, timed in turn: prefill (one prompt of 4096 tokens) and decode
+    (behind 4096 tokens; 1 and 16 sequences) tokens/s of the engines' own steps, greedy token choice included; per-class GPU time
+    from event brackets"""
     from cogstream_amd import _lib as L
-    from cogstream_amd import ops
+    from cogstream_amd import lupanex, ops, pabalix
     from cogstream_amd.llm import DecoderEngine, Qwen2Engine
-    from cogstream_amd.pabalix import parse_config
     from cogstream_amd.weights import LlmConfig, random_decoder_state, random_llm_state
     S, ctx0 = 4096, 4096
+    design = args.config
+    vocab = {"pabalix": PABALIX_VOCAB, "lupanex": LUPANEX_VOCAB}[design]
     classes = ["gemm", "attention", "norm", "other"]
 
     def profile(h, fn):
@@ -472,7 +494,7 @@ def bench_pabalix(args, dev):
     def measure(e, batch_sizes):
         res = {}
         g = torch.Generator().manual_seed(0)
-        ids = torch.randint(0, PABALIX_VOCAB, (S,), generator=g)
+        ids = torch.randint(0, vocab, (S,), generator=g)
         cache = e.new_cache(S + 256)
         emb = e.embed_tokens(ids)
 
@@ -491,6 +513,7 @@ def bench_pabalix(args, dev):
             t.append(time.perf_counter() - t0)
         sec = sorted(t)[len(t) // 2]
         res["prefill"] = {"tokens_per_s": round(S / sec, 1), "ms": round(sec * 1e3, 3), "class_ms": profile(e.handle, prefill)}
+        behind = None if cache.state is None else cache.state.clone()
         for B in batch_sizes:
             caches = [cache]
             for _ in range(B - 1):
@@ -508,7 +531,7 @@ def bench_pabalix(args, dev):
             best = []
             for rep in range(args.warmup + args.steps):
                 for c in caches:
-                    c.reset(ctx0)
+                    c.restore(ctx0, behind)
                 torch.cuda.synchronize()
                 t0 = time.perf_counter()
                 for _ in range(n):
@@ -517,16 +540,23 @@ def bench_pabalix(args, dev):
                 if rep >= args.warmup:
                     best.append((time.perf_counter() - t0) / n)
             for c in caches:
-                c.reset(ctx0)
+                c.restore(ctx0, behind)
             sec = sorted(best)[len(best) // 2]
             res[f"decode_b{B}"] = {"tokens_per_s": round(B / sec, 1), "ms_per_step": round(sec * 1e3, 4), "class_ms": profile(e.handle, step)}
         return res
 
-    out = {"metric": "Pabalix prefill tokens/sec", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
+    out = {"metric": f"{design.capitalize()} prefill tokens/sec", "unit": "tokens/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
            "higher_is_better": True, "vs_baseline": None, "dtype": "bf16", "data": "synthetic tokens, random weights",
-           "config": {"prompt": S, "context": ctx0, "vocab": PABALIX_VOCAB}, "sizes": {}}
-    for name, width, heads, q_rank, kv_rank, ff, layers in PABALIX_SIZES:
-        dc = parse_config(pabalix_config(width, heads, q_rank, kv_rank, ff, layers))
+           "config": {"prompt": S, "context": ctx0, "vocab": vocab}, "sizes": {}}
+    if design == "pabalix":
+        sizes = [(name, pabalix.parse_config(pabalix_config(width, heads, q_rank, kv_rank, ff, layers)), ff,
+                  {"width": width, "heads": heads, "q_rank": q_rank, "kv_rank": kv_rank, "ff": ff, "layers": layers})
+                 for name, width, heads, q_rank, kv_rank, ff, layers in PABALIX_SIZES]
+    else:
+        sizes = [(name, lupanex.parse_config(*lupanex_config(width, heads, ff, layers, S + 256)), ff2,
+                  {"width": width, "heads": heads, "ff": ff, "qwen2_ff": ff2, "layers": layers})
+                 for name, width, heads, ff, ff2, layers in LUPANEX_SIZES]
+    for name, dc, ff2, desc in sizes:
         st = random_decoder_state(dc, seed=1, device=dev, dtype=torch.bfloat16)
         params = sum(v.numel() for v in st.values())
         e = DecoderEngine(st, dc, dtype=torch.bfloat16, device=dev)
@@ -534,16 +564,18 @@ def bench_pabalix(args, dev):
         mine = measure(e, (1, 16))
         del e
         torch.cuda.empty_cache()
-        lc = LlmConfig(hidden_size=width, intermediate_size=ff, num_hidden_layers=layers, num_attention_heads=heads,
-                       num_key_value_heads=heads // 4, vocab_size=PABALIX_VOCAB)
-        q = Qwen2Engine(random_llm_state(lc, seed=2, device=dev, dtype=torch.bfloat16), lc, dtype=torch.bfloat16, device=dev)
+        lc = LlmConfig(hidden_size=desc["width"], intermediate_size=ff2, num_hidden_layers=desc["layers"], num_attention_heads=desc["heads"],
+                       num_key_value_heads=desc["heads"] // 4, vocab_size=vocab)
+        st = random_llm_state(lc, seed=2, device=dev, dtype=torch.bfloat16)
+        desc["qwen2_parameters"] = sum(v.numel() for v in st.values())
+        q = Qwen2Engine(st, lc, dtype=torch.bfloat16, device=dev)
+        del st
         theirs = measure(q, (1, 16))
         del q
         torch.cuda.empty_cache()
-        out["sizes"][name] = {"width": width, "heads": heads, "q_rank": q_rank, "kv_rank": kv_rank, "ff": ff, "layers": layers,
-                              "parameters": params, "pabalix": mine, "qwen2": theirs}
-        print(f"[bench pabalix] {name} done", file=sys.stderr, flush=True)
-    last = out["sizes"][PABALIX_SIZES[-1][0]]["pabalix"]["prefill"]
+        out["sizes"][name] = dict(desc, parameters=params, **{design: mine, "qwen2": theirs})
+        print(f"[bench {design}] {name} done", file=sys.stderr, flush=True)
+    last = out["sizes"][sizes[-1][0]][design]["prefill"]
     out["value"], out["ms_per_step"] = last["tokens_per_s"], last["ms"]
     return out
 
@@ -562,11 +594,11 @@ def main() -> None:
     ap.add_argument("--scaling", default="strong", choices=["weak", "strong"],
                     help="N > 1 headline: strong = --frames in total (the metric's clip at every N; default), weak = --frames "
                          "per GPU (clip of frames*N)")
-    ap.add_argument("--config", default="cfg2", choices=["cfg2", "cfg3", "cfg5", "pabalix"],
+    ap.add_argument("--config", default="cfg2", choices=["cfg2", "cfg3", "cfg5", "pabalix", "lupanex"],
                     help="cfg2: BASELINE configs[1] (64-frame clip; the metric's config). cfg3: configs[2], one 256-frame "
                          "clip at the 16384-token budget (140x280 per frame) sharded over the ranks. cfg5: configs[4], one "
-                         "64-frame clip per GPU answered through the whole product API (replicas, no collective). pabalix: prefill and "
-                         "decode of Pabalix at sizes of real layers (random weights), beside Qwen2 layers of equal size")
+                         "64-frame clip per GPU answered through the whole product API (replicas, no collective). pabalix, lupanex: "
+                         "prefill and decode of that design at sizes of real layers (random weights), beside Qwen2 layers of equal size")
     ap.add_argument("--no-cfg3", action="store_true", help="skip the extra configs[2] measurement of the default run")
     ap.add_argument("--payload", default="projected", choices=["projected", "encoder"],
                     help="N > 1: what the all-gather carries (3584-wide projected tokens / 1152-wide encoder tokens, "
@@ -619,10 +651,10 @@ def main() -> None:
     debug_applied = L.debug_from_spec(args.debug)
     from cogstream_amd.parallel import frame_shards, gather_tokens
     from cogstream_amd.preprocess_gpu import preprocess_videos_gpu
-    if args.config == "pabalix":
+    if args.config in ("pabalix", "lupanex"):
         if world > 1:
-            raise SystemExit("--config pabalix runs on one GPU")
-        print(json.dumps(bench_pabalix(args, dev)), flush=True)
+            raise SystemExit(f"--config {args.config} runs on one GPU")
+        print(json.dumps(bench_decoder(args, dev)), flush=True)
         return
     if args.config == "cfg5":
         out = bench_cfg5(args, rank, world, dev, ranks_seen)

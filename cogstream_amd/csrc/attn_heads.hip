@@ -1,6 +1,6 @@
 // Head rows of softmax attention with per-head keys and values (cogs_attn_mixer) behind the fused projection: optional RMS norm of
-// every query and key head row (no weight), the query's temperature, the score scale in log2 units, and the cache rows. The attention
-// itself is mla.hip's.
+// every query and key head row (no weight), the query's temperature, the score scale in log2 units, and the cache rows, padding
+// included (a tile's rows past the end repeat a row's last columns under a weight of zero). The attention itself is mla.hip's.
 #include "common.h"
 #include "kernels.h"
 
@@ -18,7 +18,7 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
     const int total = p.heads + 2 * p.kv_heads;
     for (int j = wid; j < total; j += 4) {
         const bool is_q = j < p.heads, is_k = !is_q && j < p.heads + p.kv_heads;
-        const int kh = is_q ? 0 : (j - p.heads) % p.kv_heads, cols = is_q || is_k ? p.dkp : p.dvp;
+        const int kh = is_q ? 0 : (j - p.heads) % p.kv_heads, cols = is_q || is_k ? p.dkp : p.dvp, out_cols = is_q || is_k ? p.dkp : p.kvw - p.dkp;
         const T* x = t + (is_q || is_k ? (long)j * p.dkp : (long)(p.heads + p.kv_heads) * p.dkp + (long)kh * p.dvp);
         T* y = is_q ? reinterpret_cast<T*>(p.q) + (long)row * p.heads * p.dkp + (long)j * p.dkp
                     : reinterpret_cast<T*>(s.cache) + (p.layer_off + (long)kh * p.kvw) * s.max_len + (long)pos * p.kvw + (is_k ? 0 : p.dkp);
@@ -37,7 +37,7 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
 #pragma unroll
         for (int e = 0; e < E; ++e) {
             const int d = 4 * lane + 256 * e;
-            if (d < cols) st4_f<T>(y + d, v[e] * f);
+            if (d < out_cols) st4_f<T>(y + d, v[e] * f);
         }
     }
 }
@@ -53,7 +53,7 @@ void launch(hipStream_t st, const CogsAttnHeads& a, int rows, int cols) {
 
 int cogs_k_attn_heads(hipStream_t st, int dtype, const CogsAttnHeads& a, int rows) {
     if (rows <= 0) return COGS_OK;
-    const int cols = a.dkp > a.dvp ? a.dkp : a.dvp;
+    const int cols = a.dkp > a.kvw - a.dkp ? a.dkp : a.kvw - a.dkp;
     if (a.heads <= 0 || a.kv_heads <= 0 || a.dim <= 0 || a.dkp % 4 || a.dvp % 4 || a.ldt % 4 || a.kvw % 4 || a.dkp + a.dvp > a.kvw) return COGS_E_INVALID;
     if (cols > 2048) return COGS_E_UNSUPPORTED;
     if (dtype == COGS_DT_BF16) launch<bf16_t>(st, a, rows, cols);

@@ -678,7 +678,7 @@ def random_decoder_state(cfg: DecoderConfig, seed: int = 3, device="cpu", dtype=
         if "norm" in last:
             t = 1 + 0.1 * t
         elif name.split(".")[1:2] in (["hc1"], ["hc2"]):
-            t = 0.3 * t + {"in": shape[-1] ** -0.5, "out": 1.0, "mix": 0.7 * torch.eye(shape[-1], device=device)}[last]
+            t = 0.2 * t + {"in": shape[-1] ** -0.5, "out": 1.0, "mix": torch.eye(shape[-1], device=device)}[last]
         elif last == "A_log":
             t = t - 2
         elif len(shape) == 2 and last not in ("embed", "pos", "rel"):

@@ -16,7 +16,7 @@ from oracle import lupanex as lo
 pytestmark = pytest.mark.gpu
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 # largest row error of the logits. bfloat16: about twice what rounding the operands of the matrix products does to these models
-TOL = {torch.float32: 2e-5, torch.bfloat16: 4e-2}
+TOL = {torch.float32: 2e-5, torch.bfloat16: 2e-2}
 TINY = 2.5        # the eight-wide models have nothing to average rounding errors over
 DTYPES = [torch.float32, torch.bfloat16]
 LONG = {"wide": 100, "large": 100}
@@ -137,16 +137,16 @@ def alone(mech):
     elif mech == "hyper1":                 # a single stream with weights of its own
         cfg = config([attention(heads=2), delta(heads=2, kv_heads=1)], width=64, streams=1)
     elif mech == "loop":
-        cfg = config([delta(heads=2, kv_heads=2), attention(heads=2)], width=64, loop=(0, 1, 5))
+        cfg = config([delta(heads=2, kv_heads=2), attention(heads=2)], width=64, loop=(0, 1, 4))
     elif mech == "feed_forward":
         cfg = config([delta(heads=1, kv_heads=1, dim=4, vdim=4, ff=200)], width=64)
         st = state(cfg)
         st["l0.mix.o"] *= 0
         st["l0.mlp.up"] *= 2
     elif mech == "positions":              # one word over and over
-        cfg = config([attention(heads=2, ff=None)], width=64, vocab=1 + 1)
+        cfg = config([attention(heads=2, ff=None)], width=64)
         st = state(cfg)
-        st["embed"][1] = st["embed"][0]
+        st["embed"][:] = st["embed"][0]
     st = state(cfg) if st is None else st
     return cfg, {k: v.to(torch.bfloat16).float() for k, v in st.items()}
 
@@ -260,7 +260,7 @@ def test_a_write_is_read_back_from_any_distance(dev, dtype):
         if at is None:
             without = lg[ask]
         else:
-            assert rms_err(lg[ask:], without[None]) > 0.3
+            assert rms_err(lg[ask:], without[None]) > 0.2
         for cuts in ((), [ask], [32, 64, 97], [2, 3, ask - 2], [max(at or 1, 1), (at or 1) + 1] if (at or 1) + 1 < n else [at]):
             assert rms_err(run(e, toks, cuts)[ask:], lg[ask:]) < TOL[dtype], (at, cuts)
 

@@ -261,7 +261,7 @@ def test_faults_show_in_the_test_models(fault):
         for n in names:
             setattr(lo, n, saved[n])
     # (a state or key lost at one place is looked for right behind it; the last ones are small by nature and show in float32)
-    assert rms_err(bad[80:], good[80:]) > (0.005 if fault in ("temperature", "gelu_form") else 0.06)
+    assert rms_err(bad[80:], good[80:]) > (0.005 if fault in ("temperature", "gelu_form") else 0.035)
 
 
 def test_shapes_helper_names_every_attention_table():
