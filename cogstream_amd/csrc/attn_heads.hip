@@ -6,7 +6,7 @@
 
 namespace {
 
-// one workgroup per new row, a wave per head row (4 columns per lane and pass)
+// a wave per head row (4 columns per lane and pass); gridDim.y workgroups share a row's heads
 template <typename T, int E>
 __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
     const int row = blockIdx.x, lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
@@ -16,7 +16,7 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
     if (p.temp_every > 0.0) qs *= 1.f + (float)p.temp_coef * logf((float)(floor((pos + 1) / p.temp_every) + 1.0));
     const T* t = reinterpret_cast<const T*>(p.t) + (long)row * p.ldt;
     const int total = p.heads + 2 * p.kv_heads;
-    for (int j = wid; j < total; j += 4) {
+    for (int j = blockIdx.y * 4 + wid; j < total; j += 4 * gridDim.y) {
         const bool is_q = j < p.heads, is_k = !is_q && j < p.heads + p.kv_heads;
         const int kh = is_q ? 0 : (j - p.heads) % p.kv_heads, cols = is_q || is_k ? p.dkp : p.dvp, out_cols = is_q || is_k ? p.dkp : p.kvw - p.dkp;
         const T* x = t + (is_q || is_k ? (long)j * p.dkp : (long)(p.heads + p.kv_heads) * p.dkp + (long)kh * p.dvp);
@@ -44,9 +44,10 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
 
 template <typename T>
 void launch(hipStream_t st, const CogsAttnHeads& a, int rows, int cols) {
-    if (cols <= 256) hipLaunchKernelGGL((attn_heads_kernel<T, 1>), dim3(rows), dim3(256), 0, st, a);
-    else if (cols <= 512) hipLaunchKernelGGL((attn_heads_kernel<T, 2>), dim3(rows), dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((attn_heads_kernel<T, 8>), dim3(rows), dim3(256), 0, st, a);
+    const dim3 grid(rows, rows <= 64 ? (a.heads + 2 * a.kv_heads + 3) / 4 : 1);       // few rows: latency
+    if (cols <= 256) hipLaunchKernelGGL((attn_heads_kernel<T, 1>), grid, dim3(256), 0, st, a);
+    else if (cols <= 512) hipLaunchKernelGGL((attn_heads_kernel<T, 2>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((attn_heads_kernel<T, 8>), grid, dim3(256), 0, st, a);
 }
 
 }  // namespace

@@ -259,7 +259,7 @@ struct Step {
             COGS_TRY(lin(g));
         }
         CogsDelta a{k.t32, G.ldt, m.heads, G.headsp, m.kv_heads, G.dk, G.dv, m.vdim, m.taps, G.channels, m.conv, m.neg_a, m.dt_bias, m.norm, d.w.eps,
-                    1.f / sqrtf((float)m.dim), k.dq, k.dk, k.dv, k.dbg, k.dout, k.drec, k.att, G.oin, k.seqs, k.rowseq, k.rowpos, run.state_off};
+                    1.f / sqrtf((float)m.dim), S, k.dq, k.dk, k.dv, k.dbg, k.dout, k.drec, k.att, G.oin, k.seqs, k.rowseq, k.rowpos, run.state_off};
         {
             PROF(COGS_PROF_ATTN);
             if (token_step(S, nseq)) COGS_TRY(cogs_k_delta_step(st, d.w.dtype, a, nseq));

@@ -43,8 +43,84 @@ __device__ __forceinline__ float conv_silu(const CogsDelta& p, const float* x, c
     return y / (1.f + expf(-y));
 }
 
-// one workgroup per new row; a wave per q / k head
+// quick silu: the activation behind a short convolution
+__device__ __forceinline__ float silu_q(float y) { return y * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-1.4426950408889634f * y)); }
+
+// RUN consecutive rows of a sequence at a time: a wave walks one q / k head, or 64 E channels of v, or the heads' beta and ln g, with
+// the convolution's window in registers and the whole run's inputs requested ahead. E: 64-channel steps of a head; TAPS: taps, rounded up
+template <int E, int TAPS, int RUN>
 __global__ __launch_bounds__(256) void delta_inputs_kernel(CogsDelta p) {
+    const CogsSeq s = p.seqs[blockIdx.z];
+    const int lane = threadIdx.x & 63, wid = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+    const int i0 = blockIdx.x * RUN, n = min(RUN, s.len - i0);
+    if (n <= 0) return;
+    const int nqk = 2 * p.kv_heads, nv = p.heads * p.dvp, units = nqk + (nv + 64 * E - 1) / (64 * E);
+    const int unit = blockIdx.y * 4 + wid, v0 = nqk * p.dkp;
+    const long row0 = s.row0 + i0;
+    const float* x = p.t + row0 * p.ldt;
+    if (unit > units) return;
+    if (unit == units) {
+        const float *tb = x + v0 + 2 * nv, *ta = tb + p.headsp;
+        for (int i = lane; i < n * p.heads; i += 64) {
+            const int r = i / p.heads, h = i - r * p.heads;
+            p.bg[(row0 * p.heads + i) * 2] = sigmoid_f(tb[(long)r * p.ldt + h]);
+            p.bg[(row0 * p.heads + i) * 2 + 1] = p.neg_a[h] * softplus_f(ta[(long)r * p.ldt + h] + p.dt_bias[h]);
+        }
+        return;
+    }
+    const bool is_v = unit >= nqk;
+    const int c0 = is_v ? v0 + (unit - nqk) * 64 * E : unit * p.dkp, size = is_v ? min(64 * E, v0 + nv - c0) : p.dkp;
+    const float* ring = s.state + p.state_off + (long)p.heads * p.dkp * p.dvp;
+    float w[TAPS][E], in[TAPS - 1 + RUN][E];          // in[TAPS - 1 + r]: row i0 + r
+    int ch[E];
+#pragma unroll
+    for (int e = 0; e < E; ++e) ch[e] = c0 + min(lane + 64 * e, size - 1);
+#pragma unroll
+    for (int r = 0; r < RUN; ++r)
+#pragma unroll
+        for (int e = 0; e < E; ++e) in[TAPS - 1 + r][e] = x[(long)min(r, n - 1) * p.ldt + ch[e]];
+#pragma unroll
+    for (int j = 1; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+            const int i = i0 - j, pos = s.pos0 + i;
+            float v = 0.f;
+            if (j < p.taps && pos >= 0) v = i >= 0 ? x[ch[e] - (long)j * p.ldt] : ring[(long)(pos % p.taps) * p.channels + ch[e]];
+            in[TAPS - 1 - j][e] = v;
+        }
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j)
+#pragma unroll
+        for (int e = 0; e < E; ++e) w[j][e] = j < p.taps ? p.conv[(long)(p.taps - 1 - j) * p.channels + ch[e]] : 0.f;
+    float* out[E];                                    // (v's pieces may cross heads)
+#pragma unroll
+    for (int e = 0; e < E; ++e) {
+        const int c = ch[e] - v0, hv = c / p.dvp;
+        out[e] = is_v ? p.v + ((long)hv * p.rows + row0) * p.dvp + (c - hv * p.dvp)
+                      : (unit < p.kv_heads ? p.q : p.k) + ((long)(unit % p.kv_heads) * p.rows + row0) * p.dkp + (ch[e] - c0);
+    }
+    const long ld = is_v ? p.dvp : p.dkp;
+    const float scale = unit < p.kv_heads ? p.q_scale : 1.f;
+#pragma unroll
+    for (int r = 0; r < RUN; ++r) {
+        float y[E], ss = 0.f;
+#pragma unroll
+        for (int e = 0; e < E; ++e) {
+            float a = w[0][e] * in[TAPS - 1 + r][e];
+#pragma unroll
+            for (int j = 1; j < TAPS; ++j) a = fmaf(w[j][e], in[TAPS - 1 + r - j][e], a);
+            y[e] = lane + 64 * e < size ? silu_q(a) : 0.f;
+            ss = fmaf(y[e], y[e], ss);
+        }
+        const float f = is_v ? 1.f : unit_scale(wave_sum(ss)) * scale;
+#pragma unroll
+        for (int e = 0; e < E; ++e)
+            if (r < n && lane + 64 * e < size) out[e][r * ld] = y[e] * f;
+    }
+}
+
+// the same for any size: one workgroup per new row; a wave per q / k head
+__global__ __launch_bounds__(256) void delta_inputs_any_kernel(CogsDelta p) {
     const int row = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int sq = p.rowseq[row], pos = p.rowpos[row];
     const CogsSeq s = p.seqs[sq];
@@ -61,7 +137,7 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(CogsDelta p) {
         }
         float f = unit_scale(wave_sum(ss));
         if (j < p.kv_heads) f *= p.q_scale;
-        float* o = (j < p.kv_heads ? p.q : p.k) + ((long)row * p.kv_heads + j % p.kv_heads) * p.dkp;
+        float* o = (j < p.kv_heads ? p.q : p.k) + ((long)(j % p.kv_heads) * p.rows + row) * p.dkp;
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const int d = lane + 64 * e;
@@ -69,7 +145,7 @@ __global__ __launch_bounds__(256) void delta_inputs_kernel(CogsDelta p) {
         }
     }
     const int v0 = 2 * p.kv_heads * p.dkp, nv = p.heads * p.dvp;
-    for (int i = tid; i < nv; i += 256) p.v[(long)row * nv + i] = conv_silu(p, x, ring, v0 + i, pos, back);
+    for (int i = tid; i < nv; i += 256) p.v[((long)(i / p.dvp) * p.rows + row) * p.dvp + i % p.dvp] = conv_silu(p, x, ring, v0 + i, pos, back);
     const float *tb = x + v0 + 2 * nv, *ta = tb + p.headsp;
     for (int h = tid; h < p.heads; h += 256) {
         p.bg[((long)row * p.heads + h) * 2] = sigmoid_f(tb[h]);
@@ -98,19 +174,19 @@ __global__ __launch_bounds__(64) void delta_recur_kernel(CogsDelta p) {
     for (int i = 0; i < s.len; ++i) {
         const long row = s.row0 + i;
         const bool fresh = s.pos0 + i == 0;
-        const float *q = p.q + (row * p.kv_heads + kh) * p.dkp, *k = p.k + (row * p.kv_heads + kh) * p.dkp;
+        const float *q = p.q + ((long)kh * p.rows + row) * p.dkp, *k = p.k + ((long)kh * p.rows + row) * p.dkp;
         const float beta = p.bg[(row * p.heads + h) * 2], g = expf(p.bg[(row * p.heads + h) * 2 + 1]);
         float a = 0.f;
         if (!fresh)
             for (int d = 0; d < p.dkp; ++d) a = fmaf(S[(long)d * p.dvp] * g, k[d], a);
-        const float u = beta * (p.v[(row * p.heads + h) * p.dvp + col] - a);
+        const float u = beta * (p.v[((long)h * p.rows + row) * p.dvp + col] - a);
         float o = 0.f;
         for (int d = 0; d < p.dkp; ++d) {
             const float v = fmaf(k[d], u, fresh ? 0.f : S[(long)d * p.dvp] * g);
             S[(long)d * p.dvp] = v;
             o = fmaf(v, q[d], o);
         }
-        p.o[(row * p.heads + h) * p.dvp + col] = o;
+        p.o[((long)h * p.rows + row) * p.dvp + col] = o;
     }
 }
 
@@ -140,7 +216,7 @@ __global__ __launch_bounds__(192) void delta_chunk_kernel(CogsDelta p) {
     const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
     const long row0 = s.row0 + chunk * CH;
     const int kh = h / (p.heads / p.kv_heads);
-    const long ld = (long)p.kv_heads * p.dkp;
+    const long k0 = ((long)kh * p.rows + row0) * p.dkp + 4 * g;
     const int ta = wid > 0 ? 1 : 0, tb = wid == 2 ? 1 : 0;
     if (tid < CH) {
         const int r = min(tid, n - 1);
@@ -153,9 +229,9 @@ __global__ __launch_bounds__(192) void delta_chunk_kernel(CogsDelta p) {
         for (int i = 1; i < CH; ++i) cum[i] += cum[i - 1];
     f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
     const long ra = min(16 * ta + li, n - 1), rb = min(16 * tb + li, n - 1);
-    const float* ka = p.k + (row0 + ra) * ld + (long)kh * p.dkp + 4 * g;
-    const float* qa = p.q + (row0 + ra) * ld + (long)kh * p.dkp + 4 * g;
-    const float* kb = p.k + (row0 + rb) * ld + (long)kh * p.dkp + 4 * g;
+    const float* ka = p.k + k0 + ra * p.dkp;
+    const float* qa = p.q + k0 + ra * p.dkp;
+    const float* kb = p.k + k0 + rb * p.dkp;
     for (int d = 0; d < p.dkp; d += 16) {
         const f32x4 a = *reinterpret_cast<const f32x4*>(ka + d), b = *reinterpret_cast<const f32x4*>(kb + d), q = *reinterpret_cast<const f32x4*>(qa + d);
         kk = mfma4(a, b, kk);
@@ -210,100 +286,212 @@ __global__ __launch_bounds__(192) void delta_chunk_kernel(CogsDelta p) {
     }
 }
 
-// NK: 16-row tiles of S per wave
+// what a wave needs of one chunk; loaded one chunk ahead
 template <int NK>
-__global__ __launch_bounds__(256) void delta_scan_kernel(CogsDelta p) {
+struct ScanIn {
+    f32x4 tm[3], pm[2], eg[2], ec[2], v[2], k[2][NK], q[2][NK], kt[2][NK];
+    float gl;
+};
+
+// NK: 16-row tiles of S per wave. A chunk: S^T k from the state (partial sums of the waves meet in LDS: one barrier), then, while they
+// do, S^T q; U; the new state beside P U. The read-outs' partial sums ride on the next chunk's barrier, and waves 0 and 1 finish and
+// store 16 rows of them each behind it (waves 2 and 3 form copies of P U that nobody reads: they would wait otherwise). One wave per
+// SIMD issues in order, so the next chunk's loads are spread between the matrix instructions, and no product is one long chain.
+template <int NK>
+__global__ __launch_bounds__(256, 1) void delta_scan_kernel(CogsDelta p) {
     __shared__ __attribute__((aligned(16))) f32x4 red[2][4][4][64];
-    const int h = blockIdx.y, col0 = blockIdx.x * 16, seq = blockIdx.z;
+    // workgroups go round the XCDs: the columns of a head stay on one, whose L2 then serves its K and Q once
+    const int ng = p.dvp >> 4, place = blockIdx.x >> 3, h = (blockIdx.x & 7) + 8 * (place / ng), col0 = (place % ng) * 16, seq = blockIdx.z;
+    if (h >= p.heads) return;
     const CogsSeq s = p.seqs[seq];
     const int tid = threadIdx.x, lane = tid & 63, li = lane & 15, g = lane >> 4;
-    const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int wid = __builtin_amdgcn_readfirstlane(tid >> 6), half = wid & 1;
     const int kh = h / (p.heads / p.kv_heads);
-    const long ld = (long)p.kv_heads * p.dkp, ldv = (long)p.heads * p.dvp;
-    const float* K = p.k + s.row0 * ld + (long)kh * p.dkp;
-    const float* Q = p.q + s.row0 * ld + (long)kh * p.dkp;
-    const float* V = p.v + s.row0 * ldv + (long)h * p.dvp + col0 + li;
-    float* O = p.o + s.row0 * ldv + (long)h * p.dvp + col0 + li;
+    const int ld = p.dkp, ldv = p.dvp;
+    const float* K = p.k + ((long)kh * p.rows + s.row0) * ld;
+    const float* Q = p.q + ((long)kh * p.rows + s.row0) * ld;
+    const float* V = p.v + ((long)h * p.rows + s.row0) * ldv + col0;
+    float* O = p.o + ((long)h * p.rows + s.row0) * ldv + col0;
     float* S = s.state + p.state_off + (long)h * p.dkp * p.dvp + col0 + li;
     const int tiles = p.dkp >> 4;
     f32x4 st[NK];
+    int tn[NK];                                  // tiles past the end repeat the last one, and their S is kept at zero
+    float live[NK];
 #pragma unroll
     for (int n = 0; n < NK; ++n) {
         st[n] = f32x4{0.f, 0.f, 0.f, 0.f};
         const int t = wid + 4 * n;
+        tn[n] = 16 * min(t, tiles - 1);
+        live[n] = t < tiles ? 1.f : 0.f;
         if (t < tiles && s.pos0 > 0)
 #pragma unroll
             for (int r = 0; r < 4; ++r) st[n][r] = S[(long)(16 * t + 4 * g + r) * p.dvp];
     }
     const int nc = (s.len + CH - 1) / CH;
-    for (int c = 0; c < nc; ++c) {
-        const int r0 = c * CH, last = s.len - 1;
-        const float* rec = chunk_rec(p, s, seq, c, h);
-        f32x4 tm[3], pm[3], eg[2], ec[2];
+    // a lane's places in a chunk's rows (bytes); a ragged last chunk repeats its last row
+    unsigned ko[2], to[2][4], vo[2][4], oo[4];
 #pragma unroll
-        for (int i = 0; i < 3; ++i) {
-            tm[i] = frag(rec + i * TILE, 16, li, g);
-            pm[i] = frag(rec + (3 + i) * TILE, 16, li, g);
-        }
+    for (int r = 0; r < 4; ++r) oo[r] = ((16 * half + 4 * g + r) * ldv + li) * 4;
+    const unsigned ro = (li * 16 + 4 * g) * 4, ego = 16 * g;
+    auto places = [&](int valid) {
 #pragma unroll
         for (int a = 0; a < 2; ++a) {
-            eg[a] = *reinterpret_cast<const f32x4*>(rec + 6 * TILE + 16 * a + 4 * g);
-            ec[a] = *reinterpret_cast<const f32x4*>(rec + 6 * TILE + CH + 16 * a + 4 * g);
-        }
-        const float gl = rec[6 * TILE + 2 * CH];
-        f32x4 v[2], x[2], y[2];
+            ko[a] = (min(16 * a + li, valid - 1) * ld + 4 * g) * 4;
 #pragma unroll
-        for (int a = 0; a < 2; ++a) {
-            x[a] = y[a] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-            for (int r = 0; r < 4; ++r) v[a][r] = V[(long)min(r0 + 16 * a + 4 * g + r, last) * ldv];
-#pragma unroll
-            for (int n = 0; n < NK; ++n) {
-                const int t = wid + 4 * n;
-                if (t >= tiles) continue;
-                const long off = (long)min(r0 + 16 * a + li, last) * ld + 16 * t + 4 * g;
-                x[a] = mfma4(*reinterpret_cast<const f32x4*>(K + off), st[n], x[a]);
-                y[a] = mfma4(*reinterpret_cast<const f32x4*>(Q + off), st[n], y[a]);
+            for (int r = 0; r < 4; ++r) {
+                const int row = min(16 * a + 4 * g + r, valid - 1);
+                to[a][r] = (row * ld + li) * 4;
+                vo[a][r] = (row * ldv + li) * 4;
             }
         }
+    };
+    places(CH);
+    auto at4 = [](const float* base, unsigned bytes) { return *reinterpret_cast<const f32x4*>(reinterpret_cast<const char*>(base) + bytes); };
+    auto at1 = [](const float* base, unsigned bytes) { return *reinterpret_cast<const float*>(reinterpret_cast<const char*>(base) + bytes); };
+    // load i of a chunk: the 12 NK + 18 of them in the order of their use
+    struct From { const float *k, *q, *v, *rec; };
+    From f{K, Q, V, chunk_rec(p, s, seq, 0, h)};
+    const long step_k = (long)CH * ld, step_v = (long)CH * ldv, step_rec = (long)p.heads * REC;
+    int at = 0;                                                // the chunk f points to
+    auto advance = [&] {                                       // (the last chunk is loaded again rather than nothing)
+        if (at + 1 >= nc) return;
+        ++at;
+        f.k += step_k; f.q += step_k; f.v += step_v; f.rec += step_rec;
+        if ((at + 1) * CH > s.len) places(s.len - at * CH);
+    };
+    constexpr int L_K = 2 * NK, L_V = L_K + 8, L_TM = L_V + 3, L_EG = L_TM + 2, L_Q = L_EG + 2 * NK, L_EC = L_Q + 2, L_KT = L_EC + 8 * NK, L_ALL = L_KT + 3;
+    auto load = [&](ScanIn<NK>& in, int i) {
+        if (i < L_K) in.k[i & 1][i >> 1] = at4(f.k + tn[i >> 1], ko[i & 1]);
+        else if (i < L_V) in.v[(i - L_K) >> 2][(i - L_K) & 3] = at1(f.v, vo[(i - L_K) >> 2][(i - L_K) & 3]);
+        else if (i < L_TM) in.tm[i - L_V] = at4(f.rec + (i - L_V) * TILE, ro);
+        else if (i < L_EG) in.eg[i - L_TM] = at4(f.rec + 6 * TILE + 16 * (i - L_TM), ego);
+        else if (i < L_Q) in.q[(i - L_EG) & 1][(i - L_EG) >> 1] = at4(f.q + tn[(i - L_EG) >> 1], ko[(i - L_EG) & 1]);
+        else if (i < L_EC) in.ec[i - L_Q] = at4(f.rec + 6 * TILE + CH + 16 * (i - L_Q), ego);
+        else if (i < L_KT) in.kt[((i - L_EC) >> 2) & 1][(i - L_EC) >> 3][(i - L_EC) & 3] = at1(f.k + tn[(i - L_EC) >> 3], to[((i - L_EC) >> 2) & 1][(i - L_EC) & 3]);
+        else if (i < L_ALL - 1) in.pm[i - L_KT] = at4(f.rec + (3 + half + (i - L_KT)) * TILE, ro);      // half 0: P(0,0) and one without use; 1: P(1,0), P(1,1)
+        else if (i < L_ALL) in.gl = f.rec[6 * TILE + 2 * CH];
+    };
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    const float second = half ? 1.f : 0.f;                     // rows 0 .. 15 have no P(0,1)
+    f32x4 y[2] = {zero, zero}, po = zero, peg = zero;          // the previous chunk's: partial S^T q, P U and e^G of this wave's rows
+    auto sum4 = [&](f32x4 (*rd)[4][64], int a) { return (rd[0][a][lane] + rd[1][a][lane]) + (rd[2][a][lane] + rd[3][a][lane]); };
+    auto store = [&](int c, const f32x4& o, bool ragged) {
+        float* oc = O + (long)c * CH * ldv;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+            if (!ragged || c * CH + 16 * half + 4 * g + r < s.len) *reinterpret_cast<float*>(reinterpret_cast<char*>(oc) + oo[r]) = o[r];
+    };
+    auto meet = [&] {                                          // (loads of the next chunk stay in flight)
+        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+        __builtin_amdgcn_s_barrier();
+        asm volatile("" ::: "memory");
+    };
+    auto mfma = [](float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); };
+    // chunk c from `in`, the next one into nx
+    auto chunk = [&](int c, const ScanIn<NK>& in, ScanIn<NK>& nx) {
+        advance();
+        constexpr int STEPS = 8 * NK + 8 * NK / 2 + 6;         // pairs of matrix instructions
+        int step = 0, done = 0;
+        auto feed = [&] {                                      // this pair's share of the loads
+            ++step;
+#pragma unroll
+            for (int i = 0; i < L_ALL; ++i)
+                if (i >= done && i < (L_ALL * step + STEPS - 1) / STEPS) load(nx, i);
+            done = (L_ALL * step + STEPS - 1) / STEPS;
+            __builtin_amdgcn_sched_barrier(0);
+        };
+        f32x4 x[2][2] = {{zero, zero}, {zero, zero}};          // [16 rows][half of the depth]
+#pragma unroll
+        for (int n = 0; n < NK; ++n)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+#pragma unroll
+                for (int a = 0; a < 2; ++a) x[a][r & 1] = mfma(in.k[a][n][r], st[n][r], x[a][r & 1]);
+                feed();
+            }
         f32x4 (*rd)[4][64] = red[c & 1];
 #pragma unroll
         for (int a = 0; a < 2; ++a) {
-            rd[wid][a][lane] = x[a];
             rd[wid][2 + a][lane] = y[a];
+            rd[wid][a][lane] = x[a][0] + x[a][1];
         }
-        __syncthreads();
-        f32x4 rr[2], u[2];
+        meet();
+        f32x4 part[3][4];
 #pragma unroll
-        for (int a = 0; a < 2; ++a) rr[a] = v[a] - eg[a] * ((rd[0][a][lane] + rd[1][a][lane]) + (rd[2][a][lane] + rd[3][a][lane]));
-        const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-        u[0] = mfma4(tm[0], rr[0], zero);
-        u[1] = mfma4(tm[2], rr[1], mfma4(tm[1], rr[0], zero));
-        if (wid < 2) {
-            f32x4 o = eg[wid] * ((rd[0][2 + wid][lane] + rd[1][2 + wid][lane]) + (rd[2][2 + wid][lane] + rd[3][2 + wid][lane]));
-            if (wid == 0) o = mfma4(pm[0], u[0], o);
-            else o = mfma4(pm[2], u[1], mfma4(pm[1], u[0], o));
+        for (int a = 0; a < 3; ++a)
+#pragma unroll
+            for (int w = 0; w < 4; ++w) part[a][w] = rd[w][a < 2 ? a : 2 + half][lane];
+        __builtin_amdgcn_sched_barrier(0);
+        y[0] = y[1] = zero;
+        f32x4 y2[2] = {zero, zero};
+#pragma unroll
+        for (int n = 0; n < NK; ++n)
 #pragma unroll
             for (int r = 0; r < 4; ++r) {
-                const int i = r0 + 16 * wid + 4 * g + r;
-                if (i <= last) O[(long)i * ldv] = o[r];
+#pragma unroll
+                for (int a = 0; a < 2; ++a) {
+                    f32x4& t = (r & 1) ? y2[a] : y[a];
+                    t = mfma(in.q[a][n][r], st[n][r], t);
+                }
+                feed();
             }
+        f32x4 rr[2], u[2] = {zero, zero}, u1 = zero;
+#pragma unroll
+        for (int a = 0; a < 2; ++a) {
+            rr[a] = in.v[a] - in.eg[a] * ((part[a][0] + part[a][1]) + (part[a][2] + part[a][3]));
+            y[a] += y2[a];
         }
 #pragma unroll
-        for (int a = 0; a < 2; ++a) u[a] *= ec[a];
+        for (int r = 0; r < 4; ++r) {                          // three chains
+            u[0] = mfma(in.tm[0][r], rr[0][r], u[0]);
+            u[1] = mfma(in.tm[1][r], rr[0][r], u[1]);
+            if (r & 1) feed();
+            u1 = mfma(in.tm[2][r], rr[1][r], u1);
+            feed();
+        }
+        u[1] += u1;
+        const f32x4 o = po + peg * ((part[2][0] + part[2][1]) + (part[2][2] + part[2][3]));
+        f32x4 ue[2], pa = zero, pb = zero, s2[NK];
+        const f32x4 up = u[1] * second;
+#pragma unroll
+        for (int a = 0; a < 2; ++a) ue[a] = u[a] * in.ec[a];
 #pragma unroll
         for (int n = 0; n < NK; ++n) {
-            const int t = wid + 4 * n;
-            if (t >= tiles) continue;
-            st[n] *= gl;
-#pragma unroll
-            for (int a = 0; a < 2; ++a) {
-                f32x4 kt;
-#pragma unroll
-                for (int r = 0; r < 4; ++r) kt[r] = K[(long)min(r0 + 16 * a + 4 * g + r, last) * ld + 16 * t + li];
-                st[n] = mfma4(kt, u[a], st[n]);
-            }
+            st[n] *= in.gl;
+            s2[n] = zero;
         }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+#pragma unroll
+            for (int n = 0; n < NK; ++n) {
+                st[n] = mfma(in.kt[0][n][r], ue[0][r], st[n]);
+                s2[n] = mfma(in.kt[1][n][r], ue[1][r], s2[n]);
+                feed();
+            }
+            pa = mfma(in.pm[0][r], u[0][r], pa);
+            pb = mfma(in.pm[1][r], up[r], pb);
+        }
+#pragma unroll
+        for (int n = 0; n < NK; ++n) st[n] = (st[n] + s2[n]) * live[n];
+        po = pa + pb;
+        peg = half ? in.eg[1] : in.eg[0];
+        if (c > 0 && wid < 2) store(c - 1, o, false);
+    };
+    ScanIn<NK> in0, in1;
+    if (s.len < CH) places(s.len);
+#pragma unroll
+    for (int i = 0; i < L_ALL; ++i) load(in0, i);
+    for (int c = 0; c < nc; c += 2) {
+        chunk(c, in0, in1);
+        if (c + 1 >= nc) break;
+        chunk(c + 1, in1, in0);
+    }
+    {
+        f32x4 (*rd)[4][64] = red[nc & 1];
+#pragma unroll
+        for (int a = 0; a < 2; ++a) rd[wid][2 + a][lane] = y[a];
+        meet();
+        if (wid < 2) store(nc - 1, po + peg * sum4(rd, 2 + half), true);
     }
 #pragma unroll
     for (int n = 0; n < NK; ++n) {
@@ -321,7 +509,7 @@ __global__ __launch_bounds__(256) void delta_out_kernel(CogsDelta p) {
     const long nv = (long)p.heads * p.dvp;
     const float* gate = p.t + (long)row * p.ldt + 2L * p.kv_heads * p.dkp + nv;
     for (int h = wid; h < p.heads; h += 4) {
-        const float* o = p.o + row * nv + (long)h * p.dvp;
+        const float* o = p.o + ((long)h * p.rows + row) * p.dvp;
         float ss = 0.f;
         for (int d = lane * 4; d < p.dvp; d += 256) {
             const f32x4 v = *reinterpret_cast<const f32x4*>(o + d);
@@ -456,6 +644,15 @@ int launch_step(hipStream_t st, const CogsDelta& p, int nseq) {
     return COGS_LAUNCH_CHECK();
 }
 
+void launch_inputs(hipStream_t st, const CogsDelta& a, int rows, int nseq, int max_new) {
+    const int nv = a.heads * a.dvp;
+    const auto grid = [&](int e, int run) { return dim3((max_new + run - 1) / run, (2 * a.kv_heads + (nv + 64 * e - 1) / (64 * e) + 1 + 3) / 4, nseq); };
+    if (a.taps <= 4 && a.dkp <= 64) hipLaunchKernelGGL((delta_inputs_kernel<1, 4, 16>), grid(1, 16), dim3(256), 0, st, a);
+    else if (a.taps <= 4 && a.dkp <= 128) hipLaunchKernelGGL((delta_inputs_kernel<2, 4, 16>), grid(2, 16), dim3(256), 0, st, a);
+    else if (a.taps <= 8 && a.dkp <= 256) hipLaunchKernelGGL((delta_inputs_kernel<4, 8, 8>), grid(4, 8), dim3(256), 0, st, a);
+    else hipLaunchKernelGGL(delta_inputs_any_kernel, dim3(rows), dim3(256), 0, st, a);
+}
+
 bool sizes_ok(const CogsDelta& a) {
     return a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0 && a.taps > 0 && a.dkp % 16 == 0 && a.dvp % 16 == 0 && a.dkp <= 512 &&
            a.dvp <= 2048 && a.vdim > 0 && a.vdim <= a.dvp && a.channels == 2 * a.kv_heads * a.dkp + a.heads * a.dvp && a.ldt % 4 == 0 && a.ldo % 4 == 0;
@@ -467,12 +664,12 @@ size_t cogs_k_delta_rec_floats(int rows, int nseq, int heads) { return (size_t)(
 
 int cogs_k_delta_prompt(hipStream_t st, int dtype, const CogsDelta& a, int rows, int nseq, int max_new) {
     if (!sizes_ok(a) || rows <= 0 || nseq <= 0 || nseq > 65535 || a.heads > 65535) return COGS_E_INVALID;
-    hipLaunchKernelGGL(delta_inputs_kernel, dim3(rows), dim3(256), 0, st, a);
+    launch_inputs(st, a, rows, nseq, max_new);
     const int keep = (max_new < a.taps ? max_new : a.taps) * a.channels;
     hipLaunchKernelGGL(delta_tail_kernel, dim3((keep + 1023) / 1024, nseq), dim3(256), 0, st, a);
     if (a.dkp <= 256 && g_cogs_debug.delta_chunk != 0) {
         hipLaunchKernelGGL(delta_chunk_kernel, dim3((max_new + CH - 1) / CH, a.heads, nseq), dim3(192), 0, st, a);
-        const dim3 grid(a.dvp / 16, a.heads, nseq);
+        const dim3 grid((a.heads + 7) / 8 * 8 * (a.dvp / 16), 1, nseq);
         if (a.dkp <= 64) hipLaunchKernelGGL(delta_scan_kernel<1>, grid, dim3(256), 0, st, a);
         else if (a.dkp <= 128) hipLaunchKernelGGL(delta_scan_kernel<2>, grid, dim3(256), 0, st, a);
         else hipLaunchKernelGGL(delta_scan_kernel<4>, grid, dim3(256), 0, st, a);

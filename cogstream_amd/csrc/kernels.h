@@ -254,7 +254,8 @@ struct CogsDelta {
     const float* t; long ldt;            // fused projection [q | k | v | gate | beta | a]
     int heads, headsp, kv_heads, dkp, dvp, vdim, taps, channels;
     const float *conv, *neg_a, *dt_bias, *norm; float eps, q_scale;
-    float *q, *k, *v, *bg, *o, *rec;     // prompts: [rows][kv_heads][dkp] twice, [rows][heads][dvp], (beta, ln g), read-outs, chunk records
+    int rows;                            // prompts: q, k [kv_heads][rows][dkp], v [heads][rows][dvp], (beta, ln g) [rows][heads], read-outs like v, chunk records
+    float *q, *k, *v, *bg, *o, *rec;
     void* att; long ldo;                 // [rows][heads x dvp], in `dtype`
     const CogsSeq* seqs; const int* rowseq; const int* rowpos; long state_off;      // floats
 };
