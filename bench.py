@@ -452,8 +452,8 @@ def pabalix_config(width, heads, q_rank, kv_rank, ff, layers):
 
 
 # (name, width, heads, ff, Qwen2's ff, layers): heads of 128, a quarter of them as key/value heads in attention, half as q/k heads in delta
-# layers; every fourth layer is attention. Qwen2's gated feed-forward has the same number of weights (three matrices against two)
-LUPANEX_SIZES = [("w2048", 2048, 16, 8448, 5632, 8), ("w3584", 3584, 28, 28416, 18944, 4), ("w4096", 4096, 32, 16512, 11008, 8)]
+# layers; every fourth layer is attention. Qwen2's gated feed-forward has about as many weights (three matrices against two)
+LUPANEX_SIZES = [("w2048", 2048, 16, 8192, 5632, 8), ("w3584", 3584, 28, 28416, 18944, 4), ("w4096", 4096, 32, 16384, 11008, 8)]
 LUPANEX_VOCAB = 32768
 
 

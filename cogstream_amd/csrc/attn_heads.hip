@@ -1,4 +1,4 @@
-// Head rows of softmax attention with per-head keys and values (cogs_attn_mixer) behind the fused projection: optional RMS norm of
+// Head rows of softmax attention with per-head keys and values (cogs_attn_mixer) behind the fused projection (fp32): optional RMS norm of
 // every query and key head row (no weight), the query's temperature, the score scale in log2 units, and the cache rows, padding
 // included (a tile's rows past the end repeat a row's last columns under a weight of zero). The attention itself is mla.hip's.
 #include "common.h"
@@ -14,12 +14,12 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
     const CogsSeq s = p.seqs[p.rowseq[row]];
     float qs = p.scale * 1.4426950408889634f;
     if (p.temp_every > 0.0) qs *= 1.f + (float)p.temp_coef * logf((float)(floor((pos + 1) / p.temp_every) + 1.0));
-    const T* t = reinterpret_cast<const T*>(p.t) + (long)row * p.ldt;
+    const float* t = p.t + (long)row * p.ldt;
     const int total = p.heads + 2 * p.kv_heads;
     for (int j = blockIdx.y * 4 + wid; j < total; j += 4 * gridDim.y) {
         const bool is_q = j < p.heads, is_k = !is_q && j < p.heads + p.kv_heads;
         const int kh = is_q ? 0 : (j - p.heads) % p.kv_heads, cols = is_q || is_k ? p.dkp : p.dvp, out_cols = is_q || is_k ? p.dkp : p.kvw - p.dkp;
-        const T* x = t + (is_q || is_k ? (long)j * p.dkp : (long)(p.heads + p.kv_heads) * p.dkp + (long)kh * p.dvp);
+        const float* x = t + (is_q || is_k ? (long)j * p.dkp : (long)(p.heads + p.kv_heads) * p.dkp + (long)kh * p.dvp);
         T* y = is_q ? reinterpret_cast<T*>(p.q) + (long)row * p.heads * p.dkp + (long)j * p.dkp
                     : reinterpret_cast<T*>(s.cache) + (p.layer_off + (long)kh * p.kvw) * s.max_len + (long)pos * p.kvw + (is_k ? 0 : p.dkp);
         f32x4 v[E];
@@ -28,7 +28,7 @@ __global__ __launch_bounds__(256) void attn_heads_kernel(CogsAttnHeads p) {
         for (int e = 0; e < E; ++e) {
             const int d = 4 * lane + 256 * e;
             v[e] = f32x4{0.f, 0.f, 0.f, 0.f};
-            if (d < cols) v[e] = ld4_f<T>(x + d);
+            if (d < cols) v[e] = *reinterpret_cast<const f32x4*>(x + d);
 #pragma unroll
             for (int i = 0; i < 4; ++i) ss += v[e][i] * v[e][i];
         }

@@ -43,7 +43,7 @@ struct CogsDecoder {
     long rope_width = 0, cache_width = 0;     // floats per row of all rotation tables; elements per token of a cache
     long state_floats = 0;                    // fp32 recurrent state of a sequence
     // largest row widths over the layers
-    int max_t32 = 0, max_t = 0, max_cq = 0, max_q = 0, max_o = 0, max_ff = 0, max_kvcols = 0, max_kvw = 0, max_heads = 0;
+    int max_t32 = 0, max_cq = 0, max_q = 0, max_o = 0, max_ff = 0, max_kvcols = 0, max_kvw = 0, max_heads = 0;
     long max_qlat = 0, max_olat = 0;
     int max_dqk = 0, max_dv = 0, max_dheads = 0;       // gated delta rule: kv_heads x dim, heads x vdim, heads
     bool att_tail = false;
@@ -59,7 +59,7 @@ void cogs_decoder_free(CogsDecoder* d) {
 namespace {
 
 struct Work {
-    float* x; void *h, *y, *t, *cq, *q, *att, *act, *hn, *ctx, *kvx, *qlat, *olat;
+    float* x; void *h, *y, *cq, *q, *att, *act, *hn, *ctx, *kvx, *qlat, *olat;
     float *t32, *gate, *rope, *part, *dq, *dk, *dv, *dbg, *dout, *drec;
     CogsSeq* seqs; int *rowseq, *rowpos, *want;
     size_t bytes;
@@ -77,7 +77,6 @@ Work carve(const CogsDecoder& d, int S, int nseq, int64_t C, int n_want, void* w
     k.h = c.take(n * d.wp * es);
     k.y = c.take(n * d.wp * es);
     k.t32 = (float*)c.take(n * d.max_t32 * 4);
-    k.t = c.take(n * d.max_t * es);
     k.cq = c.take(n * d.max_cq * es);
     k.q = c.take(n * d.max_q * es);
     k.att = c.take(n * d.max_o * es);
@@ -225,11 +224,11 @@ struct Step {
         const int dt = d.w.dtype, rep = m.heads / m.kv_heads;
         {
             CogsGemm g;
-            g.A = k.h; g.lda = d.wp; g.W = m.in_w; g.ldw = d.wp; g.C = k.t; g.ldc = G.ldt; g.M = S; g.N = G.ldt; g.K = d.wp;
+            g.A = k.h; g.lda = d.wp; g.W = m.in_w; g.ldw = d.wp; g.C = k.t32; g.ldc = G.ldt; g.M = S; g.N = G.ldt; g.K = d.wp; g.out_f32 = 1;
             COGS_TRY(lin(g));
         }
         {
-            CogsAttnHeads a{k.t, G.ldt, m.heads, m.kv_heads, m.dim, G.dk, G.dv, G.kvw, m.qk_norm, d.w.eps, m.scale, m.temp_coef, m.temp_every,
+            CogsAttnHeads a{k.t32, G.ldt, m.heads, m.kv_heads, m.dim, G.dk, G.dv, G.kvw, m.qk_norm, d.w.eps, m.scale, m.temp_coef, m.temp_every,
                             k.q, k.seqs, k.rowseq, k.rowpos, run.cache_off};
             PROF(COGS_PROF_NORM);
             COGS_TRY(cogs_k_attn_heads(st, dt, a, S));
@@ -377,7 +376,7 @@ cogs_status cogs_decoder_load(cogs_handle h, const cogs_decoder_weights* w) {
             g.dk = up(m.dim, 32); g.dv = up(m.vdim, 16); g.kvw = up(g.dk + g.dv, 32); g.oin = up(m.heads * g.dv, 64);
             g.ldt = (m.heads + m.kv_heads) * g.dk + m.kv_heads * g.dv;
             G.rows_width = m.kv_heads * g.kvw;
-            mx(d->max_t, g.ldt); mx(d->max_q, m.heads * g.dk);
+            mx(d->max_t32, g.ldt); mx(d->max_q, m.heads * g.dk);
             oin = g.oin; ocols = m.heads * g.dv;
         } else if (L.mixer == COGS_MIX_DELTA) {
             const cogs_delta_mixer& m = L.delta;

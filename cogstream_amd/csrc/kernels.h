@@ -242,7 +242,7 @@ int cogs_k_mla_decode(hipStream_t st, const CogsMlaDecode& a);
 // softmax attention with per-head keys and values: head rows behind the fused projection (attn_heads.hip), attention by CogsMla /
 // CogsMlaDecode with kvw
 struct CogsAttnHeads {
-    const void* t; long ldt;             // [rows][q heads x dkp | k heads x dkp | v heads x dvp] in `dtype`
+    const float* t; long ldt;            // [rows][q heads x dkp | k heads x dkp | v heads x dvp]
     int heads, kv_heads, dim, dkp, dvp, kvw, norm; float eps, scale; double temp_coef, temp_every;
     void* q;                             // [rows][heads][dkp], in log2 score units
     const CogsSeq* seqs; const int* rowseq; const int* rowpos; long layer_off;

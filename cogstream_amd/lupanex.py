@@ -18,7 +18,7 @@ from .weights import DecoderConfig, DecoderLayerConfig, DeltaRule, DistanceBias,
 def parse_config(c: dict, shapes: Dict[str, Tuple[int, ...]]) -> DecoderConfig:
     """config.json, with the shapes of the checkpoint's tensors (the number of distance buckets is a shape only) -> DecoderConfig"""
     cfg = DecoderConfig(width=int(c["width"]), vocab_size=int(c["vocab"]), eps=float(c["norm"]["eps"]),
-                        embed_scale=float(c["embedding"]["scale"]), max_positions=int(c["max_positions"]), streams=int(c["streams"]))
+                        embed_scale=float(c["embedding"]["scale"]), max_positions=int(c["max_positions"]), streams=int(c.get("streams") or 0))
     loop = c.get("loop")
     if loop is not None:
         cfg.loop = Loop(int(loop["start"]), int(loop["stop"]), int(loop["times"]))

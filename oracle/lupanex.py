@@ -123,6 +123,8 @@ MIXERS = {"attention": attention, "delta": delta}
 
 
 def read(xs: List[torch.Tensor], w, pre: str) -> torch.Tensor:
+    if pre + "in" not in w:                # one plain residual stream
+        return xs[0]
     u = torch.zeros_like(xs[0])
     for s, x in enumerate(xs):
         u = u + w[pre + "in"][s] * x
@@ -130,6 +132,8 @@ def read(xs: List[torch.Tensor], w, pre: str) -> torch.Tensor:
 
 
 def write(xs: List[torch.Tensor], y: torch.Tensor, w, pre: str) -> List[torch.Tensor]:
+    if pre + "in" not in w:
+        return [xs[0] + y]
     out = []
     for t in range(len(xs)):
         z = w[pre + "out"][t] * y
@@ -153,7 +157,7 @@ def forward(cfg: dict, w: Dict[str, torch.Tensor], tokens: List[int]) -> Tuple[t
     eps = cfg["norm"]["eps"]
     T = len(tokens)
     x = w["embed"][torch.as_tensor(tokens, dtype=torch.long)] * cfg["embedding"]["scale"] + w["pos"][:T]
-    xs, states = [x] * cfg["streams"], []
+    xs, states = [x] * cfg.get("streams", 1), []
     for i in order(cfg):
         lay, p = cfg["layers"][i], f"l{i}."
         h = rms(read(xs, w, p + "hc1."), eps) * w[p + "norm1"]

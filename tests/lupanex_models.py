@@ -27,6 +27,8 @@ def config(layers, width=136, vocab=211, ff=104, eps=1e-5, streams=3, loop=None,
         out.append(lay)
     cfg = dict(architecture="Lupanex", layers=out, norm=dict(eps=eps), vocab=vocab, width=width, streams=streams,
                embedding=dict(scale=scale), max_positions=positions)
+    if streams is None:                # a plain residual
+        del cfg["streams"]
     if loop is not None:
         cfg["loop"] = dict(zip(("start", "stop", "times"), loop))
     return cfg
@@ -52,6 +54,7 @@ CONFIGS = {
     # the whole model in a loop, every size alike, a loop of one pass
     "same": config([delta(heads=4, kv_heads=4, dim=32, vdim=32, conv=4), attention(heads=4, dim=32, vdim=32, rows=32, far=64)], width=64, vocab=128, ff=64,
                    streams=4, loop=(0, 2, 2)),
+    "plain": config([delta(heads=2, kv_heads=1), attention(heads=2, kv_heads=1)], width=72, vocab=90, streams=None),
     "once": config([attention(heads=2), delta(heads=2, kv_heads=1)], width=64, vocab=96, streams=5, loop=(1, 2, 1)),
     "wide": config([delta(heads=8, kv_heads=4, dim=128, vdim=128, conv=4), attention(heads=20, kv_heads=1, dim=128, vdim=128, rows=32, far=64),
                     attention(heads=12, kv_heads=4, dim=64, vdim=64, rows=8, far=1000)], width=512, vocab=400, ff=320, streams=4),

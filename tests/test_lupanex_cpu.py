@@ -45,7 +45,7 @@ def test_a_distance_bias_without_logarithmic_buckets_is_refused():
 def test_configuration():
     for name, cfg in CONFIGS.items():
         dc = parse(public(cfg) | {"layers": cfg["layers"]})
-        assert dc.runs() == lo.order(cfg) and dc.streams == cfg["streams"] and dc.max_positions == cfg["max_positions"], name
+        assert dc.runs() == lo.order(cfg) and dc.streams == cfg.get("streams", 0) and dc.max_positions == cfg["max_positions"], name
         for lay, mine in zip(cfg["layers"], dc.layers):
             m = lay["mixer"]
             assert (mine.mixer.heads, mine.mixer.kv_heads, mine.mixer.dim, mine.mixer.vdim) == (m["heads"], m["kv_heads"], m["dim"], m["vdim"])
@@ -117,9 +117,9 @@ def test_packed_layouts_give_the_same_projections(name):
         o[:, :H * dv].view(5, H, dv)[..., :v] = val
         y = o @ _view(x.o_w, (Wp, o.shape[1]), pk).T
         assert torch.allclose(y[:, :W], val.reshape(5, -1) @ st[pre + "o"].T, atol=1e-4) and not y[:, W:].any()
-        s = cfg["streams"]
+        s = cfg.get("streams", 0)
         for q, hc in (("1", pk.layers[i].hyper1), ("2", pk.layers[i].hyper2)):
-            if q == "2" and lay["mlp"] is None:
+            if not s or q == "2" and lay["mlp"] is None:
                 continue
             assert torch.equal(_view(hc.in_, (s,), pk), st[f"l{i}.hc{q}.in"]) and torch.equal(_view(hc.out, (s,), pk), st[f"l{i}.hc{q}.out"])
             assert torch.equal(_view(hc.mix, (s, s), pk), st[f"l{i}.hc{q}.mix"])
