@@ -222,20 +222,35 @@ __global__ __launch_bounds__(192) void delta_chunk_kernel(CogsDelta p) {
         const int r = min(tid, n - 1);
         const float* bg = p.bg + ((row0 + r) * p.heads + h) * 2;
         beta_s[tid] = bg[0];
-        cum[tid] = tid < n ? (double)bg[1] : 0.0;
+        double sum = tid < n ? (double)bg[1] : 0.0;
+#pragma unroll
+        for (int o = 1; o < CH; o *= 2) {
+            const double before = __shfl_up(sum, o, CH);
+            if (tid >= o) sum += before;
+        }
+        cum[tid] = sum;
     }
-    __syncthreads();
-    if (tid == 0)
-        for (int i = 1; i < CH; ++i) cum[i] += cum[i - 1];
     f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
     const long ra = min(16 * ta + li, n - 1), rb = min(16 * tb + li, n - 1);
     const float* ka = p.k + k0 + ra * p.dkp;
     const float* qa = p.q + k0 + ra * p.dkp;
     const float* kb = p.k + k0 + rb * p.dkp;
-    for (int d = 0; d < p.dkp; d += 16) {
-        const f32x4 a = *reinterpret_cast<const f32x4*>(ka + d), b = *reinterpret_cast<const f32x4*>(kb + d), q = *reinterpret_cast<const f32x4*>(qa + d);
-        kk = mfma4(a, b, kk);
-        qk = mfma4(q, b, qk);
+    for (int d = 0; d < p.dkp; d += 64) {              // four 16-wide steps in flight; steps past the end are not multiplied
+        f32x4 a[4], b[4], q[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const int o = min(d + 16 * e, p.dkp - 16);
+            a[e] = *reinterpret_cast<const f32x4*>(ka + o);
+            b[e] = *reinterpret_cast<const f32x4*>(kb + o);
+            q[e] = *reinterpret_cast<const f32x4*>(qa + o);
+        }
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            if (d + 16 * e >= p.dkp) break;
+            kk = mfma4(a[e], b[e], kk);
+            qk = mfma4(q[e], b[e], qk);
+        }
     }
     __syncthreads();
     float* rec = chunk_rec(p, s, seq, chunk, h);

@@ -126,7 +126,7 @@ def alone(mech):
         st = state(cfg)
         st["l0.mix.q"][:20] *= 0
         st["l0.mix.k"][:20] *= 1e-4
-    elif mech in ("conv1", "conv2", "conv7"):
+    elif mech in ("conv1", "conv2", "conv7", "conv12"):
         cfg = config([delta(heads=2, conv=int(mech[4:]), ff=None)], width=64)
     elif mech == "hyper":                  # the sublayers do nothing: the streams only mix
         cfg = config([delta(heads=2, kv_heads=1), attention(heads=2)], width=64, streams=6, loop=(0, 2, 2))
@@ -152,7 +152,7 @@ def alone(mech):
 
 
 @pytest.mark.parametrize("mech", ["bias", "temperature", "temperature_fraction", "qk_norm", "groups", "delta", "delta_fast", "delta_hard", "delta_zero", "conv1", "conv2",
-                                  "conv7", "hyper", "hyper1", "loop", "feed_forward", "positions"])
+                                  "conv7", "conv12", "hyper", "hyper1", "loop", "feed_forward", "positions"])
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_mechanism_alone(dev, mech, dtype):
     cfg, st = alone(mech)
